@@ -19,6 +19,7 @@ import torch
 
 from ..cache.manager import CacheManager
 from ..kernels.api import AttnRows
+from ..kernels.hip import capture
 from ..model import Model
 from .batch import PagedView, Step, StepRow
 
@@ -270,7 +271,7 @@ class StepRunner:
         if g.graph is None:
             torch.cuda.synchronize(self.device)
             graph = torch.cuda.CUDAGraph()
-            with torch.cuda.graph(graph):
+            with capture(graph):
                 g.logits = self._forward(g.step, None)
             g.graph = graph
         g.graph.replay()

@@ -4,8 +4,10 @@ library for them (std/holon_std/ops/units.py:229); everything else is this packa
 a missing library is built, and if that fails, loading raises."""
 from __future__ import annotations
 
+import contextlib
 import copy
 import ctypes
+import gc
 import sys
 import weakref
 
@@ -22,6 +24,21 @@ _DT = {torch.float32: 0, torch.bfloat16: 1}
 
 class KernelError(RuntimeError):
     pass
+
+
+@contextlib.contextmanager
+def capture(graph: "torch.cuda.CUDAGraph"):
+    """Record into `graph`, with Python's garbage collector off while the recording lasts: a collection inside it may
+    destroy another graph, an event or pinned memory that only a dead reference cycle (an engine let go of) still held,
+    and those destructors make calls that a recording does not allow, which ends the process."""
+    on = gc.isenabled()
+    gc.disable()
+    try:
+        with torch.cuda.graph(graph):
+            yield
+    finally:
+        if on:
+            gc.enable()
 
 
 def _ptr(t: torch.Tensor | None) -> int | None:
@@ -329,7 +346,7 @@ class HipKernels:
                 call()
             torch.cuda.synchronize()
             graph = torch.cuda.CUDAGraph()
-            with torch.cuda.graph(graph):
+            with capture(graph):
                 keep = [call() for call in calls]
             graph.replay()
             start, end = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)

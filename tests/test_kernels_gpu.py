@@ -998,3 +998,27 @@ def test_kernels_refuse_what_they_do_not_serve(hip):
         hip.linear_add(_randn(4, 1024, dtype=bf), w, hip.tile_weight(other), _randn(4, 512, dtype=bf))
     with pytest.raises(KernelError):
         hip.linear_add(_randn(4, 1024, dtype=bf), w, tiled, torch.zeros(4, 512, dtype=bf))   # residual on the CPU
+
+
+def test_nothing_is_collected_while_a_graph_is_recorded():
+    """Python's garbage collector is off inside a recording (what a collection destroys may make calls that a recording
+    does not allow) and on again behind it, also behind one that fails."""
+    import gc
+
+    from holon_amd.kernels.hip import capture
+    x = torch.ones(64, device="cuda")
+    y = x * 2
+    graph = torch.cuda.CUDAGraph()
+    assert gc.isenabled()
+    with capture(graph):
+        assert not gc.isenabled()
+        y = x * 2
+    assert gc.isenabled()
+    for i in range(3):
+        x.fill_(float(i))
+        graph.replay()
+        assert torch.equal(y, torch.full_like(y, 2.0 * i))
+    with pytest.raises(RuntimeError, match="stop here"):
+        with capture(torch.cuda.CUDAGraph()):
+            raise RuntimeError("stop here")
+    assert gc.isenabled()
