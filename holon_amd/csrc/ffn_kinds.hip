@@ -220,14 +220,16 @@ __global__ void __launch_bounds__(256) moe_gate_kernel(const T* __restrict__ gat
 }
 // The other router, one block of 256 threads a token: float32 logits z_e = x . router[e] + bias[e]; the `top` largest
 // are chosen (equal ones: the lower index first) and weighted by the softmax over the chosen logits alone, every other
-// expert 0. Rows of `router` beyond the experts are gates: their columns hold sigmoid(x . router[r]).
+// expert 0. `groups` > 1: only experts of the `keep` groups of neighbours whose largest logits are best can be chosen
+// (equal groups: the lower one). Rows of `router` beyond the experts are gates: their columns hold sigmoid(x . router[r]).
 // Every thread takes a slice of the token's row against all router rows, sixteen rows at a time (their loads do not
 // wait for each other); a wave's lanes are summed by shuffles and the four waves' partial sums in wave order. Up to 64
 // experts one wave then makes the choice with an expert a lane; more are ranked by the whole block.
 template <typename T>
 __global__ void __launch_bounds__(256) moe_router_top_kernel(const T* __restrict__ x, const float* __restrict__ router,
                                                              const float* __restrict__ bias, float* __restrict__ weights,
-                                                             int width, int experts, int rows_r, int top) {
+                                                             int width, int experts, int rows_r, int top, int groups,
+                                                             int keep) {
   __shared__ float part_s[4][ROUTE_MAX_E + 1];
   __shared__ float z_s[ROUTE_MAX_E + 1];
   __shared__ float e_s[ROUTE_MAX_E];
@@ -275,14 +277,28 @@ __global__ void __launch_bounds__(256) moe_router_top_kernel(const T* __restrict
   };
   if (experts <= WAVE) {                                  // an expert a lane
     if (wave != 0) return;
-    const float mine = lane < experts ? logit(lane) : -INFINITY;
+    float mine = lane < experts ? logit(lane) : -INFINITY;
+    if (groups > 1) {                                     // the group's largest logit, then how many groups are ahead
+      const int size = experts / groups, g = lane / size;
+      float best = -INFINITY;
+      for (int o = 0; o < experts; ++o) {
+        const float other = __shfl(mine, o, WAVE);
+        if (o / size == g) best = fmaxf(best, other);
+      }
+      int before = 0;
+      for (int o = 0; o < groups; ++o) {
+        const float other = __shfl(best, o * size, WAVE);
+        before += (other > best) || (other == best && o < g);
+      }
+      if (before >= keep) mine = -INFINITY;
+    }
     int ahead = 0;
     for (int o = 0; o < experts; ++o) {
       const float other = __shfl(mine, o, WAVE);
       ahead += (other > mine) || (other == mine && o < lane);
     }
     const float top_z = wave_max(mine);                   // the largest logit is always chosen
-    const float v = lane < experts && ahead < top ? expf(mine - top_z) : 0.f;
+    const float v = lane < experts && ahead < top && mine > -INFINITY ? expf(mine - top_z) : 0.f;
     const float sum = wave_sum(v);
     if (lane < experts) weights[t * rows_r + lane] = v / sum;
     if (rows_r > experts && lane == 0) weights[t * rows_r + experts] = 1.0f / (1.0f + expf(-logit(experts)));
@@ -290,6 +306,22 @@ __global__ void __launch_bounds__(256) moe_router_top_kernel(const T* __restrict
   }
   for (int e = threadIdx.x; e < rows_r; e += 256) z_s[e] = logit(e);
   __syncthreads();
+  if (groups > 1) {
+    const int size = experts / groups;
+    for (int g = threadIdx.x; g < groups; g += 256) {
+      float best = -INFINITY;
+      for (int i = 0; i < size; ++i) best = fmaxf(best, z_s[g * size + i]);
+      e_s[g] = best;
+    }
+    __syncthreads();
+    for (int e = threadIdx.x; e < experts; e += 256) {
+      const int g = e / size;
+      int before = 0;
+      for (int o = 0; o < groups; ++o) before += (e_s[o] > e_s[g]) || (e_s[o] == e_s[g] && o < g);
+      if (before >= keep) z_s[e] = -INFINITY;
+    }
+    __syncthreads();
+  }
   float top_z = -INFINITY;
   for (int e = threadIdx.x; e < experts; e += 256) top_z = fmaxf(top_z, z_s[e]);
   top_z = wave_max(top_z);
@@ -302,7 +334,7 @@ __global__ void __launch_bounds__(256) moe_router_top_kernel(const T* __restrict
     const float mine = z_s[e];
     int ahead = 0;
     for (int o = 0; o < experts; ++o) ahead += (z_s[o] > mine) || (z_s[o] == mine && o < e);
-    const float v = ahead < top ? expf(mine - top_z) : 0.f;
+    const float v = ahead < top && mine > -INFINITY ? expf(mine - top_z) : 0.f;
     e_s[e] = v;
     part += v;
   }
@@ -425,20 +457,23 @@ extern "C" int holon_moe_gate(const void* gate_up, const float* weights, void* y
 }
 
 extern "C" int holon_moe_router_top(const void* x, const float* router, const float* bias, float* weights, int64_t rows,
-                                    int width, int experts, int router_rows, int top, int dtype, void* stream) {
+                                    int width, int experts, int router_rows, int top, int dtype, int groups, int keep,
+                                    void* stream) {
   HOLON_CHECK(rows >= 0 && rows <= 0x7fffffffLL && width >= 1 && width <= 12288 && experts >= 1 &&
                   experts <= ROUTE_MAX_E && top >= 1 && top <= experts &&
                   (router_rows == experts || router_rows == experts + 1),
               "moe_router_top: rows=%lld of %d (at most 12,288), top %d of %d experts (at most %d), %d router rows",
               (long long)rows, width, top, experts, ROUTE_MAX_E, router_rows);
+  HOLON_CHECK(groups <= 1 || (experts % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (experts / groups)),
+              "moe_router_top: top %d of %d experts in %d groups of which %d stay open", top, experts, groups, keep);
   if (rows == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   if (dtype == HOLON_F32)
     moe_router_top_kernel<float><<<(unsigned)rows, 256, 0, s>>>((const float*)x, router, bias, weights, width, experts,
-                                                               router_rows, top);
+                                                               router_rows, top, groups, keep);
   else
     moe_router_top_kernel<bf16_t><<<(unsigned)rows, 256, 0, s>>>((const bf16_t*)x, router, bias, weights, width,
-                                                                experts, router_rows, top);
+                                                                experts, router_rows, top, groups, keep);
   HOLON_LAUNCH_OK();
   return 0;
 }

@@ -214,11 +214,13 @@ int holon_softcap(float* logits, int64_t n, float cap, void* stream);
 
 // -- recurrent mixers (recurrent.hip); rows are ranges query_start[b] .. query_start[b + 1] of the flat tokens ----------
 // y_t[c] = act(sum_j w[c, j] x_(t - taps + 1 + j)[c] (+ x_t[c])); state [state_slots, taps - 1, channels] holds each
-// request's last inputs (ignored by a row that starts at 0) and takes the row's last ones afterwards.
+// request's last inputs (ignored by a row that starts at 0) and takes the row's last ones afterwards (ring: [state_slots,
+// taps, channels], the input of position p at p % taps). Rows of x lie x_stride values apart; bias [channels] nullable.
 // rows_in_order: every row has one token and token t is row t (a decode step): one kernel then does both.
-int holon_causal_conv(const void* x, const void* w, void* state, void* y, const int32_t* slots, const int32_t* starts,
+int holon_causal_conv(const void* x, int64_t x_stride, const void* w, const void* bias, void* state, void* y,
+                      const int32_t* slots, const int32_t* starts,
                       const int32_t* query_start, const int32_t* token_row, int tokens, int rows, int channels, int taps,
-                      int state_slots, int add_input, int act, int dtype, int rows_in_order, void* stream);
+                      int state_slots, int add_input, int act, int dtype, int rows_in_order, int ring, void* stream);
 // From filtered q, k, v [T, 2 G D + H V] and the projections ab [T, 2 H]: unit q (times D^-0.5) and k [T, G, D],
 // beta = sigmoid(b), g = exp(-exp(a_log) softplus(a + dt_bias)) [T, H]; all outputs float32.
 int holon_delta_prepare(const void* qkv, const void* ab, const float* a_log, const float* dt_bias, float* qn, float* kn,
@@ -313,11 +315,17 @@ int holon_whole_norm_prepare(const void* qkv, int tokens, int heads, int kv_head
 // both [T, H (dim + rot) + kv_rank + rot]: the latent RMS-normed, the first rd of every rotated part's rot dimensions
 // turned by the position (table [table_rows, rd] float32: cosines, then sines); unrotated query parts to qn [T, H, dim],
 // rotated ones into the last rot columns of full [T, H, kv_rank + rot]; [latent, rotated key part] into the token's
-// page as a key row and as a value column.
-int holon_latent_rope_prepare(const void* both, int tokens, int heads, int dim, int rot, int kv_rank,
+// page as a key row and (copies 2) as a value column. Rows lie both_stride values apart; pages null: queries alone.
+int holon_latent_rope_prepare(const void* both, int both_stride, int tokens, int heads, int dim, int rot, int kv_rank,
                               const void* c_weight, float eps, const float* table, int rd, int table_rows,
                               const int32_t* positions, void* qn, void* full, void* pages, const int32_t* write_page,
-                              const int32_t* write_off, int page_size, int num_pages, int dtype, void* stream);
+                              const int32_t* write_off, int page_size, int num_pages, int copies, int dtype, void* stream);
+// Attention over latent entries kept once (latent_attention.hip): q [T, H, width]; pages of [P, width] entries that every
+// head reads as keys, and whose first kv_rank values as values; out [T, H, kv_rank].
+int holon_latent_attention(const void* q, void* out, const void* pages, const int32_t* table, int table_stride,
+                           int table_rows, const int32_t* slots, const int32_t* token_row, const int32_t* positions,
+                           int tokens, int heads, int width, int kv_rank, int page_size, int num_pages,
+                           const float* sink, float scale, int window, int dtype, void* stream);
 
 // The latent attention's two latents, side by side in `both` [T, q_rank + kv_rank]: each divided by its root mean square
 // and multiplied by its weight; the first to cq [T, q_rank], the second into the token's page as a key row and as a
@@ -326,9 +334,9 @@ int holon_latent_prepare(const void* both, int tokens, int q_rank, int kv_rank, 
                          const void* c_weight, float eps, void* cq, void* pages, const int32_t* write_page,
                          const int32_t* write_off, int page_size, int num_pages, int dtype, void* stream);
 // y [rows, H, B] = x [rows, H, A] times every head's own w [H, B, A], for steps of up to 16 rows; a head's results lie
-// y_head values apart (B, or more where y is part of wider rows).
+// y_head values apart (B, or more where y is part of wider rows). gate (nullable): y times sigmoid(gate[t, h B + b]).
 int holon_head_linear_rows(const void* x, const void* w, void* y, int rows, int heads, int A, int B, int y_head,
-                           int dtype, void* stream);
+                           int dtype, const void* gate, int64_t gate_stride, void* stream);
 
 // -- a block of two sublayers over one float32 stream (parallel_block.hip) ----------------------------------------------
 // x32 [rows, dim] += (d1 + d2) + row in place (each nullable; d1, d2 float32 or bfloat16 by dt1, dt2; row [dim] float32);
@@ -344,6 +352,9 @@ int holon_stream_rms_filter(float* x32, const void* d1, int dt1, const void* d2,
                             const void* w1, const void* w2, int dtw, void* y1, void* y2, int64_t rows, int dim,
                             float eps, int dt_out, const void* cw1, const void* cw2, void* held1, void* held2,
                             const int32_t* slots, const int32_t* starts, int taps, void* stream);
+// x32 [rows, dim] += gain term / sqrt(mean(term^2) + term_eps) in place; y = x / sqrt(mean(x^2) + eps) * w.
+int holon_stream_rms_post(float* x32, const void* term, int dtt, const float* gain, float term_eps, const void* w, int dtw,
+                          void* y, int64_t rows, int dim, float eps, int dt_out, void* stream);
 // y[i] = scale * x[i] as float32 (x float32 or bfloat16): a new copy.
 int holon_scale_rows(const void* x, float* y, int64_t n, int dtype, float scale, void* stream);
 
@@ -365,10 +376,10 @@ int holon_moe_router(const void* x, const float* router, const float* correction
 int holon_moe_gate(const void* gate_up, const float* weights, void* y, int64_t rows, int experts, int ff, int shared,
                    int dtype, int wstride, int shared_col, void* stream);
 // The other router: logits x . router[e] + bias[e] (nullable), the `top` largest chosen, weights the softmax over the
-// chosen logits alone; router rows beyond the experts (none or one) are gates: their columns hold a sigmoid.
-// weights [rows, router_rows].
+// chosen logits alone; router rows beyond the experts (none or one) are gates: their columns hold a sigmoid. groups > 1:
+// chosen among the `keep` groups of neighbours with the best largest logits. weights [rows, router_rows].
 int holon_moe_router_top(const void* x, const float* router, const float* bias, float* weights, int64_t rows, int width,
-                         int experts, int router_rows, int top, int dtype, void* stream);
+                         int experts, int router_rows, int top, int dtype, int groups, int keep, void* stream);
 // y = max(z, 0)^2 over n values.
 int holon_relu2(const void* z, void* y, int64_t n, int dtype, void* stream);
 
@@ -384,6 +395,27 @@ int holon_mlstm_scan(const void* proj, int width, int q_off, int k_off, int v_of
                      const int32_t* query_start, int rows, int heads, int dim, int vdim, int state_slots, int dtype,
                      int tokens, int piece_tokens, int max_pieces, const int32_t* piece_base, float* gates, float* sloc,
                      float* pk, void* stream);
+
+// -- Mamba-2's state-space dual form (mamba2.hip) ------------------------------------------------------------------------
+// A step of single tokens (row b is token b) from the raw projection [rows, width] = [z | x | B | C | dt | ...]: filter
+// (taps [C, taps], bias, the requests' inputs `held` [slots, taps, C] as a ring), step size softplus(dt + dt_bias),
+// S <- exp(-exp(a_log) dt) S + dt B x^T, y = S^T C + D x; state [slots, H, N, V] float32, y [rows, H V] float32.
+int holon_ssd_step(const void* proj, int width, const void* conv_w, const void* conv_b, void* held, const float* dt_bias,
+                   const float* a_log, const float* dvec, float* state, float* y, const int32_t* slots,
+                   const int32_t* starts, int rows, int heads, int groups, int n, int vdim, int taps, int state_slots,
+                   int dtype, void* stream);
+// The recurrence over each row's tokens from filtered xbc [T, H V + 2 G N] and dt (columns of rows dt_stride apart), rows
+// in pieces of 256 tokens (at most max_pieces a row; piece_base [rows]: the number of each row's first piece among all;
+// workspaces sums [3, H, T], sloc [pieces, H, N, V], decay [pieces, H]).
+int holon_ssd_scan(const void* xbc, const void* dt, int64_t dt_stride, const float* dt_bias, const float* a_log,
+                   const float* dvec, float* state, float* y, const int32_t* slots, const int32_t* starts,
+                   const int32_t* query_start, int rows, int tokens, int heads, int groups, int n, int vdim,
+                   int state_slots, int dtype, int max_pieces, const int32_t* piece_base, float* sums, float* sloc,
+                   float* decay, void* stream);
+// out = u / sqrt(mean(u^2) + eps) * weight over each of `parts` equal parts of a row, u = y silu(gate); gates are columns
+// of rows gate_stride apart.
+int holon_gated_parts_norm(const float* y, const void* gate, int64_t gate_stride, const void* weight, void* out, int tokens,
+                           int dim, int parts, float eps, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

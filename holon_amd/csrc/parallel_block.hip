@@ -2,6 +2,8 @@
 // layer before left to add (two terms, summed first) and a vector of the pass that begins, takes the row's mean square
 // once and writes the row normed with one weight or with two. Every sum over a row is taken in an order that the row's
 // width alone decides, so a token's result does not depend on what else is in the batch.
+#include <type_traits>
+
 #include "common.h"
 #include "holon_hip.h"
 
@@ -240,6 +242,96 @@ __global__ void __launch_bounds__(256) stream_rms_vec_kernel(float* __restrict__
   }
 }
 
+// A sublayer's result on its way into the stream: x += gain * term / sqrt(mean(term^2) + term_eps), then the row normed for
+// the next sublayer, y = x / sqrt(mean(x^2) + eps) * w. One block a row; a thread holds REGS groups of N neighbouring
+// values of both rows in registers (0: it reads back what it wrote). T: the term's and the result's type, W: the weight's.
+template <typename T, typename W, int N, int REGS>
+__global__ void __launch_bounds__(256) stream_rms_post_kernel(float* __restrict__ x32, const T* __restrict__ term,
+                                                              const float* __restrict__ gain, float term_eps,
+                                                              const W* __restrict__ w, T* __restrict__ y, int dim,
+                                                              float eps) {
+  __shared__ float part[4];
+  const int64_t base = (int64_t)blockIdx.x * dim;
+  float* x = x32 + base;
+  const T* tp = term + base;
+  constexpr int DT = sizeof(T) == 4 ? HOLON_F32 : HOLON_BF16, DW = sizeof(W) == 4 ? HOLON_F32 : HOLON_BF16;
+  auto take = [&](const auto* from, int i, float (&v)[N], auto dt) {
+    if constexpr (N == 4) load4t<decltype(dt)::value>(from, i, v);
+    else v[0] = load_as(from, i, decltype(dt)::value);
+  };
+  using TermT = std::integral_constant<int, DT>;
+  using WeightT = std::integral_constant<int, DW>;
+  using F32T = std::integral_constant<int, HOLON_F32>;
+  constexpr int R = REGS > 0 ? REGS : 1;
+  float tv[R][N], xv[R][N];
+  float sq = 0.f;
+  if constexpr (REGS > 0) {
+#pragma unroll
+    for (int e = 0; e < REGS; ++e) {
+      const int i = (threadIdx.x + e * 256) * N;
+#pragma unroll
+      for (int u = 0; u < N; ++u) tv[e][u] = xv[e][u] = 0.f;
+      if (i < dim) { take(tp, i, tv[e], TermT{}); take(x, i, xv[e], F32T{}); }
+    }
+#pragma unroll
+    for (int e = 0; e < REGS; ++e)
+#pragma unroll
+      for (int u = 0; u < N; ++u) sq += tv[e][u] * tv[e][u];
+  } else {
+    for (int i = threadIdx.x * N; i < dim; i += 256 * N) {
+      take(tp, i, tv[0], TermT{});
+#pragma unroll
+      for (int u = 0; u < N; ++u) sq += tv[0][u] * tv[0][u];
+    }
+  }
+  sq = block_sum_256(sq, part);
+  const float rt = 1.0f / sqrtf(sq / (float)dim + term_eps);
+  float sx = 0.f;
+  auto join = [&](int i, const float (&t)[N], float (&v)[N]) {
+    float g[N];
+    take(gain, i, g, F32T{});
+#pragma unroll
+    for (int u = 0; u < N; ++u) { v[u] += t[u] * rt * g[u]; sx += v[u] * v[u]; }
+    if constexpr (N == 4) store4t<HOLON_F32>(x, i, v);
+    else x[i] = v[0];
+  };
+  auto emit = [&](int i, const float (&v)[N], float r) {
+    float g[N], o[N];
+    take(w, i, g, WeightT{});
+#pragma unroll
+    for (int u = 0; u < N; ++u) o[u] = v[u] * r * g[u];
+    if constexpr (N == 4) store4t<DT>(y + base, i, o);
+    else store_as(y + base, i, DT, o[0]);
+  };
+  if constexpr (REGS > 0) {
+#pragma unroll
+    for (int e = 0; e < REGS; ++e) {
+      const int i = (threadIdx.x + e * 256) * N;
+      if (i < dim) join(i, tv[e], xv[e]);
+    }
+  } else {
+    for (int i = threadIdx.x * N; i < dim; i += 256 * N) {
+      take(tp, i, tv[0], TermT{});
+      take(x, i, xv[0], F32T{});
+      join(i, tv[0], xv[0]);
+    }
+  }
+  sx = block_sum_256(sx, part);
+  const float r = 1.0f / sqrtf(sx / (float)dim + eps);
+  if constexpr (REGS > 0) {
+#pragma unroll
+    for (int e = 0; e < REGS; ++e) {
+      const int i = (threadIdx.x + e * 256) * N;
+      if (i < dim) emit(i, xv[e], r);
+    }
+  } else {
+    for (int i = threadIdx.x * N; i < dim; i += 256 * N) {
+      take(x, i, xv[0], F32T{});
+      emit(i, xv[0], r);
+    }
+  }
+}
+
 __global__ void scale_rows_kernel(const void* __restrict__ x, float* __restrict__ y, int64_t n, int dt, float scale) {
   for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x)
     y[i] = load_as(x, i, dt) * scale;
@@ -314,6 +406,34 @@ extern "C" int holon_stream_rms_filter(float* x32, const void* d1, int dt1, cons
   else SRMSF_BY_TAPS(8);
 #undef SRMSF_BY_TAPS
 #undef SRMSF
+  HOLON_LAUNCH_OK();
+  return 0;
+}
+
+extern "C" int holon_stream_rms_post(float* x32, const void* term, int dtt, const float* gain, float term_eps,
+                                     const void* w, int dtw, void* y, int64_t rows, int dim, float eps, int dt_out,
+                                     void* stream) {
+  HOLON_CHECK(rows >= 0 && dim > 0 && rows <= 0x7fffffffLL, "stream_rms_post: rows=%lld dim=%d", (long long)rows, dim);
+  HOLON_CHECK(dtt == dt_out && (dtw == dtt || dtw == HOLON_F32),
+              "stream_rms_post: a term of the result's type, a weight of that type or float32");
+  if (rows == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+#define SRP(T, W, N, R)                                                                                             \
+  stream_rms_post_kernel<T, W, N, R><<<(unsigned)rows, 256, 0, s>>>(x32, (const T*)term, gain, term_eps, (const W*)w, \
+                                                                    (T*)y, dim, eps)
+#define SRP_BY_SIZE(T, W)                                                     \
+  do {                                                                        \
+    if (dim % 4 == 0 && dim <= 1024) SRP(T, W, 4, 1);                         \
+    else if (dim % 4 == 0 && dim <= 2048) SRP(T, W, 4, 2);                    \
+    else if (dim % 4 == 0 && dim <= 4096) SRP(T, W, 4, 4);                    \
+    else if (dim % 4 == 0 && dim <= 8192) SRP(T, W, 4, 8);                    \
+    else SRP(T, W, 1, 0);                                                     \
+  } while (0)
+  if (dtt == HOLON_F32) SRP_BY_SIZE(float, float);
+  else if (dtw == HOLON_F32) SRP_BY_SIZE(bf16_t, float);
+  else SRP_BY_SIZE(bf16_t, bf16_t);
+#undef SRP_BY_SIZE
+#undef SRP
   HOLON_LAUNCH_OK();
   return 0;
 }

@@ -13,48 +13,57 @@
 
 namespace {
 
+// The rows of x may be columns of wider rows (x_stride values apart); `bias` is nullable. ring: the slot holds `taps`
+// inputs, that of position p at place p % taps; else the last taps - 1, oldest first.
 template <typename T>
-__global__ void causal_conv_kernel(const T* __restrict__ x, const T* __restrict__ w, T* __restrict__ state,
+__global__ void causal_conv_kernel(const T* __restrict__ x, int64_t x_stride, const T* __restrict__ w,
+                                   const T* __restrict__ bias, T* __restrict__ state,
                                    T* __restrict__ y, const int32_t* __restrict__ slots,
                                    const int32_t* __restrict__ starts, const int32_t* __restrict__ query_start,
                                    const int32_t* __restrict__ token_row, int channels, int taps, int add_input,
-                                   int act, int keep) {
+                                   int act, int keep, int ring) {
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   const int t = blockIdx.y;
   if (c >= channels) return;
   const int b = keep ? t : token_row[t];               // keep: every row has one token, token t is row t
   const int q0 = keep ? t : query_start[b];
   const int i = t - q0;
-  const bool carried = starts[b] > 0;
-  T* held = state + (int64_t)slots[b] * (taps - 1) * channels;
+  const int start = starts[b];
+  const bool carried = start > 0;
+  T* held = state + (int64_t)slots[b] * (ring ? taps : taps - 1) * channels;
   float acc = 0.f;
   for (int j = 0; j < taps; ++j) {
     const int l = i - (taps - 1) + j;
     float v = 0.f;
-    if (l >= 0) v = Elem<T>::load(x[(int64_t)(q0 + l) * channels + c]);
-    else if (carried) v = Elem<T>::load(held[(int64_t)(taps - 1 + l) * channels + c]);
+    if (l >= 0) v = Elem<T>::load(x[(q0 + l) * x_stride + c]);
+    else if (carried && (!ring || start + l >= 0))
+      v = Elem<T>::load(held[(int64_t)(ring ? (start + l) % taps : taps - 1 + l) * channels + c]);
     acc += Elem<T>::load(w[(int64_t)c * taps + j]) * v;
   }
-  if (add_input) acc += Elem<T>::load(x[(int64_t)t * channels + c]);
+  if (bias) acc += Elem<T>::load(bias[c]);
+  if (add_input) acc += Elem<T>::load(x[t * x_stride + c]);
   if (act) acc = silu<T>(acc);
   y[(int64_t)t * channels + c] = Elem<T>::store(acc);
-  if (keep) {                  // the row's one token: this thread alone reads and writes its channel of the slot
+  if (keep && ring) {
+    held[(int64_t)(start % taps) * channels + c] = x[t * x_stride + c];
+  } else if (keep) {           // the row's one token: this thread alone reads and writes its channel of the slot
     for (int e = 0; e + 2 < taps; ++e)
       held[(int64_t)e * channels + c] = carried ? held[(int64_t)(e + 1) * channels + c] : Elem<T>::store(0.f);
-    if (taps > 1) held[(int64_t)(taps - 2) * channels + c] = x[(int64_t)t * channels + c];
+    if (taps > 1) held[(int64_t)(taps - 2) * channels + c] = x[t * x_stride + c];
   }
 }
 
 // The same for prompt portions with a thread taking 16 bytes of channels at a time (channels a multiple of that; rows
 // of x, y and the slots then start on 16-byte borders): the same products in the same order.
 template <typename T>
-__global__ void __launch_bounds__(256) causal_conv_wide_kernel(const T* __restrict__ x, const T* __restrict__ w,
+__global__ void __launch_bounds__(256) causal_conv_wide_kernel(const T* __restrict__ x, int64_t x_stride,
+                                                               const T* __restrict__ w, const T* __restrict__ bias,
                                                                const T* __restrict__ state, T* __restrict__ y,
                                                                const int32_t* __restrict__ slots,
                                                                const int32_t* __restrict__ starts,
                                                                const int32_t* __restrict__ query_start,
                                                                const int32_t* __restrict__ token_row, int channels,
-                                                               int taps, int add_input, int act) {
+                                                               int taps, int add_input, int act, int ring) {
   constexpr int N = Elem<T>::kVec;
   const int c = (blockIdx.x * blockDim.x + threadIdx.x) * N;
   const int t = blockIdx.y;
@@ -62,8 +71,9 @@ __global__ void __launch_bounds__(256) causal_conv_wide_kernel(const T* __restri
   const int b = token_row[t];
   const int q0 = query_start[b];
   const int i = t - q0;
-  const bool carried = starts[b] > 0;
-  const T* held = state + (int64_t)slots[b] * (taps - 1) * channels;
+  const int start = starts[b];
+  const bool carried = start > 0;
+  const T* held = state + (int64_t)slots[b] * (ring ? taps : taps - 1) * channels;
   float acc[N];
 #pragma unroll
   for (int u = 0; u < N; ++u) acc[u] = 0.f;
@@ -71,8 +81,9 @@ __global__ void __launch_bounds__(256) causal_conv_wide_kernel(const T* __restri
   for (int j = 0; j < taps; ++j) {
     const int l = i - (taps - 1) + j;
     uint4 raw = make_uint4(0u, 0u, 0u, 0u);
-    if (l >= 0) raw = *reinterpret_cast<const uint4*>(x + (int64_t)(q0 + l) * channels + c);
-    else if (carried) raw = *reinterpret_cast<const uint4*>(held + (int64_t)(taps - 1 + l) * channels + c);
+    if (l >= 0) raw = *reinterpret_cast<const uint4*>(x + (q0 + l) * x_stride + c);
+    else if (carried && (!ring || start + l >= 0))
+      raw = *reinterpret_cast<const uint4*>(held + (int64_t)(ring ? (start + l) % taps : taps - 1 + l) * channels + c);
     const T* v = reinterpret_cast<const T*>(&raw);
 #pragma unroll
     for (int u = 0; u < N; ++u) acc[u] += Elem<T>::load(w[(int64_t)(c + u) * taps + j]) * Elem<T>::load(v[u]);
@@ -84,6 +95,7 @@ __global__ void __launch_bounds__(256) causal_conv_wide_kernel(const T* __restri
 #pragma unroll
   for (int u = 0; u < N; ++u) {
     float a = acc[u];
+    if (bias) a += Elem<T>::load(bias[c + u]);
     if (add_input) a += Elem<T>::load(own[u]);
     if (act) a = silu<T>(a);
     o[u] = Elem<T>::store(a);
@@ -92,21 +104,28 @@ __global__ void __launch_bounds__(256) causal_conv_wide_kernel(const T* __restri
 }
 
 // After the filter has read the old inputs: the slot takes the row's last taps - 1 inputs, oldest first. A thread
-// moves its channel's entries in ascending order and reads only entries at or behind the one it writes.
+// moves its channel's entries in ascending order and reads only entries at or behind the one it writes. (A ring takes the
+// row's own last inputs at their places; older ones lie where they are.)
 template <typename T>
-__global__ void causal_conv_keep_kernel(const T* __restrict__ x, T* __restrict__ state, const int32_t* __restrict__ slots,
+__global__ void causal_conv_keep_kernel(const T* __restrict__ x, int64_t x_stride, T* __restrict__ state,
+                                        const int32_t* __restrict__ slots,
                                         const int32_t* __restrict__ starts, const int32_t* __restrict__ query_start,
-                                        int channels, int taps) {
+                                        int channels, int taps, int ring) {
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   const int b = blockIdx.y;
   if (c >= channels) return;
   const int q0 = query_start[b], n = query_start[b + 1] - q0;
   const bool carried = starts[b] > 0;
-  T* held = state + (int64_t)slots[b] * (taps - 1) * channels;
+  T* held = state + (int64_t)slots[b] * (ring ? taps : taps - 1) * channels;
+  if (ring) {
+    for (int l = max(0, n - taps); l < n; ++l)
+      held[(int64_t)((starts[b] + l) % taps) * channels + c] = x[(q0 + l) * x_stride + c];
+    return;
+  }
   for (int i = 0; i < taps - 1; ++i) {
     const int l = n - (taps - 1) + i;
     T v = Elem<T>::store(0.f);
-    if (l >= 0) v = x[(int64_t)(q0 + l) * channels + c];
+    if (l >= 0) v = x[(q0 + l) * x_stride + c];
     else if (carried) v = held[(int64_t)(i + n) * channels + c];
     held[(int64_t)i * channels + c] = v;
   }
@@ -627,34 +646,38 @@ __global__ void __launch_bounds__(256) decay_lora_kernel(const float* __restrict
     else { using T = bf16_t; CALL; }             \
   } while (0)
 
-extern "C" int holon_causal_conv(const void* x, const void* w, void* state, void* y, const int32_t* slots,
+extern "C" int holon_causal_conv(const void* x, int64_t x_stride, const void* w, const void* bias, void* state, void* y,
+                                 const int32_t* slots,
                                  const int32_t* starts, const int32_t* query_start, const int32_t* token_row,
                                  int tokens, int rows, int channels, int taps, int state_slots, int add_input, int act,
-                                 int dtype, int rows_in_order, void* stream) {
+                                 int dtype, int rows_in_order, int ring, void* stream) {
   HOLON_CHECK(tokens >= 0 && rows >= 0 && channels > 0 && taps >= 1 && taps <= 16 && state_slots > 0,
               "causal_conv: tokens=%d rows=%d channels=%d taps=%d", tokens, rows, channels, taps);
   HOLON_CHECK(tokens <= 65535 && rows <= 65535, "causal_conv: %d tokens in %d rows exceed one launch", tokens, rows);
+  HOLON_CHECK(x_stride >= channels, "causal_conv: rows of %d channels %lld apart", channels, (long long)x_stride);
   if (tokens == 0 || rows == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   const dim3 block(256), grid_t((channels + 255) / 256, tokens), grid_b((channels + 255) / 256, rows);
   HOLON_CHECK(!rows_in_order || tokens == rows, "causal_conv: rows in order means one token a row, got %d in %d", tokens,
               rows);
   const int vec = dtype == HOLON_F32 ? 4 : 8;
-  if (!rows_in_order && channels % vec == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0 &&
+  if (!rows_in_order && channels % vec == 0 && x_stride % vec == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0 &&
       (uintptr_t)state % 16 == 0) {
     const dim3 grid_w((channels / vec + 255) / 256, tokens);
-    BY_DTYPE(dtype, (causal_conv_wide_kernel<T><<<grid_w, block, 0, s>>>((const T*)x, (const T*)w, (const T*)state, (T*)y,
+    BY_DTYPE(dtype, (causal_conv_wide_kernel<T><<<grid_w, block, 0, s>>>((const T*)x, x_stride, (const T*)w,
+                                                                         (const T*)bias, (const T*)state, (T*)y,
                                                                          slots, starts, query_start, token_row,
-                                                                         channels, taps, add_input, act)));
+                                                                         channels, taps, add_input, act, ring)));
   } else {
-    BY_DTYPE(dtype, (causal_conv_kernel<T><<<grid_t, block, 0, s>>>((const T*)x, (const T*)w, (T*)state, (T*)y, slots,
-                                                                    starts, query_start, token_row, channels, taps,
-                                                                    add_input, act, rows_in_order)));
+    BY_DTYPE(dtype, (causal_conv_kernel<T><<<grid_t, block, 0, s>>>((const T*)x, x_stride, (const T*)w, (const T*)bias,
+                                                                    (T*)state, (T*)y, slots, starts, query_start,
+                                                                    token_row, channels, taps, add_input, act,
+                                                                    rows_in_order, ring)));
   }
   HOLON_LAUNCH_OK();
-  if (taps > 1 && !rows_in_order) {
-    BY_DTYPE(dtype, (causal_conv_keep_kernel<T><<<grid_b, block, 0, s>>>((const T*)x, (T*)state, slots, starts,
-                                                                         query_start, channels, taps)));
+  if ((taps > 1 || ring) && !rows_in_order) {
+    BY_DTYPE(dtype, (causal_conv_keep_kernel<T><<<grid_b, block, 0, s>>>((const T*)x, x_stride, (T*)state, slots, starts,
+                                                                         query_start, channels, taps, ring)));
     HOLON_LAUNCH_OK();
   }
   return 0;

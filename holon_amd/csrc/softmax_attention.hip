@@ -237,10 +237,12 @@ __global__ void __launch_bounds__(256) latent_prepare_kernel(const T* __restrict
 // y[t, h, b] = sum_a x[t, h, a] w[h, b, a] for steps of few rows: a block takes a head and 16 of its output columns,
 // the rows' values of that head wait in LDS, and sixteen lanes share a column (each a sixteenth of A, in the order of
 // the lane), added up in a fixed order. float32 sums, one rounding.
+// gate (nullable): the result is multiplied by sigmoid(gate[t, h B + b]), the gates columns of rows gate_stride apart.
 template <typename T>
 __global__ void __launch_bounds__(256) head_linear_kernel(const T* __restrict__ x, const T* __restrict__ w,
                                                           T* __restrict__ y, int rows, int heads, int A, int B,
-                                                          int y_head) {      // y_head: values between two heads of y
+                                                          int y_head,       // y_head: values between two heads of y
+                                                          const T* __restrict__ gate, int64_t gate_stride) {
   extern __shared__ float xs[];                          // [rows, A]
   const int h = blockIdx.x, b = blockIdx.y * 16 + threadIdx.x / 16, part = threadIdx.x % 16;
   for (int i = threadIdx.x; i < rows * A; i += 256) {
@@ -283,7 +285,10 @@ __global__ void __launch_bounds__(256) head_linear_kernel(const T* __restrict__ 
       v += __shfl_xor(v, 2, WAVE);
       v += __shfl_xor(v, 4, WAVE);
       v += __shfl_xor(v, 8, WAVE);
-      if (part == 0 && b < B && t0 + r < rows) y[((int64_t)(t0 + r) * heads + h) * y_head + b] = Elem<T>::store(v);
+      if (part == 0 && b < B && t0 + r < rows) {
+        if (gate) v *= 1.0f / (1.0f + expf(-Elem<T>::load(gate[(t0 + r) * gate_stride + (int64_t)h * B + b])));
+        y[((int64_t)(t0 + r) * heads + h) * y_head + b] = Elem<T>::store(v);
+      }
     }
   }
 }
@@ -309,7 +314,7 @@ extern "C" int holon_latent_prepare(const void* both, int tokens, int q_rank, in
 }
 
 extern "C" int holon_head_linear_rows(const void* x, const void* w, void* y, int rows, int heads, int A, int B,
-                                      int y_head, int dtype, void* stream) {
+                                      int y_head, int dtype, const void* gate, int64_t gate_stride, void* stream) {
   HOLON_CHECK(rows >= 1 && rows <= 16 && heads > 0 && heads <= 65535 && A > 0 && B > 0 && y_head >= B &&
                   (int64_t)rows * A * 4 <= 48 * 1024,
               "head_linear (few rows): %d rows, %d heads of %d -> %d (in steps of %d)", rows, heads, A, B, y_head);
@@ -317,9 +322,11 @@ extern "C" int holon_head_linear_rows(const void* x, const void* w, void* y, int
   const size_t lds = (size_t)rows * A * sizeof(float);
   hipStream_t s = (hipStream_t)stream;
   if (dtype == HOLON_F32)
-    head_linear_kernel<float><<<grid, 256, lds, s>>>((const float*)x, (const float*)w, (float*)y, rows, heads, A, B, y_head);
+    head_linear_kernel<float><<<grid, 256, lds, s>>>((const float*)x, (const float*)w, (float*)y, rows, heads, A, B, y_head,
+                                                    (const float*)gate, gate_stride);
   else
-    head_linear_kernel<bf16_t><<<grid, 256, lds, s>>>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, rows, heads, A, B, y_head);
+    head_linear_kernel<bf16_t><<<grid, 256, lds, s>>>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, rows, heads, A, B,
+                                                     y_head, (const bf16_t*)gate, gate_stride);
   HOLON_LAUNCH_OK();
   return 0;
 }
@@ -375,21 +382,24 @@ __global__ void __launch_bounds__(256) whole_norm_prepare_kernel(
 // dimensions of every rotated part turn by the token's position (pairs (i, i + rd / 2), `table` row = rd / 2 cosines,
 // then rd / 2 sines). Unrotated query parts go to `qn` [T, H, dim], rotated ones into the last `rot` columns of `full`
 // [T, H, kv_rank + rot]; the cache entry [latent, rotated key part] into the token's page as a key row of [P, width]
-// and as a value column of [width, P].
+// and (copies 2) as a value column of [width, P]. Rows are `both_stride` apart; `pages` null: queries alone.
 template <typename T>
 __global__ void __launch_bounds__(256) latent_rope_prepare_kernel(
-    const T* __restrict__ both, int heads, int dim, int rot, int kv_rank, const T* __restrict__ c_weight, float eps,
+    const T* __restrict__ both, int both_stride, int heads, int dim, int rot, int kv_rank, const T* __restrict__ c_weight,
+    float eps,
     const float* __restrict__ table, int rd, int table_rows, const int32_t* __restrict__ positions, T* __restrict__ qn,
     T* __restrict__ full, T* __restrict__ pages, const int32_t* __restrict__ write_page,
-    const int32_t* __restrict__ write_off, int page_size, int num_pages) {
+    const int32_t* __restrict__ write_off, int page_size, int num_pages, int copies) {
   __shared__ float part[2][4];
   const int t = blockIdx.x;
   const int per = dim + rot, width = kv_rank + rot, half = rd / 2;
-  const T* row = both + (int64_t)t * (heads * per + width);
+  const T* row = both + (int64_t)t * both_stride;
   const T* tail = row + heads * per;
   float sc = 0.f, unused = 0.f;
-  for (int d = threadIdx.x; d < kv_rank; d += 256) { const float v = Elem<T>::load(tail[d]); sc += v * v; }
-  block_sum2_256(sc, unused, part);
+  if (pages) {
+    for (int d = threadIdx.x; d < kv_rank; d += 256) { const float v = Elem<T>::load(tail[d]); sc += v * v; }
+    block_sum2_256(sc, unused, part);
+  }
   const float rc = 1.0f / sqrtf(sc / (float)kv_rank + eps);
   int pos = positions[t];
   pos = pos < 0 ? 0 : (pos >= table_rows && table_rows > 0 ? table_rows - 1 : pos);
@@ -409,15 +419,16 @@ __global__ void __launch_bounds__(256) latent_rope_prepare_kernel(
     const int h = c / rot, r = c - h * rot;
     full[((int64_t)t * heads + h) * width + kv_rank + r] = Elem<T>::store(turned(row + h * per + dim, r));
   }
+  if (!pages) return;
   const int page = write_page[t], off = write_off[t];
   if (page < 0 || page >= num_pages || off < 0 || off >= page_size) return;
-  T* keys = pages + (int64_t)page * 2 * page_size * width;
+  T* keys = pages + (int64_t)page * copies * page_size * width;
   T* vals = keys + (int64_t)page_size * width;
   for (int d = threadIdx.x; d < width; d += 256) {
     const T e = d < kv_rank ? Elem<T>::store(Elem<T>::load(tail[d]) * rc * Elem<T>::load(c_weight[d]))
                             : Elem<T>::store(turned(tail + kv_rank, d - kv_rank));
     keys[(int64_t)off * width + d] = e;
-    vals[(int64_t)d * page_size + off] = e;
+    if (copies == 2) vals[(int64_t)d * page_size + off] = e;
   }
 }
 // x[t, h, :] *= sigmoid(gates[t, h]): one wave a (token, head); the gates are columns of rows `gate_stride` apart.
@@ -488,11 +499,15 @@ extern "C" int holon_whole_norm_prepare(const void* qkv, int tokens, int heads, 
   return 0;
 }
 
-extern "C" int holon_latent_rope_prepare(const void* both, int tokens, int heads, int dim, int rot, int kv_rank,
+extern "C" int holon_latent_rope_prepare(const void* both, int both_stride, int tokens, int heads, int dim, int rot,
+                                         int kv_rank,
                                          const void* c_weight, float eps, const float* table, int rd, int table_rows,
                                          const int32_t* positions, void* qn, void* full, void* pages,
                                          const int32_t* write_page, const int32_t* write_off, int page_size,
-                                         int num_pages, int dtype, void* stream) {
+                                         int num_pages, int copies, int dtype, void* stream) {
+  HOLON_CHECK(both_stride >= heads * (dim + rot) + (pages ? kv_rank + rot : 0) && (copies == 1 || copies == 2) &&
+                  (pages == nullptr || (c_weight && write_page && write_off)),
+              "latent_rope_prepare: rows of %d values, entries kept %d times", both_stride, copies);
   HOLON_CHECK(tokens >= 0 && heads > 0 && dim > 0 && rot >= 0 && kv_rank > 0 && page_size > 0 && num_pages > 0,
               "latent_rope_prepare: %d heads of %d + %d, a latent of %d, pages of %d", heads, dim, rot, kv_rank, page_size);
   HOLON_CHECK(rd >= 0 && rd % 2 == 0 && rd <= rot && (rd == 0 || (table != nullptr && table_rows > 0)),
@@ -500,15 +515,15 @@ extern "C" int holon_latent_rope_prepare(const void* both, int tokens, int heads
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   if (dtype == HOLON_F32)
-    latent_rope_prepare_kernel<float><<<tokens, 256, 0, s>>>((const float*)both, heads, dim, rot, kv_rank,
+    latent_rope_prepare_kernel<float><<<tokens, 256, 0, s>>>((const float*)both, both_stride, heads, dim, rot, kv_rank,
                                                             (const float*)c_weight, eps, table, rd, table_rows, positions,
                                                             (float*)qn, (float*)full, (float*)pages, write_page,
-                                                            write_off, page_size, num_pages);
+                                                            write_off, page_size, num_pages, copies);
   else
-    latent_rope_prepare_kernel<bf16_t><<<tokens, 256, 0, s>>>((const bf16_t*)both, heads, dim, rot, kv_rank,
+    latent_rope_prepare_kernel<bf16_t><<<tokens, 256, 0, s>>>((const bf16_t*)both, both_stride, heads, dim, rot, kv_rank,
                                                              (const bf16_t*)c_weight, eps, table, rd, table_rows,
                                                              positions, (bf16_t*)qn, (bf16_t*)full, (bf16_t*)pages,
-                                                             write_page, write_off, page_size, num_pages);
+                                                             write_page, write_off, page_size, num_pages, copies);
   HOLON_LAUNCH_OK();
   return 0;
 }

@@ -15,11 +15,12 @@ from .stream32 import LayerNorm, Pending, PreNorm32
 from .dyt import DynamicTanh, Sandwich32, Scaled
 from .softmax_attention import LatentAttention, SoftmaxAttention
 from .mlstm import MLSTM
+from .mamba2 import Mamba2
 from .diff_attention import DiffAttention
 from .parallel_block import Parallel32, RMSNorm32
 
 __all__ = ["FLOAT32", "INT32", "MODEL", "Build", "EmbedPart", "NormPart", "PagedState", "ParamDecl", "Part", "PartialSums", "SlotState", "Stream", "PreNorm",
            "Embedding", "LMHead", "SwiGLU", "Linear", "GQA", "Normed", "RMSNorm", "NoPosition", "Rope", "rope_table", "BandedRope", "CausalConv", "DecayMemory", "GatedDelta",
            "SigmoidWindowAttention", "LayerNorm", "Pending", "PreNorm32", "ParallelMixers",
-           "DynamicTanh", "Sandwich32", "Scaled", "LatentAttention", "SoftmaxAttention", "MLSTM", "YarnRope",
+           "DynamicTanh", "Sandwich32", "Scaled", "LatentAttention", "SoftmaxAttention", "MLSTM", "Mamba2", "YarnRope",
            "MoE", "PolyNormFFN", "Parallel32", "RMSNorm32", "DiffAttention", "DenseFFN"]

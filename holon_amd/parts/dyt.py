@@ -7,10 +7,13 @@ norm is elementwise and any number of them fuse with the adds around them. Arith
 
     x += m post1(mixer(pre1(x)));   x += m post2(ffn(pre2(x)))
 
-with `m` a constant of the model (`residual_mult`). A layer may lack the feed-forward. A block with `reentry` adds the
+with `m` a constant of the model (`residual_mult`), and with `layer_scale` a learned vector per sublayer beside it (`ls1`,
+`ls2`, multiplied element by element behind the post norm). A layer may lack the feed-forward. The norms are Dynamic
+Tanhs or RMS norms over float32 rows (`parts/parallel_block.py`). A block with `reentry` adds the
 embedding's rows (`Stream.origin`) to x in front of every run of it but the first (a range of layers that runs several
 times, fed the embedding again at each pass). Every add and the norms on both sides of it are one kernel
-(`csrc/dyt.hip`): a sublayer's result travels as a `Scaled` term until the next norm reads the stream.
+(`csrc/dyt.hip`; for RMS norms `csrc/parallel_block.hip`): a sublayer's result travels as a `Scaled` term until the next
+norm reads the stream.
 """
 from __future__ import annotations
 
@@ -85,15 +88,17 @@ register_kernel(KernelOp("dyt_stream", dyt_stream_plain, "holon_dyt_stream",
 
 
 class Scaled:
-    """A sublayer's result that is not yet in the stream: what is to be added is scale * norm(term)."""
+    """A sublayer's result that is not yet in the stream: what is to be added is scale * norm(term). `gain` (float32
+    [W], from the norm's `output_gain`) stands for the norm's weight, the scale and any learned scale in one vector: what
+    is to be added is then gain times the norm of the term without its weight."""
 
-    def __init__(self, term: torch.Tensor, norm: "DynamicTanh", scale: float) -> None:
-        self.term, self.norm, self.scale = term, norm, scale
+    def __init__(self, term: torch.Tensor, norm: NormPart, scale: float, gain: torch.Tensor | None = None) -> None:
+        self.term, self.norm, self.scale, self.gain = term, norm, scale, gain
 
     def index_select(self, dim: int, index: torch.Tensor) -> "Scaled":
         if dim != 0:
             raise ValueError("Scaled.index_select: rows only (dim 0)")
-        return Scaled(self.term.index_select(0, index), self.norm, self.scale)
+        return Scaled(self.term.index_select(0, index), self.norm, self.scale, self.gain)
 
 
 @register_part("norm", "dyt")
@@ -135,15 +140,18 @@ class DynamicTanh(NormPart):
 class Sandwich32(Part):
     """x += m post1(mixer(pre1(x))); x += m post2(ffn(pre2(x))) over a float32 stream; see the module's text. The four
     norms are of the kind the layer names (`norm`), called `norm1`, `norm1b`, `norm2`, `norm2b`; that kind's `add`
-    must take `Scaled` terms (the Dynamic Tanh does)."""
+    must take `Scaled` terms (the Dynamic Tanh and `rms32` do). `layer_scale` asks for a norm that folds a vector behind
+    it into its weight (`output_gain`: `rms32`)."""
 
     graph_safe = True
     reads_origin = False
 
     def __init__(self, build: Build, *, layer: int, hidden: int, mixer: PartRef, ffn: PartRef | None, norm: PartRef,
-                 scale: float = 1.0, reentry: bool = False) -> None:
+                 scale: float = 1.0, reentry: bool = False, layer_scale: bool = False) -> None:
         super().__init__(build)
         self.hidden, self.scale = hidden, float(scale)
+        self.layer_scale = bool(layer_scale)
+        self.gain1 = self.gain2 = None
         self.attach("norm1", build.make(norm, dim=hidden))
         self.attach("mixer", build.make(mixer, layer=layer, hidden=hidden))
         self.attach("norm1b", build.make(norm, dim=hidden))
@@ -152,22 +160,38 @@ class Sandwich32(Part):
             self.attach("norm2", build.make(norm, dim=hidden))
             self.attach("ffn", build.make(ffn, layer=layer, hidden=hidden))
             self.attach("norm2b", build.make(norm, dim=hidden))
+        if self.layer_scale:
+            if not hasattr(self.norm1b, "output_gain"):
+                raise ValueError(f"sandwich32: a learned scale behind norm {norm.kind!r}, which does not fold one")
+            self.declare("ls1", (hidden,), kind=FLOAT32, init="norm")
+            if ffn is not None:
+                self.declare("ls2", (hidden,), kind=FLOAT32, init="norm")
         self.reentry = bool(reentry)
         self.reads_origin = self.reentry
+
+    def finalize(self) -> None:
+        """Where the norm says how, its weight, the scale and the learned scale become one float32 vector a sublayer."""
+        if hasattr(self.norm1b, "output_gain") and self.norm1b.weight is not None:
+            self.gain1 = self.norm1b.output_gain(self.scale, self.ls1 if self.layer_scale else None)
+            if self.ffn is not None:
+                self.gain2 = self.norm2b.output_gain(self.scale, self.ls2 if self.layer_scale else None)
+
+    def extra_tensors(self):
+        return [g for g in (self.gain1, self.gain2) if g is not None]
 
     def forward(self, stream: Stream, step, site) -> Stream:
         h = stream.h
         if h.dtype != torch.float32 or h is stream.origin:       # the stream becomes float32 rows of its own (the
-            h = stream.h = h.to(torch.float32, copy=True)        # embedding's rows stay as they are)
+            h = stream.h = self.kernels.widen_rows(h)            # embedding's rows stay as they are)
         again = stream.origin if self.reentry and site.turn > 0 else None
         a = self.norm1.add(stream.delta, h, extra=again)[0]
         stream.delta = stream.stats = None
-        mixed = Scaled(self.mixer(a, step, site), self.norm1b, self.scale)
+        mixed = Scaled(self.mixer(a, step, site), self.norm1b, self.scale, self.gain1)
         if self.ffn is None:
             stream.delta = mixed
             return stream
         x = self.norm2.add(mixed, h)[0]
-        stream.delta = Scaled(self.ffn(x, step), self.norm2b, self.scale)
+        stream.delta = Scaled(self.ffn(x, step), self.norm2b, self.scale, self.gain2)
         return stream
 
     __call__ = forward

@@ -168,29 +168,38 @@ def _moe_gate_hip(launch, gate_up, weights, ff, shared, shared_weight=False):
     return y
 
 
-def moe_router_top_plain(x, router, bias, experts, top):
+def moe_router_top_plain(x, router, bias, experts, top, groups=1, keep=1):
     """x [T, W] (any dtype), router [R, W] float32 with R = experts or experts + 1, bias [experts] float32 or None:
     the float32 logits z = x . router[e] + bias[e]; the `top` largest are chosen (equal ones: the lower index first)
-    and weighted by the softmax over the chosen logits alone, every other expert 0. A last row beyond the experts is a
-    gate: its column holds sigmoid(x . router[experts]). -> [T, R] float32."""
+    and weighted by the softmax over the chosen logits alone, every other expert 0. `groups` > 1: only experts of the
+    `keep` best of as many equal groups of neighbours can be chosen, a group's score being its largest logit. A last
+    row beyond the experts is a gate: its column holds sigmoid(x . router[experts]). -> [T, R] float32."""
     z = x.float() @ router.float().T
     logits = z[:, :experts] + (bias.float() if bias is not None else 0.0)
-    order = torch.sort(logits, dim=-1, descending=True, stable=True).indices[:, :top]
+    choice = logits
+    if groups > 1:
+        best = logits.view(-1, groups, experts // groups).amax(-1)
+        best = torch.sort(best, dim=-1, descending=True, stable=True).indices[:, :keep]
+        open_ = torch.zeros((logits.shape[0], groups), dtype=torch.bool, device=x.device).scatter_(1, best, True)
+        choice = logits.masked_fill(~open_.repeat_interleave(experts // groups, dim=1), float("-inf"))
+    order = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
     chosen = logits.gather(1, order)
     w = torch.zeros_like(logits).scatter_(1, order, torch.softmax(chosen, dim=-1))
     return torch.cat((w, torch.sigmoid(z[:, experts:])), dim=1).contiguous()
 
 
-def _moe_router_top_hip(launch, x, router, bias, experts, top):
+def _moe_router_top_hip(launch, x, router, bias, experts, top, groups=1, keep=1):
     (t, w), r = x.shape, router.shape[0]
     _need(x.is_cuda and x.is_contiguous() and x.dtype in _DT and router.is_contiguous() and router.dtype == torch.float32
           and router.shape == (r, w) and r in (experts, experts + 1) and 1 <= top <= experts <= 1024 and w <= 12288
-          and (bias is None or (bias.dtype == torch.float32 and bias.is_contiguous() and bias.shape == (experts,))),
-          f"moe_router_top: rows {tuple(x.shape)} {x.dtype}, router {tuple(router.shape)}, top {top} of {experts}")
+          and (bias is None or (bias.dtype == torch.float32 and bias.is_contiguous() and bias.shape == (experts,)))
+          and (groups <= 1 or (experts % groups == 0 and 1 <= keep <= groups and top <= keep * (experts // groups))),
+          f"moe_router_top: rows {tuple(x.shape)} {x.dtype}, router {tuple(router.shape)}, top {top} of {experts}, "
+          f"{groups} groups of which {keep}")
     weights = torch.empty((t, r), dtype=torch.float32, device=x.device)
     if t:
         launch(x.data_ptr(), router.data_ptr(), None if bias is None else bias.data_ptr(), weights.data_ptr(), t, w,
-               experts, r, int(top), _DT[x.dtype])
+               experts, r, int(top), _DT[x.dtype], int(groups), int(keep))
     return weights
 
 
@@ -215,7 +224,7 @@ register_kernel(KernelOp("moe_router", moe_router_plain, "holon_moe_router",
 register_kernel(KernelOp("moe_gate", moe_gate_plain, "holon_moe_gate", [_P, _P, _P, _L, _I, _I, _I, _I, _I, _I],
                          _moe_gate_hip))
 register_kernel(KernelOp("moe_router_top", moe_router_top_plain, "holon_moe_router_top",
-                         [_P, _P, _P, _P, _L, _I, _I, _I, _I, _I], _moe_router_top_hip))
+                         [_P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _I], _moe_router_top_hip))
 register_kernel(KernelOp("relu2", relu2_plain, "holon_relu2", [_P, _P, _L, _I], _relu2_hip))
 
 
@@ -293,7 +302,9 @@ class MoE(Part):
     """A mixture of SiLU-gated experts with a router, and an optional shared expert that every token uses.
 
     `score` "softmax_top" is the other router: float32 logits z = W_r x + b (`router_bias`), the `top` largest z are
-    chosen and weighted by the softmax over the chosen z alone (no groups, no scale). `shared_gated`: the shared
+    chosen and weighted by the softmax over the chosen z alone (no scale); with `groups` only among the `keep` groups
+    whose largest z are best. (A softmax over all experts whose chosen scores are then divided by their sum gives the
+    same weights: the largest score is always among the chosen, so their sum is never near zero.) `shared_gated`: the shared
     expert's output is multiplied by sigmoid(w_sg . x), one number a token; w_sg rides as one more row of the router's
     weights, so the router's kernel leaves that weight too. What follows describes `score` "sigmoid".
 
@@ -315,8 +326,8 @@ class MoE(Part):
             raise ValueError(f"moe: top {top} of {experts} experts")
         if score not in ("sigmoid", "softmax_top"):
             raise ValueError(f"moe: no router score {score!r} (sigmoid, softmax_top)")
-        if score == "softmax_top" and (groups > 1 or float(scale) != 1.0):
-            raise ValueError("moe: the softmax over the chosen logits comes without groups and without a scale")
+        if score == "softmax_top" and float(scale) != 1.0:
+            raise ValueError("moe: the softmax over the chosen logits comes without a scale")
         if shared_gated and (not shared or score != "softmax_top"):
             raise ValueError("moe: a gate on the shared expert needs a shared expert and the softmax_top router")
         self.score, self.shared_gated = score, bool(shared_gated)
@@ -372,7 +383,7 @@ class MoE(Part):
         k = self.kernels
         if self.score == "softmax_top":
             weights = k.moe_router_top(x, self.router, self.router_bias if self.has_bias else None, self.experts,
-                                       self.top)
+                                       self.top, self.groups, self.keep)
             act = k.moe_gate(self.gate_up(x), weights, self.inter, self.shared, shared_weight=self.shared_gated)
             return self.all_down(act)
         weights = k.moe_router(x, self.router, self.correction if self.has_bias else None, self.top, self.groups,

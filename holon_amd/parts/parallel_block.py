@@ -11,6 +11,10 @@ filter over time on every channel whose last taps - 1 inputs are part of the req
 feed-forward; its second norm and filter are then not built. With `shared_norm` the block has one norm and both
 sublayers read its result: x += mixer(f1(norm1(x))) + ffn(f1(norm1(x))).
 
+A norm on both sides of a sublayer (`block sandwich32`, `parts/dyt.py`) meets here as one kernel too (`stream_rms_post`):
+the sublayer's result is divided by its own root mean square, multiplied by a vector and added to the stream, and the sum
+is normed for the next sublayer.
+
 The norm `rms32` may hold its weight around zero (`one_plus`): y = x / sqrt(mean(x^2) + eps) * (1 + w); the sum 1 + w is
 formed once after loading, in float32, and kept in float32 whatever the engine's dtype.
 """
@@ -25,6 +29,7 @@ from ..registry import register_part
 from ..spec import PartRef
 from .base import FLOAT32, Build, NormPart, Part, Stream
 from .convs import CausalConv
+from .dyt import Scaled
 from .stream32 import Pending, _terms
 
 _P, _I, _L, _F = ctypes.c_void_p, ctypes.c_int, ctypes.c_int64, ctypes.c_float
@@ -133,6 +138,30 @@ def _stream_rms_filter_hip(launch, x32, terms, row, w1, w2, eps, out_dtype, taps
     return y1, y2
 
 
+def stream_rms_post_plain(x32, term, gain, term_eps, w, eps, out_dtype):
+    """x32 [T, W] float32, updated in place: x += gain * term / sqrt(mean(term^2) + term_eps) with `term` [T, W] in any
+    dtype and `gain` [W] float32. Then the answer x / sqrt(mean(x^2) + eps) * w in `out_dtype`. float32 arithmetic, one
+    rounding of the answer."""
+    t = term.float()
+    x32.add_(t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + term_eps) * gain)
+    return (x32 * torch.rsqrt(x32.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
+
+
+def _stream_rms_post_hip(launch, x32, term, gain, term_eps, w, eps, out_dtype):
+    _need(x32.is_cuda and x32.is_contiguous() and x32.dtype == torch.float32 and x32.dim() == 2,
+          "stream_rms_post: the stream is contiguous float32 rows on the GPU")
+    rows, dim = x32.shape
+    _need(term.is_cuda and term.is_contiguous() and term.shape == x32.shape and term.dtype in _DT,
+          "stream_rms_post: the term must be contiguous rows of the stream's shape")
+    _need(gain.is_contiguous() and gain.dtype == torch.float32 and gain.shape == (dim,) and w.is_contiguous()
+          and w.shape == (dim,) and w.dtype in _DT and out_dtype in _DT, "stream_rms_post: vectors of the rows' width")
+    y = torch.empty((rows, dim), dtype=out_dtype, device=x32.device)
+    if rows:
+        launch(x32.data_ptr(), term.data_ptr(), _DT[term.dtype], gain.data_ptr(), float(term_eps), w.data_ptr(),
+               _DT[w.dtype], y.data_ptr(), rows, dim, float(eps), _DT[out_dtype])
+    return y
+
+
 def scale_rows_plain(x, scale):
     """x [T, W] -> a new float32 tensor of scale * x."""
     return x.float() * scale
@@ -150,6 +179,8 @@ register_kernel(KernelOp("stream_rms", stream_rms_plain, "holon_stream_rms",
 register_kernel(KernelOp("stream_rms_filter", stream_rms_filter_plain, "holon_stream_rms_filter",
                          [_P, _P, _I, _P, _I, _P, _P, _P, _I, _P, _P, _L, _I, _F, _I, _P, _P, _P, _P, _P, _P, _I],
                          _stream_rms_filter_hip))
+register_kernel(KernelOp("stream_rms_post", stream_rms_post_plain, "holon_stream_rms_post",
+                         [_P, _P, _I, _P, _F, _P, _I, _P, _L, _I, _F, _I], _stream_rms_post_hip))
 register_kernel(KernelOp("scale_rows", scale_rows_plain, "holon_scale_rows", [_P, _P, _L, _I, _F], _scale_rows_hip))
 
 
@@ -182,9 +213,23 @@ class RMSNorm32(NormPart):
 
     __call__ = forward
 
-    def add(self, x, residual: torch.Tensor) -> tuple[torch.Tensor, torch.Tensor]:
-        """(norm(residual + x), residual + x): `residual` is float32 and takes the sum in place; `x` is a tensor or
-        `Pending` terms."""
+    def output_gain(self, scale: float, vector: torch.Tensor | None = None) -> torch.Tensor:
+        """weight * scale [* vector] in float32: everything behind this norm's division when its result is multiplied
+        by a constant and a vector before it joins a stream (a `Scaled` term's `gain`)."""
+        gain = self.weight.float() * scale
+        return (gain * vector.float() if vector is not None else gain).contiguous()
+
+    def add(self, x, residual: torch.Tensor, extra: torch.Tensor | None = None) -> tuple[torch.Tensor, torch.Tensor]:
+        """(norm(residual + x [+ extra]), the sum): `residual` is float32 and takes the sum in place; `x` is None, a
+        tensor, `Pending` terms, or a `Scaled` term behind an RMS norm."""
+        if isinstance(x, Scaled):
+            if extra is not None:
+                residual.add_(extra)
+            gain = x.gain if x.gain is not None else x.norm.output_gain(x.scale)
+            return self.kernels.stream_rms_post(residual, x.term, gain, x.norm.eps, self.weight, self.eps,
+                                                self.build.dtype), residual
+        if extra is not None:
+            residual.add_(extra)
         return self.kernels.stream_rms(residual, _terms(x), getattr(x, "row", None), self.weight, None, self.eps,
                                        self.build.dtype)[0], residual
 

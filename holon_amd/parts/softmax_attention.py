@@ -97,18 +97,21 @@ def _softmax_attention_hip(launch, q, pages, table, rows, token_row, positions, 
     return out
 
 
-def head_linear_plain(x, weight, out=None):
+def head_linear_plain(x, weight, out=None, gate=None):
     """x [T, H, A], weight [H, B, A] -> [T, H, B]: every head's own small projection, sums in float32, the result in
     x's dtype. `out`: where the result goes, the first B columns of every head of a tensor [T, H, B'] with B' >= B
-    (a view whose last dimension is contiguous); it is returned."""
-    y = torch.einsum("tha,hba->thb", x, weight.to(x.dtype))
+    (a view whose last dimension is contiguous); it is returned. `gate` [T, H B] (columns of wider rows will do): the
+    result is multiplied by its sigmoid."""
+    y = torch.matmul(x.transpose(0, 1), weight.to(x.dtype).transpose(1, 2).contiguous()).transpose(0, 1)
+    if gate is not None:
+        y = (y.float() * torch.sigmoid(gate.float()).reshape(y.shape)).to(x.dtype)
     if out is None:
         return y.contiguous()
     out.copy_(y)
     return out
 
 
-def _head_linear_hip(launch, x, weight, out=None):
+def _head_linear_hip(launch, x, weight, out=None, gate=None):
     """Steps of up to 16 rows: this package's kernel (the weights stream once, no copy of the result); more rows: the
     vendor library's batched product."""
     t, heads, a = x.shape
@@ -119,10 +122,14 @@ def _head_linear_hip(launch, x, weight, out=None):
     if out is not None and not (out.shape == (t, heads, b) and out.dtype == x.dtype and out.stride(2) == 1
                                 and out.stride(0) == heads * out.stride(1) and out.stride(1) >= b):
         raise ValueError(f"head_linear: the result's place {tuple(out.shape)} with strides {out.stride()} does not fit")
+    if gate is not None and not (gate.is_cuda and gate.dtype == x.dtype and gate.shape == (t, heads * b)
+                                 and gate.stride(1) == 1):
+        raise ValueError(f"head_linear: gates {tuple(gate.shape)} {gate.dtype} for {t} rows of {heads} heads of {b}")
     if not 1 <= t <= 16 or t * a * 4 > 48 * 1024:
-        return head_linear_plain(x, weight, out)
+        return head_linear_plain(x, weight, out, gate)
     y = out if out is not None else torch.empty((t, heads, b), dtype=x.dtype, device=x.device)
-    launch(x.data_ptr(), weight.data_ptr(), y.data_ptr(), t, heads, a, b, y.stride(1), _DT[x.dtype])
+    launch(x.data_ptr(), weight.data_ptr(), y.data_ptr(), t, heads, a, b, y.stride(1), _DT[x.dtype], _ptr(gate),
+           gate.stride(0) if gate is not None else 0)
     return y
 
 
@@ -169,22 +176,21 @@ def _whole_norm_prepare_hip(launch, qkv, heads, kv_heads, dim, vdim, q_weight, k
 
 
 def latent_rope_prepare_plain(both, heads, dim, rot, kv_rank, c_weight, eps, table, positions, pages, write_page,
-                              write_off, page_size):
-    """both [T, H (dim + rot) + kv_rank + rot]: every head's query as [dim unrotated, rot rotated], then the latent's
-    projection and one rotated key part that all heads share. The latent is divided by its root mean square and
+                              write_off, page_size, copies=2):
+    """both [T, H (dim + rot) + kv_rank + rot] (rows may be wider): every head's query as [dim unrotated, rot rotated],
+    then the latent's projection and one rotated key part that all heads share. The latent is divided by its root mean square and
     multiplied by `c_weight` (float32 inside, one rounding); the first table.shape[1] dimensions of every rotated part
     (queries and key) are rotated by the token's position, half-split pairing, `table` [positions, rotary_dim] float32
     holding cosines then sines. The token's cache entry [latent, rotated key part] goes into `pages` [pages, 2 P
-    (kv_rank + rot)] twice, as a key (row of [P, kv_rank + rot]) and as a value (column of [kv_rank + rot, P]).
+    (kv_rank + rot)] twice, as a key (row of [P, kv_rank + rot]) and as a value (column of [kv_rank + rot, P]); `copies`
+    1: once, as the row, into pages of [P, kv_rank + rot] alone. `pages` None: the rows hold queries alone and nothing
+    is stored.
     Returns (the unrotated query parts [T, H, dim], the queries in the cache's space [T, H, kv_rank + rot] with the
     rotated parts in their last `rot` columns and the first kv_rank left for the caller to fill)."""
     t = both.shape[0]
     width = kv_rank + rot
     q = both[:, : heads * (dim + rot)].view(t, heads, dim + rot)
-    tail = both[:, heads * (dim + rot):]
-    cf = tail[:, :kv_rank].float()
-    c = (cf * torch.rsqrt(cf.pow(2).mean(-1, keepdim=True) + eps) * c_weight.float()).to(both.dtype)
-    rd = table.shape[1] if table is not None else 0
+    tail = both[:, heads * (dim + rot): heads * (dim + rot) + width]
 
     def turn(x):                                   # x [T, n, rot]
         if not rd:
@@ -193,37 +199,87 @@ def latent_rope_prepare_plain(both, heads, dim, rot, kv_rank, c_weight, eps, tab
         cos, sin = cs[:, None, : rd // 2], cs[:, None, rd // 2:]
         a, b = x[..., : rd // 2].float(), x[..., rd // 2: rd].float()
         return torch.cat(((a * cos - b * sin).to(x.dtype), (b * cos + a * sin).to(x.dtype), x[..., rd:]), dim=-1)
-    entry = torch.cat((c, turn(tail[:, None, kv_rank:])[:, 0]), dim=-1)
-    keys = pages[:, : page_size * width].view(-1, page_size, width)
-    vals = pages[:, page_size * width:].view(-1, width, page_size)
-    keys[write_page[:t].long(), write_off[:t].long()] = entry
-    vals[write_page[:t].long(), :, write_off[:t].long()] = entry
+    rd = table.shape[1] if table is not None else 0
     full = torch.zeros((t, heads, width), dtype=both.dtype, device=both.device)
     full[..., kv_rank:] = turn(q[..., dim:])
+    if pages is None:
+        return q[..., :dim].contiguous(), full
+    cf = tail[:, :kv_rank].float()
+    c = (cf * torch.rsqrt(cf.pow(2).mean(-1, keepdim=True) + eps) * c_weight.float()).to(both.dtype)
+    entry = torch.cat((c, turn(tail[:, None, kv_rank:])[:, 0]), dim=-1)
+    keys = pages[:, : page_size * width].view(-1, page_size, width)
+    keys[write_page[:t].long(), write_off[:t].long()] = entry
+    if copies == 2:
+        vals = pages[:, page_size * width:].view(-1, width, page_size)
+        vals[write_page[:t].long(), :, write_off[:t].long()] = entry
     return q[..., :dim].contiguous(), full
 
 
 def _latent_rope_prepare_hip(launch, both, heads, dim, rot, kv_rank, c_weight, eps, table, positions, pages, write_page,
-                             write_off, page_size):
+                             write_off, page_size, copies=2):
     t = both.shape[0]
     width = kv_rank + rot
     rd = table.shape[1] if table is not None else 0
-    ok = both.is_cuda and both.is_contiguous() and both.dtype in _DT and both.shape[1] == heads * (dim + rot) + width \
-        and pages.dtype == both.dtype and pages.is_contiguous() and pages.dim() == 2 \
-        and pages.shape[1] == 2 * page_size * width and c_weight.dtype == both.dtype and c_weight.is_contiguous() \
-        and c_weight.shape == (kv_rank,) and write_page.shape[0] >= t and write_off.shape[0] >= t \
-        and positions.shape[0] >= t and rd % 2 == 0 and rd <= rot \
+    ok = both.is_cuda and both.is_contiguous() and both.dtype in _DT \
+        and both.shape[1] >= heads * (dim + rot) + (width if pages is not None else 0) \
+        and positions.shape[0] >= t and rd % 2 == 0 and rd <= rot and copies in (1, 2) \
         and (table is None or (table.dtype == torch.float32 and table.is_contiguous()))
+    if ok and pages is not None:
+        ok = pages.dtype == both.dtype and pages.is_contiguous() and pages.dim() == 2 \
+            and pages.shape[1] == copies * page_size * width and c_weight.dtype == both.dtype and c_weight.is_contiguous() \
+            and c_weight.shape == (kv_rank,) and write_page.shape[0] >= t and write_off.shape[0] >= t
     if not ok:
-        raise ValueError(f"latent_rope_prepare: rows {tuple(both.shape)} {both.dtype}, pages {tuple(pages.shape)} do not "
-                         f"fit {heads} heads of {dim} + {rot}, a latent of {kv_rank}, page {page_size}")
+        raise ValueError(f"latent_rope_prepare: rows {tuple(both.shape)} {both.dtype}, pages "
+                         f"{None if pages is None else tuple(pages.shape)} do not fit {heads} heads of {dim} + {rot}, a latent of {kv_rank}, page {page_size}")
     q = torch.empty((t, heads, dim), dtype=both.dtype, device=both.device)
     full = torch.empty((t, heads, width), dtype=both.dtype, device=both.device)
     if t:
-        launch(both.data_ptr(), t, heads, dim, rot, kv_rank, c_weight.data_ptr(), float(eps), _ptr(table), rd,
+        launch(both.data_ptr(), both.shape[1], t, heads, dim, rot, kv_rank, _ptr(c_weight), float(eps), _ptr(table), rd,
                table.shape[0] if table is not None else 0, positions.data_ptr(), q.data_ptr(), full.data_ptr(),
-               pages.data_ptr(), write_page.data_ptr(), write_off.data_ptr(), page_size, pages.shape[0], _DT[both.dtype])
+               _ptr(pages), _ptr(write_page), _ptr(write_off), page_size, pages.shape[0] if pages is not None else 1,
+               copies, _DT[both.dtype])
     return q, full
+
+
+def latent_attention_plain(q, pages, table, rows, token_row, positions, kv_rank, page_size, sink, scale, window):
+    """Attention over latent entries kept once: q [T, H, W], `pages` [pages, P W], a token's entry a row of W values that
+    every head reads as its key, and the entry's first `kv_rank` values as its value. Rows, table, sink and window as
+    for `softmax_attention`. -> [T, H, kv_rank] in q's dtype; scores, weights and sums in float32."""
+    t, heads, width = q.shape
+    keys = pages.view(-1, page_size, width)
+    up = (lambda x: x) if q.dtype == torch.float64 else (lambda x: x.float())
+    out = torch.zeros((t, heads, kv_rank), dtype=up(q).dtype, device=q.device)
+    pos, slot_of, row_of = positions.tolist(), rows.slots.tolist(), token_row.tolist()
+    for i in range(t):
+        js = torch.arange(max(0, pos[i] - window + 1) if window > 0 else 0, pos[i] + 1, device=q.device)
+        e = up(keys[table[slot_of[row_of[i]], (js // page_size)].long(), js % page_size])          # [n, W]
+        s = up(q[i]) @ e.T * scale                                                                  # [H, n]
+        top = s.max(1, keepdim=True).values
+        if sink is not None:
+            top = torch.maximum(top, up(sink)[:, None])
+        w = torch.exp(s - top)
+        den = w.sum(1, keepdim=True)
+        if sink is not None:
+            den = den + torch.exp(up(sink)[:, None] - top)
+        out[i] = (w @ e[:, :kv_rank]) / den
+    return out.to(q.dtype)
+
+
+def _latent_attention_hip(launch, q, pages, table, rows, token_row, positions, kv_rank, page_size, sink, scale, window):
+    t, heads, width = q.shape
+    ok = q.is_cuda and q.is_contiguous() and q.dtype in _DT and pages.dtype == q.dtype and pages.is_contiguous() \
+        and pages.dim() == 2 and pages.shape[1] == page_size * width and 0 < kv_rank <= width \
+        and table.dtype == torch.int32 and table.is_contiguous() and token_row.shape[0] >= t and positions.shape[0] >= t \
+        and (sink is None or (sink.dtype == torch.float32 and sink.is_contiguous() and sink.shape == (heads,)))
+    if not ok:
+        raise ValueError(f"latent_attention: q {tuple(q.shape)} {q.dtype}, pages {tuple(pages.shape)} do not fit entries of "
+                         f"{width} with latents of {kv_rank}, page {page_size}")
+    out = torch.empty((t, heads, kv_rank), dtype=q.dtype, device=q.device)
+    if t:
+        launch(q.data_ptr(), out.data_ptr(), pages.data_ptr(), table.data_ptr(), table.shape[1], table.shape[0],
+               rows.slots.data_ptr(), token_row.data_ptr(), positions.data_ptr(), t, heads, width, kv_rank, page_size,
+               pages.shape[0], _ptr(sink), float(scale), int(window), _DT[q.dtype])
+    return out
 
 
 def latent_prepare_plain(both, q_rank, q_weight, c_weight, eps, pages, write_page, write_off, page_size):
@@ -298,12 +354,15 @@ register_kernel(KernelOp("softmax_attention", softmax_attention_plain, "holon_so
                          [_P, _P, _P, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _F, _I, _I, _F, _P, _P, _I, _I],
                          _softmax_attention_hip))
 register_kernel(KernelOp("head_linear", head_linear_plain, "holon_head_linear_rows",
-                         [_P, _P, _P, _I, _I, _I, _I, _I, _I], _head_linear_hip))
+                         [_P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _L], _head_linear_hip))
 register_kernel(KernelOp("whole_norm_prepare", whole_norm_prepare_plain, "holon_whole_norm_prepare",
                          [_P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _P, _P, _P, _I, _I, _I], _whole_norm_prepare_hip))
 register_kernel(KernelOp("latent_rope_prepare", latent_rope_prepare_plain, "holon_latent_rope_prepare",
-                         [_P, _I, _I, _I, _I, _I, _P, _F, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I],
+                         [_P, _I, _I, _I, _I, _I, _I, _P, _F, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I],
                          _latent_rope_prepare_hip))
+register_kernel(KernelOp("latent_attention", latent_attention_plain, "holon_latent_attention",
+                         [_P, _P, _P, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _F, _I, _I],
+                         _latent_attention_hip))
 register_kernel(KernelOp("latent_prepare", latent_prepare_plain, "holon_latent_prepare",
                          [_P, _I, _I, _I, _P, _P, _F, _P, _P, _P, _P, _I, _I, _I], _latent_prepare_hip))
 register_kernel(KernelOp("head_gate", head_gate_plain, "holon_head_gate", [_P, _P, _L, _L, _I, _I, _I], _head_gate_hip))
@@ -511,14 +570,27 @@ class LatentAttention(Part):
     columns for the rotated part). `position` (a registered position part with a `table`) rotates the first
     `rotary_dim` of the rot_dim dimensions; one that says `interleaved` has the rows of W_q and W_dkv reordered once
     so that the kernels' half-split pairing rotates the design's pairs. `sink`: one number a head in the softmax's
-    denominator."""
+    denominator.
+
+    Options of the second form. `entries` 1: the cache holds an entry once, as a row, and the attention kernel takes the
+    row's first kv_rank values as its value (2: as key and as value, for the kernels that want values transposed).
+    `gate`: the heads' results are multiplied, value by value, by sigmoid(W_g x); W_g rides in the merged product.
+    `own_kv` False: the layer has no W_dkv and attends over the entries another layer's run has cached
+    (`Run.reads`), with its own W_q, W_uk and W_uv."""
 
     graph_safe = True
 
     def __init__(self, build: Build, *, heads: int, dim: int, vdim: int, kv_rank: int, norm: PartRef, hidden: int,
                  layer: int, q_rank: int = 0, rot_dim: int = 0, position: PartRef | None = None, sink: bool = False,
-                 scale: float | None = None, window: int = 0, name: str = "") -> None:
+                 scale: float | None = None, window: int = 0, gate: bool = False, entries: int = 2, own_kv: bool = True,
+                 name: str = "") -> None:
         super().__init__(build)
+        if q_rank > 0 and (gate or entries != 2 or not own_kv):
+            raise ValueError("latent_attention: queries through a latent of their own come without a gate, with entries "
+                             "kept as key and as value, and with a latent of the layer's own")
+        if entries not in (1, 2):
+            raise ValueError(f"latent_attention: an entry is kept once or twice, not {entries} times")
+        self.has_gate, self.entries, self.own_kv = bool(gate), int(entries), bool(own_kv)
         if q_rank > 0 and (rot_dim > 0 or position is not None):
             raise ValueError("latent_attention: queries through a latent of their own come without a rotated part")
         if position is not None and rot_dim < 2:
@@ -535,8 +607,11 @@ class LatentAttention(Part):
             self.attach("uq", Linear(build, inp=q_rank, out=heads * dim))
         else:
             self.attach("q", Linear(build, inp=hidden, out=heads * (dim + self.rot_dim)))
-        self.attach("dkv", Linear(build, inp=hidden, out=self.width))
-        self.attach("dkv_norm", build.make(norm, dim=kv_rank))
+        if self.own_kv:
+            self.attach("dkv", Linear(build, inp=hidden, out=self.width))
+            self.attach("dkv_norm", build.make(norm, dim=kv_rank))
+        if self.has_gate:
+            self.attach("g", Linear(build, inp=hidden, out=heads * vdim))
         self.declare("uk", (heads * dim, kv_rank))
         self.declare("uv", (heads * vdim, kv_rank))
         self.attach("o", Linear(build, inp=heads * vdim, out=hidden))
@@ -552,7 +627,7 @@ class LatentAttention(Part):
                                                   # norms the latents and writes the cache
 
     def state(self):
-        return [PagedState(self.state_name, elems=2 * self.width, window=self.window)]
+        return [PagedState(self.state_name, elems=self.entries * self.width, window=self.window)]
 
     def finalize(self) -> None:
         first = self.dq if self.q_rank > 0 else self.q
@@ -563,41 +638,58 @@ class LatentAttention(Part):
             order = [h * per + r for h in range(self.heads) for r in list(range(self.dim)) + [self.dim + r for r in one]]
             dev = first.weight.device
             self.q.weight = self.q.weight.index_select(0, torch.tensor(order, device=dev)).contiguous()
-            order = list(range(self.kv_rank)) + [self.kv_rank + r for r in one]
-            self.dkv.weight = self.dkv.weight.index_select(0, torch.tensor(order, device=dev)).contiguous()
-        self.down = Linear.merge(self.build, first, self.dkv)
-        self.drop("dq" if self.q_rank > 0 else "q")
-        self.drop("dkv")
+            if self.own_kv:
+                order = list(range(self.kv_rank)) + [self.kv_rank + r for r in one]
+                self.dkv.weight = self.dkv.weight.index_select(0, torch.tensor(order, device=dev)).contiguous()
+        merged = ["dq" if self.q_rank > 0 else "q"] + (["dkv"] if self.own_kv else []) + (["g"] if self.has_gate else [])
+        self.gate_at = sum(getattr(self, name).out for name in merged) - self.heads * self.vdim      # W_g's first column
+        if self.q_rank == 0 and first.weight is not None:      # rows of zeros pad the product to a multiple of 16, which
+            last = getattr(self, merged[-1])                   # the few-row products ask for
+            pad = -sum(getattr(self, name).out for name in merged) % 16
+            if pad:
+                last.weight = torch.cat((last.weight, last.weight.new_zeros((pad, last.inp)))).contiguous()
+                last.out += pad
+        self.down = Linear.merge(self.build, *(getattr(self, name) for name in merged))
+        for name in merged:
+            self.drop(name)
         self._children["down"] = self.down
-        norms = [self.dkv_norm] + ([self.dq_norm] if self.q_rank > 0 else [])
+        norms = ([self.dkv_norm] if self.own_kv else []) + ([self.dq_norm] if self.q_rank > 0 else [])
         specs = [n.fusion() for n in norms]
-        if all(sp is not None and sp.get("norm") == "rmsnorm" and sp["weight"] is not None for sp in specs) \
+        if specs and all(sp is not None and sp.get("norm") == "rmsnorm" and sp["weight"] is not None for sp in specs) \
                 and len({sp["eps"] for sp in specs}) == 1:
             self._fused = float(specs[0]["eps"])
-        if self.q_rank == 0 and self._fused is None:
+        if self.q_rank == 0 and self._fused is None and self.own_kv:
             raise ValueError("latent_attention: the form with a rotated part needs an RMS norm on the latent")
         if self.uk is not None:
             # [H, kv_rank, dim]: what turns a head's query into the latent's space; [H, vdim, width]: a head's values
             self.uk_t = self.uk.view(self.heads, self.dim, self.kv_rank).transpose(1, 2).contiguous()
             self.uv_h = self.uv.view(self.heads, self.vdim, self.kv_rank)
-            if self.rot_dim:
+            if self.rot_dim and self.entries == 2:
                 pad = torch.zeros((self.heads, self.vdim, self.rot_dim), dtype=self.uv.dtype, device=self.uv.device)
                 self.uv_h = torch.cat((self.uv_h, pad), dim=-1).contiguous()
 
     def extra_tensors(self):
         held = [self.uk_t] if self.uk_t is not None else []
-        return held + ([self.uv_h] if self.rot_dim and self.uv_h is not None else [])
+        return held + ([self.uv_h] if self.rot_dim and self.entries == 2 and self.uv_h is not None else [])
 
     def forward(self, x: torch.Tensor, step, site) -> torch.Tensor:
         k = self.kernels
         t = x.shape[0]
+        if site.writes != self.own_kv:
+            raise ValueError("latent_attention: a layer with a latent of its own writes its cache; one without reads "
+                             "another run's")
         held = site.paged[self.state_name]
         view = step.paged[held.group]
         both = self.down(x)
         if self.q_rank == 0:                      # norm, rotation and the cache write in one kernel
-            q, full = k.latent_rope_prepare(both, self.heads, self.dim, self.rot_dim, self.kv_rank,
-                                            self.dkv_norm.weight, self._fused, getattr(self.position, "table", None),
-                                            step.positions, held.pages, view.write_page, view.write_off, view.page_size)
+            table = getattr(self.position, "table", None)
+            if self.own_kv:
+                q, full = k.latent_rope_prepare(both, self.heads, self.dim, self.rot_dim, self.kv_rank,
+                                                self.dkv_norm.weight, self._fused, table, step.positions, held.pages,
+                                                view.write_page, view.write_off, view.page_size, copies=self.entries)
+            else:
+                q, full = k.latent_rope_prepare(both, self.heads, self.dim, self.rot_dim, self.kv_rank, None, 0.0, table,
+                                                step.positions, None, None, None, view.page_size)
             k.head_linear(q, self.uk_t, out=full[..., : self.kv_rank])
             q = full
         else:
@@ -610,9 +702,15 @@ class LatentAttention(Part):
                 k.kv_write(c, c, held.pages.view(-1, 2, 1, view.page_size * self.kv_rank), view.write_page,
                            view.write_off, view.page_size)
             q = k.head_linear(self.uq(cq).view(t, self.heads, self.dim), self.uk_t)
-        mixed = attend(k, q, held, view, step, 1, self.width, self.sink if self.has_sink else None, self.scale,
-                       self.window)
-        out = k.head_linear(mixed.view(t, self.heads, self.width), self.uv_h)
+        sink = self.sink if self.has_sink else None
+        if self.entries == 1:
+            mixed = k.latent_attention(q, held.pages, view.table, step.rows, step.token_row, step.positions, self.kv_rank,
+                                       view.page_size, sink, self.scale, self.window)
+        else:
+            mixed = attend(k, q, held, view, step, 1, self.width, sink, self.scale, self.window
+                           ).view(t, self.heads, self.width)
+        gate = both[:, self.gate_at: self.gate_at + self.heads * self.vdim] if self.has_gate else None
+        out = k.head_linear(mixed, self.uv_h, gate=gate) if gate is not None else k.head_linear(mixed, self.uv_h)
         return self.o(out.view(t, self.heads * self.vdim))
 
     __call__ = forward
