@@ -25,7 +25,8 @@ prompts of 32,768 tokens at the Qwen3-4B shape, 512 tokens each at temperature 0
 feed-forward, vocabulary; random weights): a 2,048-token prompt and decode at batch 8 near a context of 2,048, at two
 sizes (`--sizes`), one line with both models' figures and the bytes a decode step must read. `--only` runs one model
 (for a profiler). --workload dopirax measures Dopirax the same way, beside Nevodra (the nearest design: both sublayers
-on one float32 stream, a capped attention, experts) and Qwen3 (`--beside`).
+on one float32 stream, a capped attention, experts) and Qwen3 (`--beside`); --workload falisun measures Falisun beside
+Nevodra (latent attention, experts) and Qwen3.
 """
 from __future__ import annotations
 
@@ -192,8 +193,33 @@ def dopirax_config(z: dict) -> dict:
             "embedding": {"scale": 1.0}, "layers": [layer(i) for i in range(z["layers"])]}
 
 
+def falisun_config(z: dict) -> dict:
+    """A Falisun model of a size's layers, in fours: a Mamba-2 layer (values of twice the width in heads of 64, a state of
+    128 rows, one group of B and C), latent attention (the size's heads, a latent of 512 and 64 rotated dimensions: cache
+    entries of 576), another Mamba-2 layer, and latent attention that reads the entries of the one before; over eight
+    experts of an eighth of the size's feed-forward of which a token uses four, in four groups of which three stay
+    open, beside a shared one of a quarter."""
+    mlp = {"kind": "moe", "expert": {"ff": z["ff"] // 8}, "shared": {"ff": z["ff"] // 4},
+           "router": {"experts": 8, "top": 4, "groups": {"count": 4, "keep": 3}}}
+
+    def layer(i: int) -> dict:
+        if i % 2 == 0:
+            return {"type": "mamba2", "mlp": mlp, "mixer": {"heads": 2 * z["width"] // 64, "vdim": 64, "state": 128,
+                                                            "groups": 1, "norm_groups": 1, "conv": 4}}
+        m = {"heads": z["heads"], "dim": z["dim"], "rot_dim": 64, "vdim": z["dim"], "kv_rank": 512,
+             "scale": (z["dim"] + 64) ** -0.5,
+             "rot": {"dims": 64, "base": 10000.0,
+                     "scaling": {"factor": 40.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+        if i % 4 == 3:
+            m["kv_from"] = i - 2
+        return {"type": "latent_attention", "mixer": m, "mlp": mlp}
+    return {"architecture": "Falisun", "width": z["width"], "vocab": z["vocab"], "norm": {"eps": 1e-6},
+            "layers": [layer(i) for i in range(z["layers"])]}
+
+
 DESIGN_CONFIGS = {"tolurax": tolurax_config, "relanex": relanex_config, "nevodra": nevodra_config,
-                  "dopirax": dopirax_config}
+                  "dopirax": dopirax_config, "falisun": falisun_config}
+BESIDE = {"dopirax": "nevodra,qwen3", "falisun": "nevodra,qwen3"}      # what a design is measured beside (others: qwen3)
 
 
 def design_cache_bytes(name: str, cfg_json: dict, z: dict, item: int, batch: int, context: int) -> int:
@@ -203,7 +229,10 @@ def design_cache_bytes(name: str, cfg_json: dict, z: dict, item: int, batch: int
     total = 0
     for layer in cfg_json["layers"]:
         m = layer["mixer"]
-        if name == "dopirax":                       # every layer reads all of a cache, its own or another layer's
+        if name == "falisun":                       # an entry once, read as key and value, by the layer that shares it too
+            if layer["type"] == "latent_attention":
+                total += (m["kv_rank"] + m["rot_dim"]) * item * batch * context
+        elif name == "dopirax":                       # every layer reads all of a cache, its own or another layer's
             maps = 2 if layer["type"] == "attention_2" else 1     # differential layers keep the keys of both maps
             total += m["kv_heads"] * (maps * m["dim"] + m["vdim"]) * item * batch * context
         elif layer["type"] == "parallel":             # the window's keys and values
@@ -225,7 +254,7 @@ def qwen3_config(z: dict) -> dict:
 
 
 def design(a) -> int:
-    """A design (Tolurax or Relanex) beside Qwen3 at equal sizes: prompt and decode throughput, one line."""
+    """A design beside others at equal sizes: prompt and decode throughput, one line."""
     import gc
 
     import torch
@@ -239,7 +268,7 @@ def design(a) -> int:
     for size in a.sizes.split(","):
         z = DESIGN_SIZES[size]
         ours = DESIGN_CONFIGS[a.workload](z)
-        others = [n for n in (a.beside or ("nevodra,qwen3" if a.workload == "dopirax" else "qwen3")).split(",") if n]
+        others = [n for n in (a.beside or BESIDE.get(a.workload, "qwen3")).split(",") if n]
         beside = [(n, qwen3_config(z) if n == "qwen3" else DESIGN_CONFIGS[n](z)) for n in others if n != a.workload]
         for name, cfg_json in [(a.workload, ours)] + beside:
             if a.only and a.only != name:
@@ -250,7 +279,8 @@ def design(a) -> int:
                 graphs=not a.no_graphs, products=a.products, prefix_cache=False))
             item = 2 if a.dtype == "bfloat16" else 4
             weights = sum(getattr(o, n).numel() * getattr(o, n).element_size()
-                          for path, o, n, _ in engine.model.named_params() if not path.startswith("embed."))
+                          for path, o, n, _ in engine.model.named_params()
+                          if not path.startswith("embed.") or engine.model.lm_head.tied)     # (a tied head reads it all)
             # what a request keeps in its slot (the recurrences' matrices, the filters' inputs): read and written a step
             state = sum(t[0].numel() * t.element_size() for _, _, t in engine.cache.slot_states)
             times = []
@@ -313,14 +343,14 @@ def main(argv: list[str] | None = None) -> int:
     ap.add_argument("--context", type=int, default=CONTEXT, help="the context the timed decode steps end at")
     ap.add_argument("--prompt", type=int, default=PROMPT, help="tokens of the timed prompt")
     ap.add_argument("--no-graphs", action="store_true")
-    ap.add_argument("--workload", choices=("decode", "mixed", "long", "tolurax", "relanex", "nevodra", "dopirax"),
+    ap.add_argument("--workload", choices=("decode", "mixed", "long", *DESIGN_CONFIGS),
                     default="decode")
-    ap.add_argument("--sizes", default="2k,4k", help="--workload tolurax|relanex|nevodra|dopirax: which of its sizes (2k, 4k) to run")
-    ap.add_argument("--only", choices=("tolurax", "relanex", "nevodra", "dopirax", "qwen3"), default=None,
-                    help="--workload tolurax|relanex|nevodra|dopirax: one model only")
+    ap.add_argument("--sizes", default="2k,4k", help="--workload of a design: which of its sizes (2k, 4k) to run")
+    ap.add_argument("--only", choices=(*DESIGN_CONFIGS, "qwen3"), default=None,
+                    help="--workload of a design: one model only")
     ap.add_argument("--beside", default=None,
                     help="--workload of a design: the models it is measured beside, with commas (default: qwen3; for "
-                         "dopirax: nevodra,qwen3)")
+                         "dopirax and falisun: nevodra,qwen3)")
     ap.add_argument("--products", choices=("own", "vendor", "timed"), default="timed",
                     help="EngineConfig.products: which kernel products of 17 to 1,024 rows take (reported in the line)")
     a = ap.parse_args(argv)

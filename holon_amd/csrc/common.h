@@ -59,6 +59,11 @@ __device__ __forceinline__ void load_to_lds16(const void* base, uint32_t lane_by
   asm volatile("s_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, %1"
                : : "v"(lane_bytes), "s"(base), "s"(lds_wave_base) : "memory", "m0");
 }
+// The same with an address of the lane's own, wherever it lies.
+__device__ __forceinline__ void load_to_lds16_from(const void* lane_address, uint32_t lds_wave_base) {
+  asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off"
+               : : "v"(lane_address), "s"(lds_wave_base) : "memory", "m0");
+}
 // A 16-byte load into registers that the compiler does not track either, for kernels whose other loads are the copies
 // above: the compiler counts only the loads it knows, so where both kinds are under way the waits it inserts before a
 // known load's first use come out wrong for the mix (far too early a wait, measured). The caller waits

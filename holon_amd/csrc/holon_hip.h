@@ -326,6 +326,19 @@ int holon_latent_attention(const void* q, void* out, const void* pages, const in
                            int table_rows, const int32_t* slots, const int32_t* token_row, const int32_t* positions,
                            int tokens, int heads, int width, int kv_rank, int page_size, int num_pages,
                            const float* sink, float scale, int window, int dtype, void* stream);
+// The same on the matrix cores, bfloat16, no window: prompt portions (rows listed in row_ids, of at most max_query tokens)
+// and decode rows (a row's keys cut into `splits` <= 64 shares of `per`, a multiple of 64; with more than one share
+// part_o [rows, heads, splits, kv_rank] and part_ml [rows, heads, splits, 2] float32 take the partial results).
+int holon_latent_cores_supported(int width, int kv_rank);
+int holon_latent_prefill_bf16(const void* q, void* out, const void* pages, const int32_t* table, int table_stride,
+                              int table_rows, const int32_t* slots, const int32_t* lens, const int32_t* qstart,
+                              const int32_t* row_ids, int rows, int max_query, int heads, int width, int kv_rank,
+                              int page_size, int num_pages, const float* sink, float scale, void* stream);
+int holon_latent_decode_bf16(const void* q, void* out, const void* pages, const int32_t* table, int table_stride,
+                             int table_rows, const int32_t* slots, const int32_t* lens, const int32_t* qstart,
+                             const int32_t* row_ids, int rows, int max_len, int heads, int width, int kv_rank,
+                             int page_size, int num_pages, const float* sink, float scale, int splits, int per,
+                             float* part_o, float* part_ml, void* stream);
 
 // The latent attention's two latents, side by side in `both` [T, q_rank + kv_rank]: each divided by its root mean square
 // and multiplied by its weight; the first to cq [T, q_rank], the second into the token's page as a key row and as a

@@ -7,10 +7,17 @@
 // and weigh them with the tile's weights, handed round from the lanes that hold them. Every wave keeps a running maximum,
 // sum and weighted values; the four are combined at the end in wave order, the sink joining there. Which keys a wave takes
 // and in which order is decided by the query's position alone. Scores, weights and sums are float32.
+//
+// The matrix-core kernels (bfloat16, no window): prompt portions and decode rows, below.
 #include "common.h"
 #include "holon_hip.h"
 
 #define LAT_MAX 1024
+
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16x4_t __attribute__((ext_vector_type(4)));
+typedef short s16x4_t __attribute__((ext_vector_type(4)));
+typedef float f32x4_t __attribute__((ext_vector_type(4)));
 
 namespace {
 
@@ -107,7 +114,449 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(
     out[((int64_t)t * heads + h) * kv_rank + d] = Elem<T>::store(o * inv);
   }
 }
+
+// -- on the matrix cores ------------------------------------------------------------------------------------------------
+// A tile's 16 rows are (token, head) pairs in the order they lie in: all heads read the same entries, so a row is no more
+// than a query of `width` values at a position. Operands (v_mfma_f32_16x16x32_bf16: lane l = 16 g + c holds eight values
+// of row / column c; the result's lane holds rows 4 g + r, r < 4, of column c):
+//   S^T = E Q^T     A = 16 entries x 32 of their values, rows as they lie; two products cover 32 keys, and lane (g, c)
+//                   then holds the scores of keys 4 g + r and 16 + 4 g + r of query c. In that order of the inner
+//                   dimension they are the B operand of
+//   O^T = E_c^T P^T A = 16 of the latent's values x 32 keys: the entries' columns, which ds_read_b64_tr_b16 reads out of
+//                   LDS transposed (16 lanes give the addresses of 4 rows x 16 values and get a column's 4 rows each).
+// So an entry lies in memory once and in LDS once, and serves both products from there.
+// Entries come into LDS by the memory pipeline (16 bytes a lane, a wave's 64 lanes into one contiguous kilobyte). A row's
+// pitch in LDS is WP / 2 + 8 words, 8 times an odd number: eight neighbouring rows then start 8 banks apart, which keeps
+// the transposed reads and the row reads free of conflicts. A row's columns from `width` on repeat its first ones (the
+// query is zero there); rows past the last key repeat the last key's entry (their weights are zero).
+// RP, WP: the latent's and the entry's widths, padded to the next sizes that are compiled.
+struct LatArgs {
+  const bf16_t* q;
+  bf16_t* out;
+  const bf16_t* pages;
+  const int32_t* table;
+  const int32_t* slots;
+  const int32_t* lens;
+  const int32_t* qstart;
+  const int32_t* row_ids;
+  const float* sink;
+  float* part_o;
+  float* part_ml;
+  int table_stride, table_rows, num_pages, page_size, heads, width, kv_rank;
+  int per, splits;             // decode rows: keys a block takes (a multiple of 64), blocks a (row, 16 heads)
+  float scale_log2;
+};
+
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+__device__ __forceinline__ bf16x4_t read_transposed(const unsigned char* p) {
+  typedef __attribute__((address_space(3))) s16x4_t* lds_ptr;
+  return __builtin_bit_cast(bf16x4_t, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)p));
+}
+
+__device__ __forceinline__ float max_over_groups(float v) {   // over the four lane groups of 16
+  const auto rows = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  v = fmaxf(__uint_as_float(rows[0]), __uint_as_float(rows[1]));
+  const auto halves = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  return fmaxf(__uint_as_float(halves[0]), __uint_as_float(halves[1]));
+}
+
+// KEYS entries on their way into one buffer: what each lane of a block of four waves copies.
+template <int WP, int KEYS>
+struct EntryCopies {
+  static constexpr int PC = WP / 8 + 2;                  // 16-byte pieces a row takes in LDS
+  static constexpr int PITCH = PC * 16, BYTES = KEYS * PITCH, NI = KEYS * PC / 64, CI = (NI + 3) / 4;
+  static_assert(KEYS * PC % 64 == 0 && (PC / 2) % 2 == 1, "whole kilobytes, an odd multiple of 8 words a row");
+  int row[CI];                                           // the row a piece belongs to, and its place in the entry
+  uint32_t col[CI];
+  uint32_t lds0;
+  int wave;
+  __device__ __forceinline__ void init(const unsigned char* lds, int width) {
+    wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
+    lds0 = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void*)lds;
+    const int pieces = width / 8;
+#pragma unroll
+    for (int i = 0; i < CI; ++i) {
+      const int at = (wave + 4 * i) * 64 + threadIdx.x % WAVE, c = at % PC;
+      row[i] = min(at / PC, KEYS - 1);
+      col[i] = (uint32_t)(c < pieces ? c : c % pieces) * 16;
+    }
+  }
+  // `from`: the byte offset of every row's entry among the pages, in LDS
+  __device__ __forceinline__ void copy(const bf16_t* pages, const int64_t* from, uint32_t buffer) const {
+#pragma unroll
+    for (int i = 0; i < CI; ++i) {
+      if (wave + 4 * i >= NI) break;                     // (the same in all of a wave's lanes)
+      load_to_lds16_from(reinterpret_cast<const unsigned char*>(pages) + from[row[i]] + col[i],
+                         __builtin_amdgcn_readfirstlane(lds0 + buffer + (uint32_t)(wave + 4 * i) * 1024));
+    }
+  }
+};
+
+// The byte offset of a key's entry (an id the pool does not have reads page 0: nothing outside the pages is touched).
+__device__ __forceinline__ int64_t entry_at(const LatArgs& a, int page, int key) {
+  page = page < 0 || page >= a.num_pages ? 0 : page;
+  return ((int64_t)page * a.page_size + key % a.page_size) * a.width * 2;
+}
+
+__device__ __forceinline__ const int32_t* table_row(const LatArgs& a, int b) {
+  int slot = a.slots[b];
+  slot = slot < 0 ? 0 : (slot >= a.table_rows ? a.table_rows - 1 : slot);
+  return a.table + (int64_t)slot * a.table_stride;
+}
+
+// Prompt portions: a block of four waves owns 64 consecutive rows and walks the keys in stages of 32, the next stage on
+// its way into one buffer while the other is worked on. Blocks are dealt so that the one a block shares its compute unit
+// with (half a launch later) is its mirror image in length.
+template <int RP, int WP>
+__global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatArgs a) {
+  using EC = EntryCopies<WP, 32>;
+  constexpr int KS = WP / 32, DT = RP / 16, PG = 1024;
+  __shared__ __attribute__((aligned(1024))) unsigned char stage_lds[2 * EC::BYTES];
+  __shared__ int64_t from_s[2][32];
+  __shared__ int32_t pg_s[PG];
+  const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE, g = lane / 16, c = lane % 16;
+  const int b = a.row_ids[blockIdx.y];
+  const int qs = a.qstart[b], nq = a.qstart[b + 1] - qs, n = a.lens[b];
+  const int rows = nq * a.heads, tiles = (rows + 63) / 64, half = (tiles + 1) / 2, idx = blockIdx.x;
+  if (idx >= tiles || n <= 0) return;                    // (the same in all of the block's threads)
+  const int range = idx < half ? tiles - 1 - idx : idx - half;
+  const int32_t* trow = table_row(a, b);
+  for (int i = tid; i < min(PG, a.table_stride); i += 256) pg_s[i] = trow[i];
+  const int m0 = range * 64 + wave * 16, row = m0 + c;
+  const bool valid = row < rows;
+  const int ti = valid ? row / a.heads : 0, head = valid ? row % a.heads : 0, before = n - nq;
+  const int qpos = valid ? before + ti : -1;
+  const int wave_first = before + min(m0, rows - 1) / a.heads;
+  const int wave_last = m0 < rows ? before + (min(rows, m0 + 16) - 1) / a.heads : -1;
+  const int key_hi = before + (min(rows, range * 64 + 64) - 1) / a.heads, kb_last = key_hi / 32 * 32;
+  EC ec;
+  ec.init(stage_lds, a.width);
+  bf16x8_t qf[KS];
+  {
+    const bf16_t* qp = a.q + ((int64_t)(qs + ti) * a.heads + head) * a.width + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      if (valid && ks * 32 + 8 * g < a.width) qf[ks] = *reinterpret_cast<const bf16x8_t*>(qp + ks * 32);
+      else
+#pragma unroll
+        for (int i = 0; i < 8; ++i) qf[ks][i] = (__bf16)0.f;
+    }
+  }
+  f32x4_t o[DT];
+#pragma unroll
+  for (int d = 0; d < DT; ++d) o[d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+  lds_barrier();                                         // the block's table is in LDS
+  auto find = [&](int kb, int buf) {                     // where the entries of the stage at kb lie
+    if (tid < 32) {
+      const int key = min(kb + tid, n - 1), at = min(key / a.page_size, a.table_stride - 1);
+      from_s[buf][tid] = entry_at(a, at < PG ? pg_s[at] : trow[at], key);
+    }
+  };
+  find(0, 0);
+  find(32, 1);
+  lds_barrier();
+  ec.copy(a.pages, from_s[0], 0);
+  wait_loads_but<0>();
+  lds_barrier();
+  for (int kb = 0, buf = 0; kb <= kb_last; kb += 32, buf ^= 1) {
+    if (kb < kb_last) ec.copy(a.pages, from_s[buf ^ 1], (uint32_t)(buf ^ 1) * EC::BYTES);
+    if (kb + 32 < kb_last) find(kb + 64, buf);           // (this stage's own places have been read a stage ago)
+    if (kb <= wave_last) {
+      const unsigned char* lds = stage_lds + buf * EC::BYTES;
+      const unsigned char* kp = lds + c * EC::PITCH + g * 16;
+      f32x4_t s0 = f32x4_t{0.f, 0.f, 0.f, 0.f}, s1 = s0;
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const bf16x8_t k0 = *reinterpret_cast<const bf16x8_t*>(kp + ks * 64);
+        const bf16x8_t k1 = *reinterpret_cast<const bf16x8_t*>(kp + 16 * EC::PITCH + ks * 64);
+        s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qf[ks], s0, 0, 0, 0);
+        s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qf[ks], s1, 0, 0, 0);
+      }
+      float sv[8];
+#pragma unroll
+      for (int r = 0; r < 8; ++r) sv[r] = r < 4 ? s0[r] : s1[r - 4];
+      if (kb + 31 > wave_first) {
+#pragma unroll
+        for (int r = 0; r < 8; ++r)
+          if (kb + 16 * (r / 4) + 4 * g + r % 4 > qpos) sv[r] = -INFINITY;
+      }
+      float mx = fmaxf(fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3])), fmaxf(fmaxf(sv[4], sv[5]), fmaxf(sv[6], sv[7])));
+      mx = max_over_groups(mx);
+      const float m_new = fmaxf(m, mx * a.scale_log2);
+      const float m_use = m_new == -INFINITY ? 0.f : m_new;
+      bf16x8_t pb;
+      float psum = 0.f;
+#pragma unroll
+      for (int r = 0; r < 8; ++r) {
+        const float p = __builtin_amdgcn_exp2f(fmaf(sv[r], a.scale_log2, -m_use));
+        psum += p;
+        pb[r] = (__bf16)p;
+      }
+      if (__any(m_new != m)) {
+        const float alpha = __builtin_amdgcn_exp2f(m - m_use);
+        l *= alpha;
+#pragma unroll
+        for (int d = 0; d < DT; ++d) o[d] *= alpha;
+        m = m_new;
+      }
+      l += psum;
+      const unsigned char* vp = lds + (4 * g + c / 4) * EC::PITCH + (c % 4) * 8;
+#pragma unroll
+      for (int d = 0; d < DT; ++d) {
+        const bf16x4_t lo = read_transposed(vp + d * 32), hi = read_transposed(vp + 16 * EC::PITCH + d * 32);
+        const bf16x8_t v = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
+        o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pb, o[d], 0, 0, 0);
+      }
+    }
+    wait_loads_but<0>();                                 // the next stage has landed (this wave's share of it)
+    lds_barrier();
+  }
+  l += __shfl_xor(l, 16, WAVE);
+  l += __shfl_xor(l, 32, WAVE);
+  if (!valid) return;
+  if (a.sink) l += __builtin_amdgcn_exp2f(a.sink[head] * 1.4426950408889634f - m);
+  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  bf16_t* op = a.out + ((int64_t)(qs + ti) * a.heads + head) * a.kv_rank + 4 * g;
+#pragma unroll
+  for (int d = 0; d < DT; ++d) {
+    if (d * 16 + 4 * g >= a.kv_rank) break;
+    ushort4 w;
+    w.x = float_to_bf16(o[d][0] * inv);
+    w.y = float_to_bf16(o[d][1] * inv);
+    w.z = float_to_bf16(o[d][2] * inv);
+    w.w = float_to_bf16(o[d][3] * inv);
+    *reinterpret_cast<ushort4*>(op + d * 16) = w;
+  }
+}
+
+// Decode rows: a block of four waves takes a share of a row's keys for 16 heads, 64 keys at a time: wave w scores keys
+// 16 w .. 16 w + 15, the maxima and the weights meet in LDS, and wave w sums a quarter of the latent's columns over all 64.
+// One block a row writes the result; more leave (values, maximum, sum) for the merge below.
+template <int RP, int WP>
+__global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatArgs a) {
+  using EC = EntryCopies<WP, 64>;
+  constexpr int KS = WP / 32, DW = RP / 64;              // d-tiles of 16 a wave
+  __shared__ __attribute__((aligned(1024))) unsigned char tile_lds[EC::BYTES];
+  __shared__ int64_t from_s[64];
+  __shared__ float red_s[4][16];
+  __shared__ __attribute__((aligned(8))) bf16_t p_s[4][4][16][4];      // [wave][lane group][head][key of the four]
+  const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE, g = lane / 16, c = lane % 16;
+  const int b = a.row_ids[blockIdx.z], split = blockIdx.x, h0 = blockIdx.y * 16;
+  const int n = a.lens[b], token = a.qstart[b];
+  const int lo = split * a.per, hi = min(n, lo + a.per);             // keys lo .. hi - 1
+  const int head = h0 + c;
+  const bool valid = head < a.heads;
+  const int64_t cell = ((int64_t)blockIdx.z * a.heads + (valid ? head : 0)) * a.splits + split;
+  if (lo >= hi) {                                        // (the same in all of the block's threads) nothing of this row
+    if (a.splits > 1 && tid < 16 && valid) { a.part_ml[cell * 2] = -INFINITY; a.part_ml[cell * 2 + 1] = 0.f; }
+    return;
+  }
+  const int32_t* trow = table_row(a, b);
+  EC ec;
+  ec.init(tile_lds, a.width);
+  bf16x8_t qf[KS];
+  {
+    const bf16_t* qp = a.q + ((int64_t)token * a.heads + (valid ? head : 0)) * a.width + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      if (valid && ks * 32 + 8 * g < a.width) qf[ks] = *reinterpret_cast<const bf16x8_t*>(qp + ks * 32);
+      else
+#pragma unroll
+        for (int i = 0; i < 8; ++i) qf[ks][i] = (__bf16)0.f;
+    }
+  }
+  f32x4_t o[DW];
+#pragma unroll
+  for (int d = 0; d < DW; ++d) o[d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+  for (int kb = lo; kb < hi; kb += 64) {
+    if (tid < 64) {
+      const int key = min(kb + tid, hi - 1);
+      from_s[tid] = entry_at(a, trow[min(key / a.page_size, a.table_stride - 1)], key);
+    }
+    lds_barrier();                                       // (and every wave has left the tile before)
+    ec.copy(a.pages, from_s, 0);
+    wait_loads_but<0>();
+    lds_barrier();
+    const unsigned char* kp = tile_lds + (16 * wave + c) * EC::PITCH + g * 16;
+    f32x4_t s0 = f32x4_t{0.f, 0.f, 0.f, 0.f}, s1 = s0;
+#pragma unroll
+    for (int ks = 0; ks < KS; ks += 2) {
+      s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kp + ks * 64), qf[ks], s0, 0, 0, 0);
+      if (ks + 1 < KS)
+        s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kp + ks * 64 + 64),
+                                                     qf[ks + 1 < KS ? ks + 1 : 0], s1, 0, 0, 0);
+    }
+    float sv[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) sv[r] = kb + 16 * wave + 4 * g + r < hi ? s0[r] + s1[r] : -INFINITY;
+    const float mx = max_over_groups(fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3])));
+    if (g == 0) red_s[wave][c] = mx * a.scale_log2;
+    lds_barrier();
+    const float m_new = fmaxf(fmaxf(fmaxf(red_s[0][c], red_s[1][c]), fmaxf(red_s[2][c], red_s[3][c])), m);
+    const float alpha = __builtin_amdgcn_exp2f(m - m_new);           // (a tile holds at least one key: m_new is finite)
+    m = m_new;
+    l *= alpha;
+    ushort4 w;
+    float p[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) { p[r] = __builtin_amdgcn_exp2f(fmaf(sv[r], a.scale_log2, -m)); l += p[r]; }
+    w.x = float_to_bf16(p[0]); w.y = float_to_bf16(p[1]); w.z = float_to_bf16(p[2]); w.w = float_to_bf16(p[3]);
+    *reinterpret_cast<ushort4*>(&p_s[wave][g][c][0]) = w;
+#pragma unroll
+    for (int d = 0; d < DW; ++d) o[d] *= alpha;
+    lds_barrier();
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {                        // 32 keys: those of waves 2 j and 2 j + 1
+      const bf16x4_t plo = *reinterpret_cast<const bf16x4_t*>(&p_s[2 * j][g][c][0]);
+      const bf16x4_t phi = *reinterpret_cast<const bf16x4_t*>(&p_s[2 * j + 1][g][c][0]);
+      const bf16x8_t pb = __builtin_shufflevector(plo, phi, 0, 1, 2, 3, 4, 5, 6, 7);
+      const unsigned char* vp = tile_lds + (32 * j + 4 * g + c / 4) * EC::PITCH + (c % 4) * 8 + wave * DW * 32;
+#pragma unroll
+      for (int d = 0; d < DW; ++d) {
+        const bf16x4_t vlo = read_transposed(vp + d * 32), vhi = read_transposed(vp + 16 * EC::PITCH + d * 32);
+        o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_shufflevector(vlo, vhi, 0, 1, 2, 3, 4, 5, 6, 7), pb, o[d],
+                                                       0, 0, 0);
+      }
+    }
+  }
+  l += __shfl_xor(l, 16, WAVE);
+  l += __shfl_xor(l, 32, WAVE);
+  lds_barrier();                                         // every wave has read the last maxima
+  if (g == 0) red_s[wave][c] = l;
+  lds_barrier();
+  l = (red_s[0][c] + red_s[1][c]) + (red_s[2][c] + red_s[3][c]);
+  if (!valid) return;
+  const int d0 = wave * DW * 16 + 4 * g;
+  if (a.splits > 1) {
+    if (wave == 0 && g == 0) { a.part_ml[cell * 2] = m; a.part_ml[cell * 2 + 1] = l; }
+    float* op = a.part_o + cell * a.kv_rank + d0;
+#pragma unroll
+    for (int d = 0; d < DW; ++d)
+      if (d0 + d * 16 < a.kv_rank) *reinterpret_cast<f32x4_t*>(op + d * 16) = o[d];
+    return;
+  }
+  if (a.sink) l += __builtin_amdgcn_exp2f(a.sink[head] * 1.4426950408889634f - m);
+  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  bf16_t* op = a.out + ((int64_t)token * a.heads + head) * a.kv_rank + d0;
+#pragma unroll
+  for (int d = 0; d < DW; ++d) {
+    if (d0 + d * 16 >= a.kv_rank) break;
+    ushort4 w;
+    w.x = float_to_bf16(o[d][0] * inv);
+    w.y = float_to_bf16(o[d][1] * inv);
+    w.z = float_to_bf16(o[d][2] * inv);
+    w.w = float_to_bf16(o[d][3] * inv);
+    *reinterpret_cast<ushort4*>(op + d * 16) = w;
+  }
+}
+
+// out = sum_i 2^(m_i - M) o_i / sum_i 2^(m_i - M) l_i over a (decode row, head)'s splits (at most 64), the sink joining the
+// denominator. One block a (row, head): 128 threads take four columns each over the even splits, 128 over the odd ones.
+__global__ void __launch_bounds__(256) latent_merge_kernel(LatArgs a) {
+  __shared__ float f_s[64];
+  __shared__ float den_s;
+  __shared__ __attribute__((aligned(16))) float sum_s[LAT_MAX];
+  const int head = blockIdx.x, tid = threadIdx.x, b = a.row_ids[blockIdx.y];
+  const int64_t cell = ((int64_t)blockIdx.y * a.heads + head) * a.splits;
+  if (tid < WAVE) {
+    const float mi = tid < a.splits ? a.part_ml[(cell + tid) * 2] : -INFINITY;
+    const float li = tid < a.splits ? a.part_ml[(cell + tid) * 2 + 1] : 0.f;
+    const float top = wave_max(mi);
+    const float f = mi == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(mi - top);
+    f_s[tid] = f;
+    float den = wave_sum(f * li);
+    if (a.sink) den += __builtin_amdgcn_exp2f(a.sink[head] * 1.4426950408889634f - top);
+    if (tid == 0) den_s = den > 0.f ? 1.0f / den : 0.f;
+  }
+  __syncthreads();
+  const int side = tid / 128, d = (tid % 128) * 4;
+  for (int d4 = d; d4 < a.kv_rank; d4 += 512) {
+    f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
+    for (int i = side; i < a.splits; i += 2) {
+      const float f = f_s[i];                            // (a split that saw nothing has written no values: not read)
+      if (f != 0.f) acc += f * *reinterpret_cast<const f32x4_t*>(a.part_o + (cell + i) * a.kv_rank + d4);
+    }
+    if (side == 1) *reinterpret_cast<f32x4_t*>(&sum_s[d4]) = acc;
+    __syncthreads();
+    if (side == 0) {
+      acc += *reinterpret_cast<const f32x4_t*>(&sum_s[d4]);
+      const float inv = den_s;
+      ushort4 w;
+      w.x = float_to_bf16(acc[0] * inv); w.y = float_to_bf16(acc[1] * inv);
+      w.z = float_to_bf16(acc[2] * inv); w.w = float_to_bf16(acc[3] * inv);
+      *reinterpret_cast<ushort4*>(a.out + ((int64_t)a.qstart[b] * a.heads + head) * a.kv_rank + d4) = w;
+    }
+  }
+}
 }  // namespace
+
+#define LAT_BY_SIZE(CALL)                                                                            \
+  do {                                                                                               \
+    if (kv_rank <= 64 && width <= 96) { constexpr int RP = 64, WP = 96; CALL; }                      \
+    else if (kv_rank <= 128 && width <= 160) { constexpr int RP = 128, WP = 160; CALL; }             \
+    else if (kv_rank <= 192 && width <= 256) { constexpr int RP = 192, WP = 256; CALL; }             \
+    else if (kv_rank <= 256 && width <= 320) { constexpr int RP = 256, WP = 320; CALL; }             \
+    else { constexpr int RP = 512, WP = 576; CALL; }                                                 \
+  } while (0)
+
+// Whether the matrix-core kernels serve bfloat16 entries of these sizes.
+extern "C" int holon_latent_cores_supported(int width, int kv_rank) {
+  return kv_rank > 0 && kv_rank % 4 == 0 && kv_rank <= 512 && width % 8 == 0 && width >= kv_rank && width <= 576;
+}
+
+static int latent_cores_check(const char* what, int rows, int heads, int width, int kv_rank, int page_size, int num_pages,
+                              int table_stride, int table_rows, float scale) {
+  HOLON_CHECK(holon_latent_cores_supported(width, kv_rank), "%s: entries of %d (multiples of 8 up to 576) with latents of %d "
+              "(multiples of 4 up to 512)", what, width, kv_rank);
+  HOLON_CHECK(rows >= 0 && rows <= 65535 && heads > 0 && page_size > 0 && num_pages > 0 && table_stride > 0 && table_rows > 0 &&
+                  scale > 0.f, "%s: %d rows of %d heads, pages of %d, scale %g", what, rows, heads, page_size, scale);
+  return 0;
+}
+
+extern "C" int holon_latent_prefill_bf16(const void* q, void* out, const void* pages, const int32_t* table,
+                                         int table_stride, int table_rows, const int32_t* slots, const int32_t* lens,
+                                         const int32_t* qstart, const int32_t* row_ids, int rows, int max_query, int heads,
+                                         int width, int kv_rank, int page_size, int num_pages, const float* sink,
+                                         float scale, void* stream) {
+  if (latent_cores_check("latent_prefill", rows, heads, width, kv_rank, page_size, num_pages, table_stride, table_rows, scale))
+    return -1;
+  HOLON_CHECK(max_query > 0 && (int64_t)max_query * heads <= 0x7fffffff - 64, "latent_prefill: %d tokens of %d heads", max_query,
+              heads);
+  if (rows == 0) return 0;
+  LatArgs a{(const bf16_t*)q, (bf16_t*)out, (const bf16_t*)pages, table, slots, lens, qstart, row_ids, sink, nullptr, nullptr,
+            table_stride, table_rows, num_pages, page_size, heads, width, kv_rank, 0, 1, scale * 1.4426950408889634f};
+  const dim3 grid((max_query * heads + 63) / 64, rows);
+  LAT_BY_SIZE((latent_prefill_kernel<RP, WP><<<grid, 256, 0, (hipStream_t)stream>>>(a)));
+  HOLON_LAUNCH_OK();
+  return 0;
+}
+
+extern "C" int holon_latent_decode_bf16(const void* q, void* out, const void* pages, const int32_t* table,
+                                        int table_stride, int table_rows, const int32_t* slots, const int32_t* lens,
+                                        const int32_t* qstart, const int32_t* row_ids, int rows, int max_len, int heads,
+                                        int width, int kv_rank, int page_size, int num_pages, const float* sink,
+                                        float scale, int splits, int per, float* part_o, float* part_ml, void* stream) {
+  if (latent_cores_check("latent_decode", rows, heads, width, kv_rank, page_size, num_pages, table_stride, table_rows, scale))
+    return -1;
+  HOLON_CHECK(splits >= 1 && splits <= 64 && per > 0 && per % 64 == 0 && (int64_t)splits * per >= max_len &&
+                  (splits == 1 || (part_o && part_ml)),
+              "latent_decode: %d shares of %d keys for rows of up to %d", splits, per, max_len);
+  if (rows == 0) return 0;
+  LatArgs a{(const bf16_t*)q, (bf16_t*)out, (const bf16_t*)pages, table, slots, lens, qstart, row_ids, sink, part_o, part_ml,
+            table_stride, table_rows, num_pages, page_size, heads, width, kv_rank, per, splits, scale * 1.4426950408889634f};
+  const dim3 grid(splits, (heads + 15) / 16, rows);
+  LAT_BY_SIZE((latent_decode_kernel<RP, WP><<<grid, 256, 0, (hipStream_t)stream>>>(a)));
+  HOLON_LAUNCH_OK();
+  if (splits > 1) {
+    latent_merge_kernel<<<dim3(heads, rows), 256, 0, (hipStream_t)stream>>>(a);
+    HOLON_LAUNCH_OK();
+  }
+  return 0;
+}
 
 extern "C" int holon_latent_attention(const void* q, void* out, const void* pages, const int32_t* table,
                                       int table_stride, int table_rows, const int32_t* slots, const int32_t* token_row,

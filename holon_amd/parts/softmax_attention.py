@@ -265,6 +265,20 @@ def latent_attention_plain(q, pages, table, rows, token_row, positions, kv_rank,
     return out.to(q.dtype)
 
 
+def latent_on_cores(width: int, kv_rank: int) -> bool:
+    """Whether the matrix-core kernels serve bfloat16 entries of `width` values with latents of `kv_rank` (what the library's
+    `holon_latent_cores_supported` answers)."""
+    return 0 < kv_rank <= 512 and kv_rank % 4 == 0 and width % 8 == 0 and kv_rank <= width <= 576
+
+
+def latent_splits(pairs: int, span: int, blocks: int = 256) -> tuple[int, int]:
+    """How a decode row's keys are cut over blocks: (shares, keys a share, a multiple of 64). `pairs`: (row, 16 heads) in the
+    launch, which is to have about `blocks` blocks; at most 64 shares."""
+    tiles = max(1, -(-span // 64))
+    per = -(-tiles // max(1, min(64, tiles, blocks // max(1, pairs))))
+    return -(-tiles // per), per * 64
+
+
 def _latent_attention_hip(launch, q, pages, table, rows, token_row, positions, kv_rank, page_size, sink, scale, window):
     t, heads, width = q.shape
     ok = q.is_cuda and q.is_contiguous() and q.dtype in _DT and pages.dtype == q.dtype and pages.is_contiguous() \
@@ -274,9 +288,25 @@ def _latent_attention_hip(launch, q, pages, table, rows, token_row, positions, k
     if not ok:
         raise ValueError(f"latent_attention: q {tuple(q.shape)} {q.dtype}, pages {tuple(pages.shape)} do not fit entries of "
                          f"{width} with latents of {kv_rank}, page {page_size}")
+    general, prefill, decode = launch
     out = torch.empty((t, heads, kv_rank), dtype=q.dtype, device=q.device)
+    if q.dtype == torch.bfloat16 and window == 0 and scale > 0 and latent_on_cores(width, kv_rank):
+        common = (q.data_ptr(), out.data_ptr(), pages.data_ptr(), table.data_ptr(), table.shape[1], table.shape[0],
+                  rows.slots.data_ptr(), rows.lens.data_ptr(), rows.query_start.data_ptr())
+        sizes = (heads, width, kv_rank, page_size, pages.shape[0], _ptr(sink), float(scale))
+        if rows.n_chunk:
+            prefill(*common, rows.chunk_rows.data_ptr(), rows.n_chunk, rows.max_chunk_query, *sizes)
+        if rows.n_decode:
+            splits, per = latent_splits(rows.n_decode * (-(-heads // 16)), rows.max_decode_len)
+            parts = (None, None)
+            if splits > 1:
+                parts = (torch.empty((rows.n_decode * heads * splits * kv_rank,), dtype=torch.float32, device=q.device),
+                         torch.empty((rows.n_decode * heads * splits * 2,), dtype=torch.float32, device=q.device))
+            decode(*common, rows.decode_rows.data_ptr(), rows.n_decode, rows.max_decode_len, *sizes, splits, per,
+                   _ptr(parts[0]), _ptr(parts[1]))
+        return out
     if t:
-        launch(q.data_ptr(), out.data_ptr(), pages.data_ptr(), table.data_ptr(), table.shape[1], table.shape[0],
+        general(q.data_ptr(), out.data_ptr(), pages.data_ptr(), table.data_ptr(), table.shape[1], table.shape[0],
                rows.slots.data_ptr(), token_row.data_ptr(), positions.data_ptr(), t, heads, width, kv_rank, page_size,
                pages.shape[0], _ptr(sink), float(scale), int(window), _DT[q.dtype])
     return out
@@ -360,9 +390,11 @@ register_kernel(KernelOp("whole_norm_prepare", whole_norm_prepare_plain, "holon_
 register_kernel(KernelOp("latent_rope_prepare", latent_rope_prepare_plain, "holon_latent_rope_prepare",
                          [_P, _I, _I, _I, _I, _I, _I, _P, _F, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I],
                          _latent_rope_prepare_hip))
-register_kernel(KernelOp("latent_attention", latent_attention_plain, "holon_latent_attention",
-                         [_P, _P, _P, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _F, _I, _I],
-                         _latent_attention_hip))
+_CORES = [_P, _P, _P, _P, _I, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _F]
+register_kernel(KernelOp("latent_attention", latent_attention_plain,
+                         ("holon_latent_attention", "holon_latent_prefill_bf16", "holon_latent_decode_bf16"),
+                         ([_P, _P, _P, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _F, _I, _I], _CORES,
+                          _CORES + [_I, _I, _P, _P]), _latent_attention_hip))
 register_kernel(KernelOp("latent_prepare", latent_prepare_plain, "holon_latent_prepare",
                          [_P, _I, _I, _I, _P, _P, _F, _P, _P, _P, _P, _I, _I, _I], _latent_prepare_hip))
 register_kernel(KernelOp("head_gate", head_gate_plain, "holon_head_gate", [_P, _P, _L, _L, _I, _I, _I], _head_gate_hip))

@@ -602,3 +602,62 @@ def test_kernels_alone_against_their_plain_forms(dtype):
         only_q = both[:, : heads * (dim + rot)].contiguous()
         c = k.latent_rope_prepare(only_q, heads, dim, rot, rank, None, 0.0, tab, positions, None, None, None, page)
         assert torch.equal(c[0], a[0]) and torch.equal(c[1][..., rank:], a[1][..., rank:]), "queries alone"
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("rank,rot", [(128, 16), (96, 32), (512, 64), (192, 64), (40, 24), (256, 64), (60, 4), (384, 64)])
+def test_latent_entries_on_the_gpu(rank, rot):
+    """Attention over entries kept once: in bfloat16 the matrix-core prompt and decode kernels, in both types the general
+    kernel, prompt portions beside decode rows over scattered pages, head counts that fill tiles of 16 and that do not, a
+    row of every length around a tile's border, with and without a sink, against float64."""
+    import holon_amd.parts  # noqa: F401
+    from holon_amd.kernels import load_hip
+    from holon_amd.kernels.api import AttnRows
+    from holon_amd.kernels.registry import kernel_op
+    from holon_amd.parts.softmax_attention import latent_on_cores
+    k, dev, width = load_hip(), "cuda", rank + rot
+    assert latent_on_cores(width, rank) == bool(k.lib.holon_latent_cores_supported(width, rank))
+    g = torch.Generator().manual_seed(rank)
+    lens, counts = [300, 75, 190, 3, 129, 1, 40, 64, 65, 700, 31], [300, 1, 60, 3, 1, 1, 2, 1, 1, 1, 31]
+    qstart = [0]
+    for c in counts:
+        qstart.append(qstart[-1] + c)
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=dev)          # noqa: E731
+    decode = [b for b, c in enumerate(counts) if c == 1]
+    chunk = [b for b, c in enumerate(counts) if c > 1]
+    rows = AttnRows(slots=i32(list(range(len(lens)))), lens=i32(lens), query_start=i32(qstart), decode_rows=i32(decode),
+                    chunk_rows=i32(chunk), n_decode=len(decode), n_chunk=len(chunk),
+                    max_decode_len=max(lens[b] for b in decode), max_chunk_query=max(counts),
+                    max_chunk_len=max(lens[b] for b in chunk))
+    token_row = torch.cat([torch.full((c,), b, dtype=torch.int32) for b, c in enumerate(counts)]).to(dev)
+    positions = torch.cat([torch.arange(n - c, n, dtype=torch.int32) for n, c in zip(lens, counts)]).to(dev)
+    op = kernel_op("latent_attention").plain
+    for heads, page in ((16, 16), (3, 16), (20, 32), (1, 8), (8, 64)):
+        n_pages = sum(-(-n // page) for n in lens) + 1
+        table = torch.full((len(lens) + 1, 96), n_pages - 1, dtype=torch.int32)
+        order, at = torch.randperm(n_pages - 1, generator=g).tolist(), 0
+        for s_, n in enumerate(lens):
+            for i in range(-(-n // page)):
+                table[s_, i] = order[at]
+                at += 1
+        table = table.to(dev)
+        pages = torch.randn(n_pages, page * width, generator=g).to(dev).bfloat16()
+        for s_, n in enumerate(lens):              # what lies behind a row's last token in its page must not be read
+            if n % page:
+                pages.view(n_pages, page, width)[int(table[s_, n // page]), n % page:] = float("nan")
+        pages.view(n_pages, page, width)[n_pages - 1] = float("nan")
+        q = (torch.randn(qstart[-1], heads, width, generator=g) * 2.5 * width ** -0.5).to(dev).bfloat16()
+        sinks = [None, torch.randn(heads, generator=g).to(dev)]
+        for sink in sinks[: 2 if heads in (3, 16) else 1]:
+            args = (table, rows, token_row, positions, rank, page)
+            want = op(q.double(), pages.double(), *args, None if sink is None else sink.double(), 0.9, 0)
+            for what, got, tol in (("cores", k.latent_attention(q, pages, *args, sink, 0.9, 0), 6e-3),
+                                   ("general", k.latent_attention(q, pages, *args, sink, 0.9, 4096), 6e-3),
+                                   ("float32", k.latent_attention(q.float(), pages.float(), *args, sink, 0.9, 0), 2e-6)):
+                assert torch.isfinite(got).all(), (heads, page, what)
+                assert H.rel_rms(got, want) < tol, (heads, page, what)
+                per = ((got.double() - want).square().mean((1, 2)).sqrt() / want.square().mean((1, 2)).sqrt()).max().item()
+                assert per < 5 * tol, (heads, page, what, per)
+    window = 33                                    # a window: the general kernel
+    got = k.latent_attention(q, pages, table, rows, token_row, positions, rank, page, None, 0.9, window)
+    assert H.rel_rms(got, op(q.double(), pages.double(), table, rows, token_row, positions, rank, page, None, 0.9, window)) < 6e-3
