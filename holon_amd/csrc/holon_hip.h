@@ -351,6 +351,10 @@ int holon_latent_prepare(const void* both, int tokens, int q_rank, int kv_rank, 
 int holon_head_linear_rows(const void* x, const void* w, void* y, int rows, int heads, int A, int B, int y_head,
                            int dtype, const void* gate, int64_t gate_stride, void* stream);
 
+// The same for bfloat16 on the matrix cores, any number of rows (A a multiple of 8; latent_attention.hip).
+int holon_head_linear_bf16(const void* x, const void* w, void* y, int rows, int heads, int A, int B, int y_head,
+                           const void* gate, int64_t gate_stride, void* stream);
+
 // -- a block of two sublayers over one float32 stream (parallel_block.hip) ----------------------------------------------
 // x32 [rows, dim] += (d1 + d2) + row in place (each nullable; d1, d2 float32 or bfloat16 by dt1, dt2; row [dim] float32);
 // then, with w1 and y1: y1 = x rsqrt(mean(x^2) + eps) w1, and with w2 and y2 the same rows with w2 (weights of dtype dtw,

@@ -492,7 +492,118 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(LatArgs a) {
     }
   }
 }
+
+// -- every head's own projection ------------------------------------------------------------------------------------------
+// y[t, h, b] = sum_a x[t, h, a] w[h, b, a], bfloat16 operands, float32 sums, one rounding; with `gate` the sum times
+// sigmoid(gate[t, h B + b]) first. A = 16 rows of w x 32, B = 32 x 16 tokens: a lane holds four neighbouring results of a
+// token. Loads past A or B read zeros or a row that is there.
+struct HeadLinear {
+  const bf16_t* x;
+  const bf16_t* w;
+  bf16_t* y;
+  const bf16_t* gate;
+  int64_t gate_stride;
+  int rows, heads, A, B, y_head, wide_out;
+};
+
+__device__ __forceinline__ bf16x8_t load_piece(const bf16_t* p, bool ok) {
+  bf16x8_t v;
+  if (ok) return *reinterpret_cast<const bf16x8_t*>(p);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = (__bf16)0.f;
+  return v;
+}
+
+__device__ __forceinline__ void head_linear_store(const HeadLinear& a, int t, int h, int b, f32x4_t v) {
+  if (t >= a.rows || b >= a.B) return;
+  if (a.gate) {
+    const bf16_t* gp = a.gate + t * a.gate_stride + (int64_t)h * a.B + b;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (b + r < a.B) v[r] *= __builtin_amdgcn_rcpf(1.0f + __expf(-bf16_to_float(gp[r])));
+  }
+  bf16_t* yp = a.y + ((int64_t)t * a.heads + h) * a.y_head + b;
+  if (a.wide_out && b + 3 < a.B) {
+    ushort4 o;
+    o.x = float_to_bf16(v[0]); o.y = float_to_bf16(v[1]); o.z = float_to_bf16(v[2]); o.w = float_to_bf16(v[3]);
+    *reinterpret_cast<ushort4*>(yp) = o;
+  } else {
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (b + r < a.B) yp[r] = float_to_bf16(v[r]);
+  }
+}
+
+// Up to 16 tokens: a block a head and 16 columns, A dealt to its four waves in steps of 32, their sums added in wave order.
+__global__ void __launch_bounds__(256) head_linear_few_kernel(HeadLinear a) {
+  __shared__ f32x4_t sum_s[3][WAVE];
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, g = lane / 16, c = lane % 16;
+  const int h = blockIdx.x, b0 = blockIdx.y * 16;
+  const bf16_t* wp = a.w + ((int64_t)h * a.B + min(b0 + c, a.B - 1)) * a.A + 8 * g;
+  const bf16_t* xp = a.x + ((int64_t)min(c, a.rows - 1) * a.heads + h) * a.A + 8 * g;
+  f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k = wave * 32; k < a.A; k += 128) {
+    const bool ok = k + 8 * g < a.A;
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(load_piece(wp + k, ok), load_piece(xp + k, ok), acc, 0, 0, 0);
+  }
+  if (wave > 0) sum_s[wave - 1][lane] = acc;
+  __syncthreads();
+  if (wave > 0) return;
+  acc = ((acc + sum_s[0][lane]) + sum_s[1][lane]) + sum_s[2][lane];
+  head_linear_store(a, c, h, b0 + 4 * g, acc);
+}
+
+// More tokens: a block 64 tokens and 128 columns of a head, a wave 32 of the columns.
+__global__ void __launch_bounds__(256) head_linear_many_kernel(HeadLinear a) {
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, g = lane / 16, c = lane % 16;
+  const int h = blockIdx.y, t0 = blockIdx.x * 64, b0 = blockIdx.z * 128 + wave * 32;
+  if (b0 >= a.B) return;
+  const bf16_t* wp[2];
+  const bf16_t* xp[4];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) wp[i] = a.w + ((int64_t)h * a.B + min(b0 + 16 * i + c, a.B - 1)) * a.A + 8 * g;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) xp[j] = a.x + ((int64_t)min(t0 + 16 * j + c, a.rows - 1) * a.heads + h) * a.A + 8 * g;
+  f32x4_t acc[2][4];
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+  for (int k = 0; k < a.A; k += 32) {
+    const bool ok = k + 8 * g < a.A;
+    bf16x8_t wf[2], xf[4];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) wf[i] = load_piece(wp[i] + k, ok);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) xf[j] = load_piece(xp[j] + k, ok);
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], xf[j], acc[i][j], 0, 0, 0);
+  }
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) head_linear_store(a, t0 + 16 * j + c, h, b0 + 16 * i + 4 * g, acc[i][j]);
+}
 }  // namespace
+
+// The per-head projection of bfloat16 rows, any number of them (A a multiple of 8, operands on 16-byte borders).
+extern "C" int holon_head_linear_bf16(const void* x, const void* w, void* y, int rows, int heads, int A, int B, int y_head,
+                                      const void* gate, int64_t gate_stride, void* stream) {
+  HOLON_CHECK(rows >= 1 && heads > 0 && heads <= 65535 && A > 0 && A % 8 == 0 && B > 0 && B <= 65535 * 16 && y_head >= B &&
+                  (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0,
+              "head_linear: %d rows, %d heads of %d (a multiple of 8) -> %d (in steps of %d)", rows, heads, A, B, y_head);
+  const HeadLinear a{(const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, (const bf16_t*)gate, gate_stride, rows, heads, A, B, y_head,
+                     (int)(y_head % 4 == 0 && (uintptr_t)y % 8 == 0)};
+  hipStream_t s = (hipStream_t)stream;
+  if (rows <= 16) head_linear_few_kernel<<<dim3(heads, (B + 15) / 16), 256, 0, s>>>(a);
+  else head_linear_many_kernel<<<dim3((rows + 63) / 64, heads, (B + 127) / 128), 256, 0, s>>>(a);
+  HOLON_LAUNCH_OK();
+  return 0;
+}
 
 #define LAT_BY_SIZE(CALL)                                                                            \
   do {                                                                                               \

@@ -103,6 +103,74 @@ __global__ void __launch_bounds__(256) causal_conv_wide_kernel(const T* __restri
   *reinterpret_cast<uint4*>(y + (int64_t)t * channels + c) = out;
 }
 
+// The same for up to four taps with a thread taking RUN neighbouring tokens: its channels' taps are read once, as whole
+// vectors, and an input serves every token of the run that it reaches. Tokens of a run may belong to different rows; an
+// input in front of its row's first token comes from the row's slot.
+template <typename T, int TAPS>
+__global__ void __launch_bounds__(256) causal_conv_run_kernel(const T* __restrict__ x, int64_t x_stride,
+                                                              const T* __restrict__ w, const T* __restrict__ bias,
+                                                              const T* __restrict__ state, T* __restrict__ y,
+                                                              const int32_t* __restrict__ slots,
+                                                              const int32_t* __restrict__ starts,
+                                                              const int32_t* __restrict__ query_start,
+                                                              const int32_t* __restrict__ token_row, int tokens,
+                                                              int channels, int add_input, int act, int ring) {
+  constexpr int N = Elem<T>::kVec, RUN = 8;
+  const int c = (blockIdx.x * blockDim.x + threadIdx.x) * N, t0 = blockIdx.y * RUN;
+  if (c >= channels) return;
+  uint4 win[RUN + TAPS - 1];                             // the inputs of tokens t0 - TAPS + 1 .. t0 + RUN - 1
+#pragma unroll
+  for (int e = 0; e < RUN + TAPS - 1; ++e) {
+    const int t = t0 - (TAPS - 1) + e;
+    win[e] = t >= 0 && t < tokens ? *reinterpret_cast<const uint4*>(x + t * x_stride + c) : make_uint4(0u, 0u, 0u, 0u);
+  }
+  float wv[N * TAPS], bv[N];
+#pragma unroll
+  for (int e = 0; e < TAPS; ++e) {                       // (N TAPS values are TAPS whole vectors)
+    const uint4 raw = *reinterpret_cast<const uint4*>(w + (int64_t)c * TAPS + e * N);
+    const T* v = reinterpret_cast<const T*>(&raw);
+#pragma unroll
+    for (int u = 0; u < N; ++u) wv[e * N + u] = Elem<T>::load(v[u]);
+  }
+#pragma unroll
+  for (int u = 0; u < N; ++u) bv[u] = bias ? Elem<T>::load(bias[c + u]) : 0.f;
+#pragma unroll
+  for (int r = 0; r < RUN; ++r) {
+    const int t = t0 + r;
+    if (t >= tokens) break;
+    const int b = token_row[t], i = t - query_start[b];
+    float acc[N];
+#pragma unroll
+    for (int u = 0; u < N; ++u) acc[u] = 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      const int l = i - (TAPS - 1) + j;
+      uint4 raw = win[r + j];
+      if (l < 0) {
+        const int start = starts[b];
+        raw = make_uint4(0u, 0u, 0u, 0u);
+        if (start > 0 && (!ring || start + l >= 0))
+          raw = *reinterpret_cast<const uint4*>(state + ((int64_t)slots[b] * (ring ? TAPS : TAPS - 1) +
+                                                         (ring ? (start + l) % TAPS : TAPS - 1 + l)) * channels + c);
+      }
+      const T* v = reinterpret_cast<const T*>(&raw);
+#pragma unroll
+      for (int u = 0; u < N; ++u) acc[u] += wv[u * TAPS + j] * Elem<T>::load(v[u]);
+    }
+    const T* own = reinterpret_cast<const T*>(&win[r + TAPS - 1]);
+    uint4 out;
+    T* o = reinterpret_cast<T*>(&out);
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+      float a = bias ? acc[u] + bv[u] : acc[u];
+      if (add_input) a += Elem<T>::load(own[u]);
+      if (act) a = silu<T>(a);
+      o[u] = Elem<T>::store(a);
+    }
+    *reinterpret_cast<uint4*>(y + (int64_t)t * channels + c) = out;
+  }
+}
+
 // After the filter has read the old inputs: the slot takes the row's last taps - 1 inputs, oldest first. A thread
 // moves its channel's entries in ascending order and reads only entries at or behind the one it writes. (A ring takes the
 // row's own last inputs at their places; older ones lie where they are.)
@@ -663,8 +731,17 @@ extern "C" int holon_causal_conv(const void* x, int64_t x_stride, const void* w,
   const int vec = dtype == HOLON_F32 ? 4 : 8;
   if (!rows_in_order && channels % vec == 0 && x_stride % vec == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0 &&
       (uintptr_t)state % 16 == 0) {
-    const dim3 grid_w((channels / vec + 255) / 256, tokens);
-    BY_DTYPE(dtype, (causal_conv_wide_kernel<T><<<grid_w, block, 0, s>>>((const T*)x, x_stride, (const T*)w,
+    const dim3 grid_w((channels / vec + 255) / 256, tokens), grid_r((channels / vec + 255) / 256, (tokens + 7) / 8);
+#define CONV_RUN(K)                                                                                                    \
+  BY_DTYPE(dtype, (causal_conv_run_kernel<T, K><<<grid_r, block, 0, s>>>((const T*)x, x_stride, (const T*)w,           \
+                                                                         (const T*)bias, (const T*)state, (T*)y, slots, \
+                                                                         starts, query_start, token_row, tokens,       \
+                                                                         channels, add_input, act, ring)))
+    const bool whole_taps = (uintptr_t)w % 16 == 0;
+    if (whole_taps && taps == 2) CONV_RUN(2);
+    else if (whole_taps && taps == 3) CONV_RUN(3);
+    else if (whole_taps && taps == 4) CONV_RUN(4);
+    else BY_DTYPE(dtype, (causal_conv_wide_kernel<T><<<grid_w, block, 0, s>>>((const T*)x, x_stride, (const T*)w,
                                                                          (const T*)bias, (const T*)state, (T*)y,
                                                                          slots, starts, query_start, token_row,
                                                                          channels, taps, add_input, act, ring)));

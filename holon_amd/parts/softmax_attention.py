@@ -112,8 +112,9 @@ def head_linear_plain(x, weight, out=None, gate=None):
 
 
 def _head_linear_hip(launch, x, weight, out=None, gate=None):
-    """Steps of up to 16 rows: this package's kernel (the weights stream once, no copy of the result); more rows: the
-    vendor library's batched product."""
+    """bfloat16: this package's matrix-core kernels. Else steps of up to 16 rows take a kernel of its own (the weights
+    stream once, no copy of the result), more rows the vendor library's batched product."""
+    few, cores = launch
     t, heads, a = x.shape
     b = weight.shape[1]
     if not (x.is_cuda and x.is_contiguous() and weight.is_contiguous() and weight.dtype == x.dtype and x.dtype in _DT
@@ -125,11 +126,15 @@ def _head_linear_hip(launch, x, weight, out=None, gate=None):
     if gate is not None and not (gate.is_cuda and gate.dtype == x.dtype and gate.shape == (t, heads * b)
                                  and gate.stride(1) == 1):
         raise ValueError(f"head_linear: gates {tuple(gate.shape)} {gate.dtype} for {t} rows of {heads} heads of {b}")
+    gates = (_ptr(gate), gate.stride(0) if gate is not None else 0)
+    if x.dtype == torch.bfloat16 and t and a % 8 == 0 and x.data_ptr() % 16 == 0 and weight.data_ptr() % 16 == 0:
+        y = out if out is not None else torch.empty((t, heads, b), dtype=x.dtype, device=x.device)
+        cores(x.data_ptr(), weight.data_ptr(), y.data_ptr(), t, heads, a, b, y.stride(1), *gates)
+        return y
     if not 1 <= t <= 16 or t * a * 4 > 48 * 1024:
         return head_linear_plain(x, weight, out, gate)
     y = out if out is not None else torch.empty((t, heads, b), dtype=x.dtype, device=x.device)
-    launch(x.data_ptr(), weight.data_ptr(), y.data_ptr(), t, heads, a, b, y.stride(1), _DT[x.dtype], _ptr(gate),
-           gate.stride(0) if gate is not None else 0)
+    few(x.data_ptr(), weight.data_ptr(), y.data_ptr(), t, heads, a, b, y.stride(1), _DT[x.dtype], *gates)
     return y
 
 
@@ -383,8 +388,9 @@ def _add_bias_hip(launch, x, bias):
 register_kernel(KernelOp("softmax_attention", softmax_attention_plain, "holon_softmax_attention",
                          [_P, _P, _P, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _F, _I, _I, _F, _P, _P, _I, _I],
                          _softmax_attention_hip))
-register_kernel(KernelOp("head_linear", head_linear_plain, "holon_head_linear_rows",
-                         [_P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _L], _head_linear_hip))
+register_kernel(KernelOp("head_linear", head_linear_plain, ("holon_head_linear_rows", "holon_head_linear_bf16"),
+                         ([_P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _L], [_P, _P, _P, _I, _I, _I, _I, _I, _P, _L]),
+                         _head_linear_hip))
 register_kernel(KernelOp("whole_norm_prepare", whole_norm_prepare_plain, "holon_whole_norm_prepare",
                          [_P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _P, _P, _P, _I, _I, _I], _whole_norm_prepare_hip))
 register_kernel(KernelOp("latent_rope_prepare", latent_rope_prepare_plain, "holon_latent_rope_prepare",
