@@ -127,7 +127,7 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(
 // So an entry lies in memory once and in LDS once, and serves both products from there.
 // Entries come into LDS by the memory pipeline (16 bytes a lane, a wave's 64 lanes into one contiguous kilobyte). A row's
 // pitch in LDS is WP / 2 + 8 words, 8 times an odd number: eight neighbouring rows then start 8 banks apart, which keeps
-// the transposed reads and the row reads free of conflicts. A row's columns from `width` on repeat its first ones (the
+// the transposed reads and the row reads free of conflicts. A row's columns from `width` on repeat its last ones (the
 // query is zero there); rows past the last key repeat the last key's entry (their weights are zero).
 // RP, WP: the latent's and the entry's widths, padded to the next sizes that are compiled.
 struct LatArgs {
@@ -161,34 +161,33 @@ __device__ __forceinline__ float max_over_groups(float v) {   // over the four l
   return fmaxf(__uint_as_float(halves[0]), __uint_as_float(halves[1]));
 }
 
-// KEYS entries on their way into one buffer: what each lane of a block of four waves copies.
-template <int WP, int KEYS>
+// KEYS entries on their way into one buffer: what each lane of a block of WAVES waves copies.
+template <int WP, int KEYS, int WAVES>
 struct EntryCopies {
   static constexpr int PC = WP / 8 + 2;                  // 16-byte pieces a row takes in LDS
-  static constexpr int PITCH = PC * 16, BYTES = KEYS * PITCH, NI = KEYS * PC / 64, CI = (NI + 3) / 4;
+  static constexpr int PITCH = PC * 16, BYTES = KEYS * PITCH, NI = KEYS * PC / 64, CI = (NI + WAVES - 1) / WAVES;
   static_assert(KEYS * PC % 64 == 0 && (PC / 2) % 2 == 1, "whole kilobytes, an odd multiple of 8 words a row");
-  int row[CI];                                           // the row a piece belongs to, and its place in the entry
-  uint32_t col[CI];
   uint32_t lds0;
-  int wave;
+  int wave, row0, col0, last;                            // of this lane's first piece; the entry's last piece
   __device__ __forceinline__ void init(const unsigned char* lds, int width) {
     wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
     lds0 = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void*)lds;
-    const int pieces = width / 8;
-#pragma unroll
-    for (int i = 0; i < CI; ++i) {
-      const int at = (wave + 4 * i) * 64 + threadIdx.x % WAVE, c = at % PC;
-      row[i] = min(at / PC, KEYS - 1);
-      col[i] = (uint32_t)(c < pieces ? c : c % pieces) * 16;
-    }
+    row0 = threadIdx.x / PC;
+    col0 = threadIdx.x % PC;
+    last = width / 8 - 1;
   }
-  // `from`: the byte offset of every row's entry among the pages, in LDS
+  // `from`: the byte offset of every row's entry among the pages, in LDS. (A lane's pieces are WAVES x 64 apart: its next row and
+  // column are found as it goes, which costs less than registers held through the kernel.)
   __device__ __forceinline__ void copy(const bf16_t* pages, const int64_t* from, uint32_t buffer) const {
+    int row = row0, col = col0;
 #pragma unroll
     for (int i = 0; i < CI; ++i) {
-      if (wave + 4 * i >= NI) break;                     // (the same in all of a wave's lanes)
-      load_to_lds16_from(reinterpret_cast<const unsigned char*>(pages) + from[row[i]] + col[i],
-                         __builtin_amdgcn_readfirstlane(lds0 + buffer + (uint32_t)(wave + 4 * i) * 1024));
+      if (wave + WAVES * i >= NI) break;                     // (the same in all of a wave's lanes)
+      load_to_lds16_from(reinterpret_cast<const unsigned char*>(pages) + from[row] + min(col, last) * 16,
+                         __builtin_amdgcn_readfirstlane(lds0 + buffer + (uint32_t)(wave + WAVES * i) * 1024));
+      row += WAVES * 64 / PC;
+      col += WAVES * 64 % PC;
+      if (col >= PC) { col -= PC; ++row; }
     }
   }
 };
@@ -205,31 +204,35 @@ __device__ __forceinline__ const int32_t* table_row(const LatArgs& a, int b) {
   return a.table + (int64_t)slot * a.table_stride;
 }
 
-// Prompt portions: a block of four waves owns 64 consecutive rows and walks the keys in stages of 32, the next stage on
-// its way into one buffer while the other is worked on. Blocks are dealt so that the one a block shares its compute unit
-// with (half a launch later) is its mirror image in length.
+// Prompt portions: a block of eight waves owns 64 consecutive rows (four tiles) and walks the keys in stages of 32, the
+// next stage on its way into one buffer while the other is worked on. Wave w scores tile w / 2 against half w % 2 of the
+// stage's keys; maxima and weights meet in LDS; then wave w sums a quarter of the latent's columns (w / 2) for two tiles
+// (w % 2): a transposed read serves two tiles, and a wave's sums take the registers of half a tile, which leaves room for
+// a stage's operands to be asked for ahead of the products. Long rows come first.
 template <int RP, int WP>
-__global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatArgs a) {
-  using EC = EntryCopies<WP, 32>;
-  constexpr int KS = WP / 32, DT = RP / 16, PG = 1024;
+__global__ void __launch_bounds__(512, 2) latent_prefill_kernel(LatArgs a) {
+  using EC = EntryCopies<WP, 32, 8>;
+  constexpr int KS = WP / 32, DQ = RP / 64, PG = 1024;   // DQ: d-tiles of 16 a wave
   __shared__ __attribute__((aligned(1024))) unsigned char stage_lds[2 * EC::BYTES];
   __shared__ int64_t from_s[2][32];
   __shared__ int32_t pg_s[PG];
+  __shared__ float max_s[2][64], alpha_s[64];
+  __shared__ __attribute__((aligned(16))) bf16_t p_s[4][2][4][16][4];  // [tile][half of the keys][lane group][row][key]
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE, g = lane / 16, c = lane % 16;
+  const int rt = wave / 2, kh = wave % 2;
   const int b = a.row_ids[blockIdx.y];
   const int qs = a.qstart[b], nq = a.qstart[b + 1] - qs, n = a.lens[b];
-  const int rows = nq * a.heads, tiles = (rows + 63) / 64, half = (tiles + 1) / 2, idx = blockIdx.x;
-  if (idx >= tiles || n <= 0) return;                    // (the same in all of the block's threads)
-  const int range = idx < half ? tiles - 1 - idx : idx - half;
+  const int rows = nq * a.heads, tiles = (rows + 63) / 64;
+  if ((int)blockIdx.x >= tiles || n <= 0) return;        // (the same in all of the block's threads)
+  const int range = tiles - 1 - blockIdx.x;
   const int32_t* trow = table_row(a, b);
-  for (int i = tid; i < min(PG, a.table_stride); i += 256) pg_s[i] = trow[i];
-  const int m0 = range * 64 + wave * 16, row = m0 + c;
+  for (int i = tid; i < min(PG, a.table_stride); i += 512) pg_s[i] = trow[i];
+  const int m0 = range * 64, row = m0 + rt * 16 + c, before = n - nq;
   const bool valid = row < rows;
-  const int ti = valid ? row / a.heads : 0, head = valid ? row % a.heads : 0, before = n - nq;
+  const int ti = valid ? row / a.heads : 0, head = valid ? row % a.heads : 0;
   const int qpos = valid ? before + ti : -1;
-  const int wave_first = before + min(m0, rows - 1) / a.heads;
-  const int wave_last = m0 < rows ? before + (min(rows, m0 + 16) - 1) / a.heads : -1;
-  const int key_hi = before + (min(rows, range * 64 + 64) - 1) / a.heads, kb_last = key_hi / 32 * 32;
+  const int blk_first = before + m0 / a.heads;
+  const int key_hi = before + (min(rows, m0 + 64) - 1) / a.heads, kb_last = key_hi / 32 * 32;
   EC ec;
   ec.init(stage_lds, a.width);
   bf16x8_t qf[KS];
@@ -243,15 +246,18 @@ __global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatArgs a) {
         for (int i = 0; i < 8; ++i) qf[ks][i] = (__bf16)0.f;
     }
   }
-  f32x4_t o[DT];
+  f32x4_t o[DQ][2];
 #pragma unroll
-  for (int d = 0; d < DT; ++d) o[d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
+  for (int d = 0; d < DQ; ++d) o[d][0] = o[d][1] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;                          // of this wave's row c: the maximum over all keys, its half's sum
   lds_barrier();                                         // the block's table is in LDS
   auto find = [&](int kb, int buf) {                     // where the entries of the stage at kb lie
     if (tid < 32) {
       const int key = min(kb + tid, n - 1), at = min(key / a.page_size, a.table_stride - 1);
-      from_s[buf][tid] = entry_at(a, at < PG ? pg_s[at] : trow[at], key);
+      int page;
+      if (at < PG) page = pg_s[at];
+      else page = trow[at];
+      from_s[buf][tid] = entry_at(a, page, key);
     }
   };
   find(0, 0);
@@ -263,51 +269,68 @@ __global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatArgs a) {
   for (int kb = 0, buf = 0; kb <= kb_last; kb += 32, buf ^= 1) {
     if (kb < kb_last) ec.copy(a.pages, from_s[buf ^ 1], (uint32_t)(buf ^ 1) * EC::BYTES);
     if (kb + 32 < kb_last) find(kb + 64, buf);           // (this stage's own places have been read a stage ago)
-    if (kb <= wave_last) {
-      const unsigned char* lds = stage_lds + buf * EC::BYTES;
-      const unsigned char* kp = lds + c * EC::PITCH + g * 16;
+    const unsigned char* lds = stage_lds + buf * EC::BYTES;
+    float sv[4];
+    {
+      const unsigned char* kp = lds + (16 * kh + c) * EC::PITCH + g * 16;
       f32x4_t s0 = f32x4_t{0.f, 0.f, 0.f, 0.f}, s1 = s0;
+      bf16x8_t kf[KS];
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) kf[ks] = *reinterpret_cast<const bf16x8_t*>(kp + ks * 64);
 #pragma unroll
       for (int ks = 0; ks < KS; ++ks) {
-        const bf16x8_t k0 = *reinterpret_cast<const bf16x8_t*>(kp + ks * 64);
-        const bf16x8_t k1 = *reinterpret_cast<const bf16x8_t*>(kp + 16 * EC::PITCH + ks * 64);
-        s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qf[ks], s0, 0, 0, 0);
-        s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qf[ks], s1, 0, 0, 0);
+        f32x4_t& s = ks % 2 ? s1 : s0;
+        s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks], qf[ks], s, 0, 0, 0);
       }
-      float sv[8];
 #pragma unroll
-      for (int r = 0; r < 8; ++r) sv[r] = r < 4 ? s0[r] : s1[r - 4];
-      if (kb + 31 > wave_first) {
+      for (int r = 0; r < 4; ++r) sv[r] = s0[r] + s1[r];
+    }
+    if (kb + 31 > blk_first) {
 #pragma unroll
-        for (int r = 0; r < 8; ++r)
-          if (kb + 16 * (r / 4) + 4 * g + r % 4 > qpos) sv[r] = -INFINITY;
-      }
-      float mx = fmaxf(fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3])), fmaxf(fmaxf(sv[4], sv[5]), fmaxf(sv[6], sv[7])));
-      mx = max_over_groups(mx);
-      const float m_new = fmaxf(m, mx * a.scale_log2);
+      for (int r = 0; r < 4; ++r)
+        if (kb + 16 * kh + 4 * g + r > qpos) sv[r] = -INFINITY;
+    }
+    const float mx = max_over_groups(fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3])));
+    if (g == 0) max_s[kh][rt * 16 + c] = mx * a.scale_log2;
+    lds_barrier();
+    {
+      const float m_new = fmaxf(m, fmaxf(max_s[0][rt * 16 + c], max_s[1][rt * 16 + c]));
       const float m_use = m_new == -INFINITY ? 0.f : m_new;
-      bf16x8_t pb;
-      float psum = 0.f;
+      const float alpha = __builtin_amdgcn_exp2f(m - m_use);
+      float p[4];
 #pragma unroll
-      for (int r = 0; r < 8; ++r) {
-        const float p = __builtin_amdgcn_exp2f(fmaf(sv[r], a.scale_log2, -m_use));
-        psum += p;
-        pb[r] = (__bf16)p;
+      for (int r = 0; r < 4; ++r) p[r] = __builtin_amdgcn_exp2f(fmaf(sv[r], a.scale_log2, -m_use));
+      ushort4 w;
+      w.x = float_to_bf16(p[0]); w.y = float_to_bf16(p[1]); w.z = float_to_bf16(p[2]); w.w = float_to_bf16(p[3]);
+      *reinterpret_cast<ushort4*>(&p_s[rt][kh][g][c][0]) = w;
+      if (kh == 0 && g == 0) alpha_s[rt * 16 + c] = alpha;
+      l = l * alpha + ((p[0] + p[1]) + (p[2] + p[3]));
+      m = m_new;
+    }
+    lds_barrier();
+    {
+      bf16x8_t pb[2];
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {                      // tiles 2 kh and 2 kh + 1
+        const bf16x4_t lo = *reinterpret_cast<const bf16x4_t*>(&p_s[2 * kh + i][0][g][c][0]);
+        const bf16x4_t hi = *reinterpret_cast<const bf16x4_t*>(&p_s[2 * kh + i][1][g][c][0]);
+        pb[i] = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
+        const float alpha = alpha_s[(2 * kh + i) * 16 + c];
+        if (__any(alpha != 1.f)) {
+#pragma unroll
+          for (int d = 0; d < DQ; ++d) o[d][i] *= alpha;
+        }
       }
-      if (__any(m_new != m)) {
-        const float alpha = __builtin_amdgcn_exp2f(m - m_use);
-        l *= alpha;
+      const unsigned char* vp = lds + (4 * g + c / 4) * EC::PITCH + (c % 4) * 8 + rt * DQ * 32;
+      bf16x8_t v[DQ];
 #pragma unroll
-        for (int d = 0; d < DT; ++d) o[d] *= alpha;
-        m = m_new;
-      }
-      l += psum;
-      const unsigned char* vp = lds + (4 * g + c / 4) * EC::PITCH + (c % 4) * 8;
+      for (int d = 0; d < DQ; ++d)
+        v[d] = __builtin_shufflevector(read_transposed(vp + d * 32), read_transposed(vp + 16 * EC::PITCH + d * 32), 0, 1, 2, 3, 4,
+                                       5, 6, 7);
 #pragma unroll
-      for (int d = 0; d < DT; ++d) {
-        const bf16x4_t lo = read_transposed(vp + d * 32), hi = read_transposed(vp + 16 * EC::PITCH + d * 32);
-        const bf16x8_t v = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
-        o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pb, o[d], 0, 0, 0);
+      for (int d = 0; d < DQ; ++d) {
+        o[d][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v[d], pb[0], o[d][0], 0, 0, 0);
+        o[d][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v[d], pb[1], o[d][1], 0, 0, 0);
       }
     }
     wait_loads_but<0>();                                 // the next stage has landed (this wave's share of it)
@@ -315,19 +338,27 @@ __global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatArgs a) {
   }
   l += __shfl_xor(l, 16, WAVE);
   l += __shfl_xor(l, 32, WAVE);
-  if (!valid) return;
-  if (a.sink) l += __builtin_amdgcn_exp2f(a.sink[head] * 1.4426950408889634f - m);
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
-  bf16_t* op = a.out + ((int64_t)(qs + ti) * a.heads + head) * a.kv_rank + 4 * g;
+  if (g == 0) max_s[kh][rt * 16 + c] = l;
+  if (g == 0 && kh == 0) alpha_s[rt * 16 + c] = valid && a.sink ? __builtin_amdgcn_exp2f(a.sink[head] * 1.4426950408889634f - m) : 0.f;
+  lds_barrier();
 #pragma unroll
-  for (int d = 0; d < DT; ++d) {
-    if (d * 16 + 4 * g >= a.kv_rank) break;
-    ushort4 w;
-    w.x = float_to_bf16(o[d][0] * inv);
-    w.y = float_to_bf16(o[d][1] * inv);
-    w.z = float_to_bf16(o[d][2] * inv);
-    w.w = float_to_bf16(o[d][3] * inv);
-    *reinterpret_cast<ushort4*>(op + d * 16) = w;
+  for (int i = 0; i < 2; ++i) {
+    const int at = (2 * kh + i) * 16 + c, r = m0 + at;
+    if (r >= rows) continue;
+    const float den = (max_s[0][at] + max_s[1][at]) + alpha_s[at];
+    const float inv = den > 0.f ? 1.0f / den : 0.f;
+    const int d0 = rt * DQ * 16 + 4 * g;
+    bf16_t* op = a.out + ((int64_t)qs * a.heads + r) * a.kv_rank + d0;
+#pragma unroll
+    for (int d = 0; d < DQ; ++d) {
+      if (d0 + d * 16 >= a.kv_rank) break;
+      ushort4 w;
+      w.x = float_to_bf16(o[d][i][0] * inv);
+      w.y = float_to_bf16(o[d][i][1] * inv);
+      w.z = float_to_bf16(o[d][i][2] * inv);
+      w.w = float_to_bf16(o[d][i][3] * inv);
+      *reinterpret_cast<ushort4*>(op + d * 16) = w;
+    }
   }
 }
 
@@ -336,7 +367,7 @@ __global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatArgs a) {
 // One block a row writes the result; more leave (values, maximum, sum) for the merge below.
 template <int RP, int WP>
 __global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatArgs a) {
-  using EC = EntryCopies<WP, 64>;
+  using EC = EntryCopies<WP, 64, 4>;
   constexpr int KS = WP / 32, DW = RP / 64;              // d-tiles of 16 a wave
   __shared__ __attribute__((aligned(1024))) unsigned char tile_lds[EC::BYTES];
   __shared__ int64_t from_s[64];
@@ -496,22 +527,27 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(LatArgs a) {
 // -- every head's own projection ------------------------------------------------------------------------------------------
 // y[t, h, b] = sum_a x[t, h, a] w[h, b, a], bfloat16 operands, float32 sums, one rounding; with `gate` the sum times
 // sigmoid(gate[t, h B + b]) first. A = 16 rows of w x 32, B = 32 x 16 tokens: a lane holds four neighbouring results of a
-// token. Loads past A or B read zeros or a row that is there.
+// token. Rows past B or the last token repeat the last one that is there; their results are not stored.
 struct HeadLinear {
   const bf16_t* x;
   const bf16_t* w;
   bf16_t* y;
   const bf16_t* gate;
   int64_t gate_stride;
-  int rows, heads, A, B, y_head, wide_out;
+  int rows, heads, A, B, y_head;
+  int wide_out, wide_gate;     // four results (few tokens) or eight (many) lie on a border of their size, gates likewise
 };
 
-__device__ __forceinline__ bf16x8_t load_piece(const bf16_t* p, bool ok) {
-  bf16x8_t v;
-  if (ok) return *reinterpret_cast<const bf16x8_t*>(p);
-#pragma unroll
-  for (int i = 0; i < 8; ++i) v[i] = (__bf16)0.f;
-  return v;
+// Eight values from column k + 8 g of a row on (`row` points at column 8 g). TAIL: A is no multiple of 32, and a piece past
+// the row's end counts as zeros (it is read from the row's start all the same: a branch around a load would keep the loads
+// from being under way together).
+template <bool TAIL>
+__device__ __forceinline__ bf16x8_t load_piece(const bf16_t* row, int k, int g, int A) {
+  if constexpr (!TAIL) return *reinterpret_cast<const bf16x8_t*>(row + k);
+  const bool ok = k + 8 * g < A;
+  uint4 v = *reinterpret_cast<const uint4*>(row + (ok ? k : -8 * g));
+  v.x = ok ? v.x : 0u; v.y = ok ? v.y : 0u; v.z = ok ? v.z : 0u; v.w = ok ? v.w : 0u;
+  return __builtin_bit_cast(bf16x8_t, v);
 }
 
 __device__ __forceinline__ void head_linear_store(const HeadLinear& a, int t, int h, int b, f32x4_t v) {
@@ -535,6 +571,7 @@ __device__ __forceinline__ void head_linear_store(const HeadLinear& a, int t, in
 }
 
 // Up to 16 tokens: a block a head and 16 columns, A dealt to its four waves in steps of 32, their sums added in wave order.
+template <bool TAIL>
 __global__ void __launch_bounds__(256) head_linear_few_kernel(HeadLinear a) {
   __shared__ f32x4_t sum_s[3][WAVE];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, g = lane / 16, c = lane % 16;
@@ -544,8 +581,7 @@ __global__ void __launch_bounds__(256) head_linear_few_kernel(HeadLinear a) {
   f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
   for (int k = wave * 32; k < a.A; k += 128) {
-    const bool ok = k + 8 * g < a.A;
-    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(load_piece(wp + k, ok), load_piece(xp + k, ok), acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(load_piece<TAIL>(wp, k, g, a.A), load_piece<TAIL>(xp, k, g, a.A), acc, 0, 0, 0);
   }
   if (wave > 0) sum_s[wave - 1][lane] = acc;
   __syncthreads();
@@ -554,39 +590,92 @@ __global__ void __launch_bounds__(256) head_linear_few_kernel(HeadLinear a) {
   head_linear_store(a, c, h, b0 + 4 * g, acc);
 }
 
-// More tokens: a block 64 tokens and 128 columns of a head, a wave 32 of the columns.
+// More tokens: a block 128 tokens and 128 columns of a head, a wave 64 by 64; a step's operands are asked for while the
+// step before is multiplied. The results pass LDS on their way out, half of a wave's tokens at a time, so that a token's 64
+// columns are stored as one whole line and its gates are read as one.
+template <bool TAIL>
 __global__ void __launch_bounds__(256) head_linear_many_kernel(HeadLinear a) {
+  constexpr int OP = 68;
+  __shared__ __attribute__((aligned(16))) float out_s[4][32 * OP];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, g = lane / 16, c = lane % 16;
-  const int h = blockIdx.y, t0 = blockIdx.x * 64, b0 = blockIdx.z * 128 + wave * 32;
-  if (b0 >= a.B) return;
-  const bf16_t* wp[2];
+  const int h = blockIdx.y, t0 = blockIdx.x * 128 + (wave % 2) * 64, b0 = blockIdx.z * 128 + (wave / 2) * 64;
+  if (b0 >= a.B || t0 >= a.rows) return;
+  const bf16_t* wp[4];
   const bf16_t* xp[4];
 #pragma unroll
-  for (int i = 0; i < 2; ++i) wp[i] = a.w + ((int64_t)h * a.B + min(b0 + 16 * i + c, a.B - 1)) * a.A + 8 * g;
+  for (int i = 0; i < 4; ++i) {
+    wp[i] = a.w + ((int64_t)h * a.B + min(b0 + 16 * i + c, a.B - 1)) * a.A + 8 * g;
+    xp[i] = a.x + ((int64_t)min(t0 + 16 * i + c, a.rows - 1) * a.heads + h) * a.A + 8 * g;
+  }
+  f32x4_t acc[4][4];
 #pragma unroll
-  for (int j = 0; j < 4; ++j) xp[j] = a.x + ((int64_t)min(t0 + 16 * j + c, a.rows - 1) * a.heads + h) * a.A + 8 * g;
-  f32x4_t acc[2][4];
-#pragma unroll
-  for (int i = 0; i < 2; ++i)
+  for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-  for (int k = 0; k < a.A; k += 32) {
-    const bool ok = k + 8 * g < a.A;
-    bf16x8_t wf[2], xf[4];
+  bf16x8_t wf[2][4], xf[2][4];
+  auto ask = [&](int k, int buf) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i) wf[i] = load_piece(wp[i] + k, ok);
+    for (int i = 0; i < 4; ++i) {
+      wf[buf][i] = load_piece<TAIL>(wp[i], k, g, a.A);
+      xf[buf][i] = load_piece<TAIL>(xp[i], k, g, a.A);
+    }
+  };
+  auto multiply = [&](int buf) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) xf[j] = load_piece(xp[j] + k, ok);
+    for (int i = 0; i < 4; ++i)
 #pragma unroll
-    for (int i = 0; i < 2; ++i)
-#pragma unroll
-      for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], xf[j], acc[i][j], 0, 0, 0);
+      for (int j = 0; j < 4; ++j)
+        acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[buf][i], xf[buf][j], acc[i][j], 0, 0, 0);
+  };
+  ask(0, 0);
+  for (int k = 0; k < a.A; k += 64) {
+    if (k + 32 < a.A) ask(k + 32, 1);
+    multiply(0);
+    if (k + 64 < a.A) ask(k + 64, 0);
+    if (k + 32 < a.A) multiply(1);
   }
+  float* mine = out_s[wave];                             // (a wave's own: its LDS operations run in order)
+  const int piece = (lane % 8) * 8, b = b0 + piece;
 #pragma unroll
-  for (int i = 0; i < 2; ++i)
+  for (int part = 0; part < 2; ++part) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) head_linear_store(a, t0 + 16 * j + c, h, b0 + 16 * i + 4 * g, acc[i][j]);
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) *reinterpret_cast<f32x4_t*>(mine + (16 * j + c) * OP + 16 * i + 4 * g) = acc[i][2 * part + j];
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int at = e * 8 + lane / 8, t = t0 + part * 32 + at;
+      if (t >= a.rows || b >= a.B) continue;
+      float v[8];
+      *reinterpret_cast<f32x4_t*>(v) = *reinterpret_cast<const f32x4_t*>(mine + at * OP + piece);
+      *reinterpret_cast<f32x4_t*>(v + 4) = *reinterpret_cast<const f32x4_t*>(mine + at * OP + piece + 4);
+      const bool whole = b + 7 < a.B;
+      if (a.gate) {
+        const bf16_t* gp = a.gate + t * a.gate_stride + (int64_t)h * a.B + b;
+        __attribute__((aligned(16))) bf16_t gv[8];
+        if (whole && a.wide_gate) *reinterpret_cast<uint4*>(gv) = *reinterpret_cast<const uint4*>(gp);
+        else
+#pragma unroll
+          for (int u = 0; u < 8; ++u) gv[u] = b + u < a.B ? gp[u] : (bf16_t)0;
+#pragma unroll
+        for (int u = 0; u < 8; ++u) v[u] *= __builtin_amdgcn_rcpf(1.0f + __expf(-bf16_to_float(gv[u])));
+      }
+      bf16_t* yp = a.y + ((int64_t)t * a.heads + h) * a.y_head + b;
+      if (whole && a.wide_out) {
+        uint4 raw;
+        bf16_t* o = reinterpret_cast<bf16_t*>(&raw);
+#pragma unroll
+        for (int u = 0; u < 8; ++u) o[u] = float_to_bf16(v[u]);
+        *reinterpret_cast<uint4*>(yp) = raw;
+      } else {
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+          if (b + u < a.B) yp[u] = float_to_bf16(v[u]);
+      }
+    }
+    __builtin_amdgcn_wave_barrier();
+  }
 }
 }  // namespace
 
@@ -596,11 +685,17 @@ extern "C" int holon_head_linear_bf16(const void* x, const void* w, void* y, int
   HOLON_CHECK(rows >= 1 && heads > 0 && heads <= 65535 && A > 0 && A % 8 == 0 && B > 0 && B <= 65535 * 16 && y_head >= B &&
                   (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0,
               "head_linear: %d rows, %d heads of %d (a multiple of 8) -> %d (in steps of %d)", rows, heads, A, B, y_head);
+  const int unit = rows <= 16 ? 4 : 8;                   // results a lane stores at once
   const HeadLinear a{(const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, (const bf16_t*)gate, gate_stride, rows, heads, A, B, y_head,
-                     (int)(y_head % 4 == 0 && (uintptr_t)y % 8 == 0)};
+                     (int)(y_head % unit == 0 && (uintptr_t)y % (2 * unit) == 0),
+                     (int)(gate_stride % 8 == 0 && B % 8 == 0 && (uintptr_t)gate % 16 == 0)};
   hipStream_t s = (hipStream_t)stream;
-  if (rows <= 16) head_linear_few_kernel<<<dim3(heads, (B + 15) / 16), 256, 0, s>>>(a);
-  else head_linear_many_kernel<<<dim3((rows + 63) / 64, heads, (B + 127) / 128), 256, 0, s>>>(a);
+  const dim3 few(heads, (B + 15) / 16), many((rows + 127) / 128, heads, (B + 127) / 128);
+  if (rows <= 16) {
+    if (A % 32) head_linear_few_kernel<true><<<few, 256, 0, s>>>(a); else head_linear_few_kernel<false><<<few, 256, 0, s>>>(a);
+  } else {
+    if (A % 32) head_linear_many_kernel<true><<<many, 256, 0, s>>>(a); else head_linear_many_kernel<false><<<many, 256, 0, s>>>(a);
+  }
   HOLON_LAUNCH_OK();
   return 0;
 }
@@ -641,7 +736,7 @@ extern "C" int holon_latent_prefill_bf16(const void* q, void* out, const void* p
   LatArgs a{(const bf16_t*)q, (bf16_t*)out, (const bf16_t*)pages, table, slots, lens, qstart, row_ids, sink, nullptr, nullptr,
             table_stride, table_rows, num_pages, page_size, heads, width, kv_rank, 0, 1, scale * 1.4426950408889634f};
   const dim3 grid((max_query * heads + 63) / 64, rows);
-  LAT_BY_SIZE((latent_prefill_kernel<RP, WP><<<grid, 256, 0, (hipStream_t)stream>>>(a)));
+  LAT_BY_SIZE((latent_prefill_kernel<RP, WP><<<grid, 512, 0, (hipStream_t)stream>>>(a)));
   HOLON_LAUNCH_OK();
   return 0;
 }
