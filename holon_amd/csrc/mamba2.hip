@@ -132,45 +132,54 @@ __global__ void __launch_bounds__(256) ssd_step_kernel(
 }
 
 // -- pieces -------------------------------------------------------------------------------------------------------------
-// `rows` x `cols` values from src (rows src_stride apart) into LDS rows of `pitch` values, zeros beyond rows_ok and
-// cols. ALIGNED: every source row starts on a 16-byte border and cols is a multiple of the vector.
+// ROWS x COLS values from src (rows src_stride apart) into LDS rows of `pitch` values, zeros beyond rows_ok and cols, in two
+// steps: `ask` sends the loads off, `put` writes what they brought (a tile's loads then travel while the tile before is
+// worked on). ALIGNED: every source row starts on a 16-byte border and cols is a multiple of the vector; else `put` does it
+// all, value by value.
 template <typename T, typename D, int ROWS, int COLS, bool ALIGNED>
-__device__ __forceinline__ void stage_tile(D* dst, int pitch, const T* src, int64_t src_stride, int rows_ok, int cols) {
-  if constexpr (ALIGNED) {
-    constexpr int N = Elem<T>::kVec, PER_ROW = COLS / N, TOTAL = ROWS * PER_ROW, PER = (TOTAL + 255) / 256;
-    uint4 raw[PER];
+struct Tile {
+  static constexpr int N = Elem<T>::kVec, PER_ROW = COLS / N, TOTAL = ROWS * PER_ROW, PER = (TOTAL + 255) / 256;
+  uint4 raw[ALIGNED ? PER : 1];
+  const T* src;
+  int64_t src_stride;
+  int rows_ok, cols;
+  __device__ __forceinline__ void ask(const T* from, int64_t stride, int rows, int columns) {
+    src = from; src_stride = stride; rows_ok = rows; cols = columns;
+    if constexpr (ALIGNED) {
 #pragma unroll
-    for (int e = 0; e < PER; ++e) {
-      const int idx = threadIdx.x + e * 256, r = idx / PER_ROW, c = (idx % PER_ROW) * N;
-      raw[e] = make_uint4(0u, 0u, 0u, 0u);
-      if (idx < TOTAL && r < rows_ok && c < cols) raw[e] = *reinterpret_cast<const uint4*>(src + r * src_stride + c);
-    }
-#pragma unroll
-    for (int e = 0; e < PER; ++e) {
-      const int idx = threadIdx.x + e * 256, r = idx / PER_ROW, c = (idx % PER_ROW) * N;
-      if (idx >= TOTAL) continue;
-      if constexpr (sizeof(D) == sizeof(T)) {
-        *reinterpret_cast<uint4*>(dst + r * pitch + c) = raw[e];
-      } else {
-        const T* v = reinterpret_cast<const T*>(&raw[e]);
-#pragma unroll
-        for (int u = 0; u < N; u += 4)
-          *reinterpret_cast<float4*>(dst + r * pitch + c + u) =
-              make_float4(Elem<T>::load(v[u]), Elem<T>::load(v[u + 1]), Elem<T>::load(v[u + 2]), Elem<T>::load(v[u + 3]));
-      }
-    }
-  } else {
-    for (int idx = threadIdx.x; idx < ROWS * COLS; idx += 256) {
-      const int r = idx / COLS, c = idx % COLS;
-      const bool ok = r < rows_ok && c < cols;
-      if constexpr (sizeof(D) == sizeof(T)) {
-        dst[r * pitch + c] = ok ? src[r * src_stride + c] : T(0);
-      } else {
-        dst[r * pitch + c] = ok ? Elem<T>::load(src[r * src_stride + c]) : 0.f;
+      for (int e = 0; e < PER; ++e) {
+        const int idx = threadIdx.x + e * 256, r = idx / PER_ROW, c = (idx % PER_ROW) * N;
+        raw[e] = make_uint4(0u, 0u, 0u, 0u);
+        if (idx < TOTAL && r < rows_ok && c < cols) raw[e] = *reinterpret_cast<const uint4*>(src + r * src_stride + c);
       }
     }
   }
-}
+  __device__ __forceinline__ void put(D* dst, int pitch) const {
+    if constexpr (ALIGNED) {
+#pragma unroll
+      for (int e = 0; e < PER; ++e) {
+        const int idx = threadIdx.x + e * 256, r = idx / PER_ROW, c = (idx % PER_ROW) * N;
+        if (idx >= TOTAL) continue;
+        if constexpr (sizeof(D) == sizeof(T)) {
+          *reinterpret_cast<uint4*>(dst + r * pitch + c) = raw[e];
+        } else {
+          const T* v = reinterpret_cast<const T*>(&raw[e]);
+#pragma unroll
+          for (int u = 0; u < N; u += 4)
+            *reinterpret_cast<float4*>(dst + r * pitch + c + u) =
+                make_float4(Elem<T>::load(v[u]), Elem<T>::load(v[u + 1]), Elem<T>::load(v[u + 2]), Elem<T>::load(v[u + 3]));
+        }
+      }
+    } else {
+      for (int idx = threadIdx.x; idx < ROWS * COLS; idx += 256) {
+        const int r = idx / COLS, c = idx % COLS;
+        const bool ok = r < rows_ok && c < cols;
+        if constexpr (sizeof(D) == sizeof(T)) dst[r * pitch + c] = ok ? src[r * src_stride + c] : T(0);
+        else dst[r * pitch + c] = ok ? Elem<T>::load(src[r * src_stride + c]) : 0.f;
+      }
+    }
+  }
+};
 
 // Inclusive sum over the block's 256 threads in thread order, in float64.
 __device__ __forceinline__ double scan_256(double v, double* wave_tot) {
@@ -225,11 +234,19 @@ __global__ void __launch_bounds__(256) ssd_state_kernel(
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   const int vcols = min(SSD_VG, vdim - v0);
-  for (int t0 = 0; t0 < cnt; t0 += KT) {
+  Tile<T, float, KT, 64 * NTW, ALIGNED> bt;
+  Tile<T, float, KT, SSD_VG, ALIGNED> xt;
+  auto ask = [&](int t0) {
     const T* rowp = xbc + (int64_t)(lo + t0) * channels;
-    stage_tile<T, float, KT, 64 * NTW, ALIGNED>(Bs, BP, rowp + inner + g * n, channels, cnt - t0, n);
-    stage_tile<T, float, KT, SSD_VG, ALIGNED>(Xs, XP, rowp + h * vdim + v0, channels, cnt - t0, vcols);
+    bt.ask(rowp + inner + g * n, channels, cnt - t0, n);
+    xt.ask(rowp + h * vdim + v0, channels, cnt - t0, vcols);
+  };
+  ask(0);
+  for (int t0 = 0; t0 < cnt; t0 += KT) {
+    bt.put(Bs, BP);
+    xt.put(Xs, XP);
     __syncthreads();
+    if (t0 + KT < cnt) ask(t0 + KT);
 #pragma unroll
     for (int ks = 0; ks < KT / 4; ++ks) {
       const int t = ks * 4 + grp;
@@ -321,21 +338,39 @@ __global__ void __launch_bounds__(256) ssd_out_kernel(const T* __restrict__ xbc,
     chi[tid] = ok ? sums[plane + from] : 0.f;
     clo[tid] = ok ? sums[2 * plane + from] : 0.f;
   }
-  stage_tile<T, T, SSD_QT, NP, ALIGNED>(Cs, CP, xbc + (int64_t)(lo + q0) * channels + inner + groups * n + g * n, channels,
-                                        cnt - q0, n);
+  const bool svec = vdim % 4 == 0;
+  const float* S = sin + (piece * heads + h) * (int64_t)n * vdim + v0;
+  Tile<float, float, KT, SSD_VG, true> st;               // the state in front of the piece, KT rows of it at a time
+  if (svec) st.ask(S, vdim, n, vcols);
+  {
+    Tile<T, T, SSD_QT, NP, ALIGNED> ct;
+    ct.ask(xbc + (int64_t)(lo + q0) * channels + inner + groups * n + g * n, channels, cnt - q0, n);
+    ct.put(Cs, CP);
+  }
+  Tile<T, T, KT, NP, ALIGNED> bt;
+  Tile<T, float, KT, SSD_VG, ALIGNED> xt;
+  auto ask = [&](int k0) {
+    const T* rowp = xbc + (int64_t)(lo + k0) * channels;
+    bt.ask(rowp + inner + g * n, channels, cnt - k0, n);
+    xt.ask(rowp + h * vdim + v0, channels, cnt - k0, vcols);
+  };
   const int wave = tid / WAVE, lane = tid % WAVE, grp = lane / 16, col = lane % 16;
   const int q = q0 + wave * 16 + col;                    // this lane's query in the piece (its column)
   f32x4 acc[4];
 #pragma unroll
   for (int j = 0; j < 4; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  // the state in front of the piece, KT rows of it at a time
-  const float* S = sin + (piece * heads + h) * (int64_t)n * vdim + v0;
-  const bool svec = vdim % 4 == 0;
   for (int n0 = 0; n0 < n; n0 += KT) {
     __syncthreads();
-    if (svec) stage_tile<float, float, KT, SSD_VG, true>(Xs, XP, S + (int64_t)n0 * vdim, vdim, n - n0, vcols);
-    else stage_tile<float, float, KT, SSD_VG, false>(Xs, XP, S + (int64_t)n0 * vdim, vdim, n - n0, vcols);
+    if (svec) {
+      st.put(Xs, XP);
+    } else {
+      Tile<float, float, KT, SSD_VG, false> one;
+      one.ask(S + (int64_t)n0 * vdim, vdim, n - n0, vcols);
+      one.put(Xs, XP);
+    }
     __syncthreads();
+    if (n0 + KT < n && svec) st.ask(S + (int64_t)(n0 + KT) * vdim, vdim, n - n0 - KT, vcols);
+    if (n0 + KT >= n) ask(0);                            // the first keys travel behind the last of the state
 #pragma unroll
     for (int kb = 0; kb < KT / 16; ++kb) {
       if (n0 + kb * 16 >= NP) break;
@@ -359,10 +394,10 @@ __global__ void __launch_bounds__(256) ssd_out_kernel(const T* __restrict__ xbc,
   const int q_last = min(q0 + SSD_QT, cnt) - 1;          // the tile's last query
   for (int k0 = 0; k0 <= q_last; k0 += KT) {
     __syncthreads();
-    const T* rowp = xbc + (int64_t)(lo + k0) * channels;
-    stage_tile<T, T, KT, NP, ALIGNED>(Bs, CP, rowp + inner + g * n, channels, cnt - k0, n);
-    stage_tile<T, float, KT, SSD_VG, ALIGNED>(Xs, XP, rowp + h * vdim + v0, channels, cnt - k0, vcols);
+    bt.put(Bs, CP);
+    xt.put(Xs, XP);
     __syncthreads();
+    if (k0 + KT <= q_last) ask(k0 + KT);
 #pragma unroll
     for (int ks = 0; ks < KT / 16; ++ks) {
       if (k0 + ks * 16 > q0 + wave * 16 + 15) break;     // keys behind every query of this wave
