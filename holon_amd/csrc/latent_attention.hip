@@ -485,13 +485,22 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatArgs a) {
 }
 
 // out = sum_i 2^(m_i - M) o_i / sum_i 2^(m_i - M) l_i over a (decode row, head)'s splits (at most 64), the sink joining the
-// denominator. One block a (row, head): 128 threads take four columns each over the even splits, 128 over the odd ones.
+// denominator. A block a (row, head, 128 columns): thread (side, column) takes four columns of splits side, side + 8, ...,
+// all asked for before the factors are known; the eight sides are added in order.
 __global__ void __launch_bounds__(256) latent_merge_kernel(LatArgs a) {
+  constexpr int SIDES = 8, EACH = 64 / SIDES;
   __shared__ float f_s[64];
   __shared__ float den_s;
-  __shared__ __attribute__((aligned(16))) float sum_s[LAT_MAX];
+  __shared__ __attribute__((aligned(16))) f32x4_t sum_s[SIDES][32];
   const int head = blockIdx.x, tid = threadIdx.x, b = a.row_ids[blockIdx.y];
   const int64_t cell = ((int64_t)blockIdx.y * a.heads + head) * a.splits;
+  const int side = tid / 32, d = blockIdx.z * 128 + (tid % 32) * 4;
+  const bool held = d < a.kv_rank;
+  f32x4_t v[EACH];
+#pragma unroll
+  for (int e = 0; e < EACH; ++e)
+    if (held && side + SIDES * e < a.splits)
+      v[e] = *reinterpret_cast<const f32x4_t*>(a.part_o + (cell + side + SIDES * e) * a.kv_rank + d);
   if (tid < WAVE) {
     const float mi = tid < a.splits ? a.part_ml[(cell + tid) * 2] : -INFINITY;
     const float li = tid < a.splits ? a.part_ml[(cell + tid) * 2 + 1] : 0.f;
@@ -503,25 +512,23 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(LatArgs a) {
     if (tid == 0) den_s = den > 0.f ? 1.0f / den : 0.f;
   }
   __syncthreads();
-  const int side = tid / 128, d = (tid % 128) * 4;
-  for (int d4 = d; d4 < a.kv_rank; d4 += 512) {
-    f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 8
-    for (int i = side; i < a.splits; i += 2) {
-      const float f = f_s[i];                            // (a split that saw nothing has written no values: not read)
-      if (f != 0.f) acc += f * *reinterpret_cast<const f32x4_t*>(a.part_o + (cell + i) * a.kv_rank + d4);
-    }
-    if (side == 1) *reinterpret_cast<f32x4_t*>(&sum_s[d4]) = acc;
-    __syncthreads();
-    if (side == 0) {
-      acc += *reinterpret_cast<const f32x4_t*>(&sum_s[d4]);
-      const float inv = den_s;
-      ushort4 w;
-      w.x = float_to_bf16(acc[0] * inv); w.y = float_to_bf16(acc[1] * inv);
-      w.z = float_to_bf16(acc[2] * inv); w.w = float_to_bf16(acc[3] * inv);
-      *reinterpret_cast<ushort4*>(a.out + ((int64_t)a.qstart[b] * a.heads + head) * a.kv_rank + d4) = w;
-    }
+  f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int e = 0; e < EACH; ++e) {
+    if (!held || side + SIDES * e >= a.splits) break;
+    const float f = f_s[side + SIDES * e];               // (a split that saw nothing has written no values: not used)
+    if (f != 0.f) acc += f * v[e];
   }
+  sum_s[side][tid % 32] = acc;
+  __syncthreads();
+  if (side > 0 || !held) return;
+#pragma unroll
+  for (int i = 1; i < SIDES; ++i) acc += sum_s[i][tid];
+  const float inv = den_s;
+  ushort4 w;
+  w.x = float_to_bf16(acc[0] * inv); w.y = float_to_bf16(acc[1] * inv);
+  w.z = float_to_bf16(acc[2] * inv); w.w = float_to_bf16(acc[3] * inv);
+  *reinterpret_cast<ushort4*>(a.out + ((int64_t)a.qstart[b] * a.heads + head) * a.kv_rank + d) = w;
 }
 
 // -- every head's own projection ------------------------------------------------------------------------------------------
@@ -758,7 +765,7 @@ extern "C" int holon_latent_decode_bf16(const void* q, void* out, const void* pa
   LAT_BY_SIZE((latent_decode_kernel<RP, WP><<<grid, 256, 0, (hipStream_t)stream>>>(a)));
   HOLON_LAUNCH_OK();
   if (splits > 1) {
-    latent_merge_kernel<<<dim3(heads, rows), 256, 0, (hipStream_t)stream>>>(a);
+    latent_merge_kernel<<<dim3(heads, rows, (kv_rank + 127) / 128), 256, 0, (hipStream_t)stream>>>(a);
     HOLON_LAUNCH_OK();
   }
   return 0;

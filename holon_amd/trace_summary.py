@@ -13,6 +13,7 @@ from __future__ import annotations
 
 import argparse
 import collections
+import re
 import sqlite3
 
 SHORT = (("_Z18gemm_skinny_kernelILi", "gemm_skinny<"), ("_Z22gemm_skinny_glu_kernelILi", "gemm_skinny_glu<"),
@@ -42,6 +43,10 @@ def short_name(name: str) -> str:
     for long, brief in SHORT:
         if name.startswith(long):
             name = brief + name[len(long):]
+    local = re.match(r"_ZN12_GLOBAL__N_1(\d+)(.*)", name)   # any other kernel of the library: length and name
+    if local:
+        n, rest = int(local[1]), local[2]
+        name = rest[:n].removesuffix("_kernel") + ("<" + rest[n + 1:] if rest[n: n + 1] == "I" else "")
     return name[:64]
 
 
@@ -54,11 +59,14 @@ def dispatches(path: str) -> list[tuple]:
     return [(n, st, en, gx // max(wx, 1), gy, gz) for n, st, en, gx, gy, gz, wx in rows]
 
 
-CLASSES = (("attention", ("attn_", "sigmoid_attention", "softmax_attention")), ("matrix products", ("gemm_", "Cijk_", "Custom_Cijk_", "hipBLASLt")),
-           ("recurrent scans", ("memory_scan", "delta_scan", "memory_pieces", "delta_pieces", "mlstm_scan")),
+CLASSES = (("attention", ("attn_", "sigmoid_attention", "softmax_attention", "latent_attention", "latent_prefill", "latent_decode",
+                          "latent_merge")),
+           ("matrix products", ("gemm_", "Cijk_", "Custom_Cijk_", "hipBLASLt", "head_linear")),
+           ("recurrent scans", ("memory_scan", "delta_scan", "memory_pieces", "delta_pieces", "mlstm_scan", "ssd_")),
            ("elementwise", ("rmsnorm", "silu_mul", "qk_norm_rope", "v_write", "kv_write", "embedding", "sum_parts",
                             "row_sumsq", "scatter_rows", "stream_norm", "dyt_stream", "widen_", "pair_rows", "softcap", "causal_conv",
-                            "head_prepare", "delta_prepare", "gated_out", "shift_mix", "shift_keep", "decay_lora")),
+                            "head_prepare", "delta_prepare", "gated_out", "shift_mix", "shift_keep", "decay_lora", "stream_rms", "latent_rope_prepare", "gated_parts_norm",
+                            "moe_gate", "moe_router")),
            ("sampling", ("argmax", "sample_kernel", "store_tokens", "logprobs")))
 
 
