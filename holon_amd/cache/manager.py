@@ -1,12 +1,13 @@
 """The cache manager: slots, paged groups with block tables, and fixed-size per-request state.
 
 A request is given a *slot* when it is admitted: its row in every block table and in every fixed-size state tensor.
-State that grows lives in pages. Paged states of equal page geometry (values per token, window, dtype), whichever runs
+State that grows lives in pages. Paged states of equal page geometry (values per token, window or chunk, dtype), whichever runs
 declare them and however many one run declares, form a *group*: one page pool, one block table, one storage tensor
 `[members, pages, page_size * elems]` with a member for every (run, state name) of the group. Page id p means row p
 of every member. Groups with different needs (all tokens, a window of them, another width) have pools and tables of
 their own; a windowed group gives pages back as soon as the window has passed them (all but the pages of the first
-tokens, where the declaration says that those stay visible), a finished request gives back everything.
+tokens, where the declaration says that those stay visible), a chunked one the pages that lie wholly in finished chunks; a
+finished request gives back everything.
 
 With a prefix index (`enable_prefix`) full pages of tokens are shared between requests that start alike: `adopt` gives
 a new request the cached pages of its longest known prefix, `publish` hands the pages a request has filled to the
@@ -74,7 +75,9 @@ class CacheManager:
                 raise ValueError(f"run {site.run} declares two states of one name: {names}")
             for d in site_decls:
                 if isinstance(d, PagedState):
-                    key = (d.elems, d.window, d.dtype or dtype, d.keep_first if d.window > 0 else 0)
+                    if d.window > 0 and d.chunk > 0:
+                        raise ValueError(f"run {site.run}: state {d.name} has a window and chunks")
+                    key = (d.elems, d.window, d.dtype or dtype, d.keep_first if d.window > 0 else 0, d.chunk)
                     keyed.setdefault(key, []).append((site.run, d.name))
                 elif isinstance(d, SlotState):
                     t = torch.zeros((max_seqs + 1, *d.shape), dtype=d.dtype or dtype, device=device)
@@ -82,12 +85,12 @@ class CacheManager:
                     self.slot_states.append((site.run, d, t))
                 else:
                     raise TypeError(f"run {site.run}: unknown state declaration {d!r}")
-        for gid, ((elems, window, gdtype, keep_first), members) in enumerate(keyed.items()):
+        for gid, ((elems, window, gdtype, keep_first, chunk), members) in enumerate(keyed.items()):
             pool = PagePool(num_pages)
             storage = torch.zeros((len(members), num_pages, page_size * elems), dtype=gdtype, device=device)
             table = np.full((max_seqs + 1, self.max_pages), pool.null, dtype=np.int32)
             runs = sorted({run for run, _ in members})
-            group = PagedGroup(gid, PagedState("", elems, window, gdtype, keep_first), runs, members, pool, storage,
+            group = PagedGroup(gid, PagedState("", elems, window, gdtype, keep_first, chunk), runs, members, pool, storage,
                                table, torch.from_numpy(table.copy()).to(device), [0] * (max_seqs + 1),
                                [0] * (max_seqs + 1), kept=-(-keep_first // page_size))
             self.groups.append(group)
@@ -144,11 +147,11 @@ class CacheManager:
     # -- shared prefixes ------------------------------------------------------------------------------------------
     def enable_prefix(self, namespace: bytes) -> bool:
         """Share full pages between requests that start with the same tokens. Only state that a page holds whole can
-        be shared: with a windowed group (whose early pages go) or fixed-size state (which no page restores) nothing
+        be shared: with a windowed or chunked group (whose early pages go) or fixed-size state (which no page restores) nothing
         is, and this returns False."""
         if self._live:
             raise RuntimeError("the prefix index is set up before requests are admitted")
-        if not self.groups or self.slot_states or any(g.decl.window > 0 for g in self.groups):
+        if not self.groups or self.slot_states or any(g.decl.window > 0 or g.decl.chunk > 0 for g in self.groups):
             return False
         self.prefix = PrefixIndex(namespace, self.page_size, [g.pool for g in self.groups])
         return True
@@ -246,13 +249,14 @@ class CacheManager:
         return self._capacity[slot]
 
     def advance(self, slot: int, computed: int) -> None:
-        """The request now has `computed` tokens in the cache: pages a window has passed are given back."""
+        """The request now has `computed` tokens in the cache: pages that a window or the chunks have passed are given back."""
         self.computed[slot] = computed
         for g in self.groups:
-            w = g.decl.window
-            if w <= 0:
+            w, c = g.decl.window, g.decl.chunk
+            if w <= 0 and c <= 0:
                 continue
-            keep_from = max(0, computed - w + 1) // self.page_size      # the next query reads keys from computed-w+1
+            # the next query, at position `computed`, reads keys from computed-w+1 or from its chunk's first position
+            keep_from = (max(0, computed - w + 1) if w > 0 else computed - computed % c) // self.page_size
             keep_from = min(keep_from, g.count[slot])
             if keep_from > g.first[slot]:
                 gone = range(max(g.first[slot], g.kept), keep_from)      # the first tokens' pages stay

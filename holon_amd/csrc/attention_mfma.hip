@@ -48,7 +48,7 @@ struct AttnArgs {
   const int32_t* row_ids;  // rows this launch serves
   int heads, kv_heads, page_size;
   float scale_log2;        // scale * log2(e)
-  int window;
+  int window;              // what a query sees of the keys up to it: see first_seen
   // decode only
   float* part_o;           // [n_rows, Hq, splits, D]
   float* part_ml;          // [n_rows, Hq, splits, 2]
@@ -252,6 +252,12 @@ __device__ __forceinline__ void attn_tiles(const AttnArgs& a, const int32_t* __r
       f1[ks] = load8(krowp + 4 * D + ks * 32);
     }
   };
+  int seen_from[NT], whole_from[NT];           // the first key a lane's row sees, and the first that all of a tile's rows see
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    seen_from[t] = first_seen(qpos[t], a.window);
+    whole_from[t] = first_seen(tile_last[t], a.window);
+  }
   const int kb_first = (key_lo / 32) * 32;
   // the blocks of kept keys that lie wholly before key_lo's block come first: 0, 32, .. below kept_end, then kb_first on
   const int kept_end = MOD ? min((kept_keys + 31) / 32 * 32, kb_first) : 0;
@@ -319,9 +325,8 @@ __device__ __forceinline__ void attn_tiles(const AttnArgs& a, const int32_t* __r
         s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf1[ks], qf[t][ks], s1, 0, 0, 0);
       }
       const int qp = qpos[t];
-      const int first = a.window > 0 ? qp - a.window + 1 : 0;
-      const bool whole = kb + 31 <= tile_first[t] && kb >= key_lo && kb + 31 <= key_hi &&
-                         (a.window <= 0 || kb >= tile_last[t] - a.window + 1);
+      const int first = seen_from[t];
+      const bool whole = kb + 31 <= tile_first[t] && kb >= key_lo && kb + 31 <= key_hi && kb >= whole_from[t];
       if constexpr (SIG)
         sigmoid_block(s0, s1, whole, kb, g, qp, first, key_lo, key_hi, a.scale, sig_bias[t], pb[t], pl[t]);
       else if constexpr (MOD)
@@ -399,7 +404,7 @@ __global__ void __launch_bounds__(256) attn_prefill_kernel(AttnArgs a) {
     tile_last[t] = p0 < nq ? n - nq + last_qi : -1;
     tile_first[t] = n - nq + p0;
     key_hi = max(key_hi, tile_last[t]);
-    if (p0 < nq) key_lo = min(key_lo, a.window > 0 ? max(0, n - nq + p0 - a.window + 1) : 0);
+    if (p0 < nq) key_lo = min(key_lo, max(0, first_seen(n - nq + p0, a.window)));
     const bf16_t* qp = a.q + ((int64_t)rr[t].token * a.heads + rr[t].head) * D + 8 * g;
 #pragma unroll
     for (int ks = 0; ks < D / 32; ++ks) {
@@ -516,14 +521,14 @@ __global__ void __launch_bounds__(256) attn_prefill_lds_kernel(AttnArgs a) {
     const int range = pass == 0 ? (int)blockIdx.x : n_ranges - 1 - (int)blockIdx.x;
     if (pass == 1 && range <= (int)blockIdx.x) break;          // an odd count: the middle range was done in pass 0
     bf16x8_t qf[NT][D / 32];
-    int qpos[NT], tile_last[NT], tile_first[NT];
+    int qpos[NT], tile_last[NT], tile_first[NT], seen_from[NT], whole_from[NT];
     RowRef rr[NT];
     int key_hi = -1, key_lo = 0x7fffffff;                      // over the whole block (all waves walk the same stages)
     {
       const int p_lo = range * TPB * tm.pos_per_tile;
       const int p_hi = min(nq, p_lo + TPB * tm.pos_per_tile) - 1;
       key_hi = n - nq + p_hi;
-      key_lo = a.window > 0 ? max(0, n - nq + p_lo - a.window + 1) : 0;
+      key_lo = max(0, first_seen(n - nq + p_lo, a.window));
     }
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
@@ -533,6 +538,8 @@ __global__ void __launch_bounds__(256) attn_prefill_lds_kernel(AttnArgs a) {
       qpos[t] = rr[t].valid ? rr[t].qpos : -1;
       tile_last[t] = p0 < nq ? n - nq + min(nq, p0 + tm.pos_per_tile) - 1 : -1;
       tile_first[t] = n - nq + p0;
+      seen_from[t] = first_seen(qpos[t], a.window);
+      whole_from[t] = first_seen(tile_last[t], a.window);
       const bf16_t* qp = a.q + ((int64_t)rr[t].token * a.heads + rr[t].head) * D + 8 * g;
 #pragma unroll
       for (int ks = 0; ks < D / 32; ++ks) {
@@ -607,8 +614,8 @@ __global__ void __launch_bounds__(256) attn_prefill_lds_kernel(AttnArgs a) {
             s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf1[ks], qf[t][ks], s1, 0, 0, 0);
           }
           const int qp = qpos[t];
-          const int first = a.window > 0 ? qp - a.window + 1 : 0;
-          const bool whole = kb + 31 <= tile_first[t] && (a.window <= 0 || kb >= tile_last[t] - a.window + 1);
+          const int first = seen_from[t];
+          const bool whole = kb + 31 <= tile_first[t] && kb >= whole_from[t];
           pb[t] = softmax_block<D / 16>(s0, s1, whole, kb, g, qp, first, 0, 0x7fffffff, a.scale_log2, m[t], l[t], o[t]);
         }
 #pragma unroll
@@ -745,7 +752,7 @@ __global__ void __launch_bounds__(256, D == 128 ? 2 : 3) attn_prefill_wide_kerne
     const int p_lo = range * 4 * tm.pos_per_tile;
     const int p_hi = min(nq, p_lo + 4 * tm.pos_per_tile) - 1;
     const int key_hi = n - nq + p_hi;                          // over the whole block (all waves walk the same stages)
-    const int key_lo = a.window > 0 ? max(0, n - nq + p_lo - a.window + 1) : 0;
+    const int key_lo = max(0, first_seen(n - nq + p_lo, a.window));
     const int p0 = (range * 4 + wave) * tm.pos_per_tile;       // this wave's tile
     const int qi = p0 + pi;
     const bool valid = pi < tm.pos_per_tile && qi < nq && hi < group;
@@ -753,6 +760,7 @@ __global__ void __launch_bounds__(256, D == 128 ? 2 : 3) attn_prefill_wide_kerne
     const int qpos = valid ? n - nq + qi : -1;
     const int tile_last = p0 < nq ? n - nq + min(nq, p0 + tm.pos_per_tile) - 1 : -1;
     const int tile_first = n - nq + p0;
+    const int first = first_seen(qpos, a.window), whole_from = first_seen(tile_last, a.window);
     bf16x8_t qf[D / 16];
     {
       const bf16_t* qp = a.q + ((int64_t)token * a.heads + head) * D + 8 * h;
@@ -826,8 +834,7 @@ __global__ void __launch_bounds__(256, D == 128 ? 2 : 3) attn_prefill_wide_kerne
           }
         }
         // value idx = 4i + r of this lane is key kb + 16*(i/2) + 8h + 4*(i%2) + r against query column c
-        const int first = a.window > 0 ? qpos - a.window + 1 : 0;
-        const bool whole = kb + 31 <= tile_first && (a.window <= 0 || kb >= tile_last - a.window + 1);
+        const bool whole = kb + 31 <= tile_first && kb >= whole_from;
         float sv[16];
 #pragma unroll
         for (int idx = 0; idx < 16; ++idx) sv[idx] = sc[idx];
@@ -1096,7 +1103,7 @@ __global__ void __launch_bounds__(256, 2) attn_prefill_dma_kernel(AttnArgs a) {
     const int p_lo = range * 4 * tm.pos_per_tile;
     const int p_hi = min(nq, p_lo + 4 * tm.pos_per_tile) - 1;
     const int key_hi = n - nq + p_hi;                          // over the whole block (all waves walk the same stages)
-    const int key_lo = a.window > 0 ? max(0, n - nq + p_lo - a.window + 1) : 0;
+    const int key_lo = max(0, first_seen(n - nq + p_lo, a.window));
     const int p0 = (range * 4 + wave) * tm.pos_per_tile;       // this wave's tile
     const int qi = p0 + pi;
     const bool valid = pi < tm.pos_per_tile && qi < nq && hi < group;
@@ -1104,6 +1111,7 @@ __global__ void __launch_bounds__(256, 2) attn_prefill_dma_kernel(AttnArgs a) {
     const int qpos = valid ? n - nq + qi : -1;
     const int tile_last = p0 < nq ? n - nq + min(nq, p0 + tm.pos_per_tile) - 1 : -1;
     const int tile_first = n - nq + p0;
+    const int first = first_seen(qpos, a.window), whole_from = first_seen(tile_last, a.window);
     bf16x8_t qf[D / 16];
     {
       const bf16_t* qp = a.q + ((int64_t)token * a.heads + head) * D + 8 * h;
@@ -1147,8 +1155,7 @@ __global__ void __launch_bounds__(256, 2) attn_prefill_dma_kernel(AttnArgs a) {
           }
         }
         // value idx = 4i + r of this lane is key kb + 16*(i/2) + 8h + 4*(i%2) + r against query column c
-        const int first = a.window > 0 ? qpos - a.window + 1 : 0;
-        const bool whole = kb + 31 <= tile_first && (a.window <= 0 || kb >= tile_last - a.window + 1);
+        const bool whole = kb + 31 <= tile_first && kb >= whole_from;
         float sv[16];
 #pragma unroll
         for (int idx = 0; idx < 16; ++idx) sv[idx] = sc[idx];
@@ -1283,9 +1290,9 @@ __global__ void __launch_bounds__(256, 1) attn_prefill_pair_kernel(AttnArgs a) {
     const int p_lo = range * TPB * tm.pos_per_tile;
     const int p_hi = min(nq, p_lo + TPB * tm.pos_per_tile) - 1;
     const int key_hi = n - nq + p_hi;                          // over the whole block (all waves walk the same stages)
-    const int key_lo = a.window > 0 ? max(0, n - nq + p_lo - a.window + 1) : 0;
+    const int key_lo = max(0, first_seen(n - nq + p_lo, a.window));
     bool valid[2];
-    int token[2], qpos[2], tile_last[2], tile_first[2];
+    int token[2], qpos[2], tile_last[2], tile_first[2], seen_from[2];
     const int head = hk * group + hi;
     bf16x8_t qf[2][D / 16];
 #pragma unroll
@@ -1295,6 +1302,7 @@ __global__ void __launch_bounds__(256, 1) attn_prefill_pair_kernel(AttnArgs a) {
       valid[t] = pi < tm.pos_per_tile && qi < nq && hi < group;
       token[t] = qs + qi;
       qpos[t] = valid[t] ? n - nq + qi : -1;
+      seen_from[t] = first_seen(qpos[t], a.window);
       tile_last[t] = p0 < nq ? n - nq + min(nq, p0 + tm.pos_per_tile) - 1 : -1;
       tile_first[t] = n - nq + p0;
       const bf16_t* qp = a.q + ((int64_t)token[t] * a.heads + head) * D + 8 * h;
@@ -1388,7 +1396,7 @@ __global__ void __launch_bounds__(256, 1) attn_prefill_pair_kernel(AttnArgs a) {
         float m_new, psum;
         bf16x8_t pb0, pb1;
         if (on0) {
-          scores_to_probs<MASK>(sc0, kb, h, qpos[0], a.window > 0 ? qpos[0] - a.window + 1 : 0, a.scale_log2, m[0],
+          scores_to_probs<MASK>(sc0, kb, h, qpos[0], seen_from[0], a.scale_log2, m[0],
                                 m_new, psum, pb0, pb1);
           if constexpr (!MASK) {     // the second tile's score products, one at a time between the first tile's exponentials
             __builtin_amdgcn_sched_group_barrier(0x008, D / 16, 0);
@@ -1406,7 +1414,7 @@ __global__ void __launch_bounds__(256, 1) attn_prefill_pair_kernel(AttnArgs a) {
           }
         }
         if (on1) {
-          scores_to_probs<MASK>(sc1, kb, h, qpos[1], a.window > 0 ? qpos[1] - a.window + 1 : 0, a.scale_log2, m[1],
+          scores_to_probs<MASK>(sc1, kb, h, qpos[1], seen_from[1], a.scale_log2, m[1],
                                 m_new, psum, pb0, pb1);
           if constexpr (!MASK) {     // the first tile's value products between the second tile's exponentials
 #pragma unroll
@@ -1430,9 +1438,9 @@ __global__ void __launch_bounds__(256, 1) attn_prefill_pair_kernel(AttnArgs a) {
       }
     };
     // a stage is unmasked when every row of both tiles sees all of it: it ends at or before the first tile's first
-    // position, and there is no window
+    // position, and neither a window nor chunks hide anything
     auto step = [&](auto last, int kb, int buf, Regs& next) {
-      if (a.window <= 0 && kb + 31 <= tile_first[0]) stage(std::false_type{}, last, kb, buf, next);
+      if (a.window == 0 && kb + 31 <= tile_first[0]) stage(std::false_type{}, last, kb, buf, next);
       else stage(std::true_type{}, last, kb, buf, next);
     };
     const int kb_first = (key_lo / 32) * 32;
@@ -1594,7 +1602,7 @@ __global__ void __launch_bounds__(512) attn_decode_kernel(AttnArgs a, FusedArgs 
   const RowRef rr = row_ref(tm, c, 0, hb, hk, group, qs, 1, n);
   // the keys this row can see, cut into `splits` ranges of keys_per_split
   const int qp_row = n - 1;
-  const int first = a.window > 0 ? max(0, qp_row - a.window + 1) : 0;
+  const int first = max(0, first_seen(qp_row, a.window));
   // every split gets an equal share of this row's own keys (a multiple of 32), whatever length the launch was
   // shaped for: a row shorter than the longest one still keeps all its waves busy
   const int base = (first / 32) * 32;
@@ -1893,7 +1901,7 @@ static int prefill_launch(const void* q, void* out, const void* pages, const int
                           int v_share = 1, const void* hgate = nullptr, int64_t hgate_stride = 0) {
   HOLON_CHECK(mfma_serves(head_dim, page_size), "attention (matrix cores): head_dim %d / page %d not served", head_dim,
               page_size);
-  HOLON_CHECK(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && window >= 0 && table_stride > 0,
+  HOLON_CHECK(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && window > -0x7fffffff && table_stride > 0,
               "attention: bad sizes");
   HOLON_CHECK(v_share >= 1 && kv_heads % v_share == 0, "attention: %d key heads do not share value heads by %d", kv_heads,
               v_share);
@@ -1913,7 +1921,7 @@ static int prefill_launch(const void* q, void* out, const void* pages, const int
                 "attention: a cap of %g, %d kept tokens, a distance bias of two numbers a head", mod->softcap,
                 mod->keep_first);
     a.scale = scale; a.softcap = mod->softcap; a.r1 = mod->r1; a.r2 = mod->r2; a.keep_first = mod->keep_first;
-    const int mnt = head_dim == 256 || window > 0 ? 1 : 2;
+    const int mnt = head_dim == 256 || window != 0 ? 1 : 2;
     dim3 grid(((tiles + mnt - 1) / mnt + 3) / 4, kv_heads * tm.head_blocks, n_rows);
     hipStream_t ms = (hipStream_t)stream;
     if (head_dim == 64) { if (mnt == 1) attn_prefill_kernel<64, 1, true><<<grid, 256, 0, ms>>>(a); else attn_prefill_kernel<64, 2, true><<<grid, 256, 0, ms>>>(a); }
@@ -2066,7 +2074,7 @@ static int decode_launch(const void* q, void* out, const void* pages, const int3
                          const void* hgate = nullptr, int64_t hgate_stride = 0) {
   HOLON_CHECK(mfma_serves(head_dim, page_size), "attention (matrix cores): head_dim %d / page %d not served", head_dim,
               page_size);
-  HOLON_CHECK(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && window >= 0 && table_stride > 0,
+  HOLON_CHECK(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && window > -0x7fffffff && table_stride > 0,
               "attention: bad sizes");
   HOLON_CHECK(v_share >= 1 && kv_heads % v_share == 0 && ((v_share == 1 && hgate == nullptr) || fused == nullptr),
               "attention: %d key heads do not share value heads by %d", kv_heads, v_share);
@@ -2079,8 +2087,9 @@ static int decode_launch(const void* q, void* out, const void* pages, const int3
               "partials within 64 KB of LDS)", waves, splits, head_dim);
   HOLON_CHECK(splits == waves || (part_o && part_ml), "attention decode: %d splits over blocks need a workspace",
               splits / waves);
-  // (a window's keys are walked from a 32-key border on, and never more keys than the longest row holds)
-  const int span = window > 0 && window + 31 < max_len ? window + 31 : max_len;
+  // (a window's or chunk's keys are walked from a 32-key border on, and never more keys than the longest row holds)
+  const int reach = window < 0 ? -window : window;
+  const int span = reach > 0 && reach < max_len - 31 ? reach + 31 : max_len;
   HOLON_CHECK((int64_t)splits * keys_per_split >= span, "attention decode: %d splits of %d keys do not cover %d keys",
               splits, keys_per_split, span);
   if (n_rows <= 0) return 0;

@@ -35,6 +35,20 @@ template <> __device__ __forceinline__ float silu<bf16_t>(float g) {
   return g * __builtin_amdgcn_rcpf(1.0f + __expf(-g));
 }
 
+// The tanh form of gelu, 0.5 z (1 + tanh(u)) with u = sqrt(2 / pi) (z + 0.044715 z^3), as z sigmoid(2 u): the same number
+// with one exponential and no difference of near-equal ones.
+template <typename T> __device__ __forceinline__ float gelu_tanh(float z) {
+  const float two_u = 1.5957691216057308f * (z + 0.044715f * z * z * z);
+  if constexpr (sizeof(T) == 4) return z / (1.0f + expf(-two_u));
+  else return z * __builtin_amdgcn_rcpf(1.0f + __expf(-two_u));
+}
+
+// A gated feed-forward's activation: 0 silu, 1 gelu in its tanh form.
+template <int ACT, typename T> __device__ __forceinline__ float gate_act(float z) {
+  if constexpr (ACT == 1) return gelu_tanh<T>(z);
+  else return silu<T>(z);
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = WAVE / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, WAVE);
@@ -81,6 +95,12 @@ __device__ __forceinline__ void wait_loads_but() {          // until at most N o
   __builtin_amdgcn_s_waitcnt((N & 15) | ((N >> 4) << 14) | (7 << 4) | (15 << 8));
 }
 
+// The first key that the query at position `pos` sees: window 0: key 0; w > 0: the last w keys (what is returned may lie
+// before key 0); w < 0: the query's own chunk of -w positions, chunks counted from position 0. It never falls as `pos`
+// grows, so the first query of a tile says where its keys begin and the last one from where all of its queries see them.
+__device__ __forceinline__ int first_seen(int pos, int window) {
+  return window > 0 ? pos - window + 1 : (window < 0 && pos > 0 ? pos - pos % -window : 0);
+}
 
 // Host side: every entry point returns 0 or a negative code and leaves a message for holon_last_error().
 void holon_set_error(const char* fmt, ...);

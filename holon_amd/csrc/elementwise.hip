@@ -324,22 +324,22 @@ extern "C" int holon_rmsnorm_parts(const float* parts, int splits, void* residua
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-template <typename T>
-__global__ void silu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int64_t tokens, int inter) {
+template <typename T, int ACT>
+__global__ void gated_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int64_t tokens, int inter) {
   const int64_t n = tokens * inter;
   for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x) {
     const int64_t t = i / inter;
     const int c = (int)(i - t * inter);
     const float g = Elem<T>::load(gu[t * 2 * inter + c]);
     const float u = Elem<T>::load(gu[t * 2 * inter + inter + c]);
-    const float s = Elem<T>::round(silu<T>(g));
+    const float s = Elem<T>::round(gate_act<ACT, T>(g));
     out[i] = Elem<T>::store(s * u);
   }
 }
 
 // 16 bytes of gate and 16 bytes of up per thread (widths that are multiples of the vector).
-template <typename T>
-__global__ void silu_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int64_t tokens, int inter) {
+template <typename T, int ACT>
+__global__ void gated_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int64_t tokens, int inter) {
   constexpr int V = Elem<T>::kVec;
   const int per_row = inter / V;
   const int64_t n = tokens * per_row;
@@ -355,15 +355,16 @@ __global__ void silu_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ ou
 #pragma unroll
     for (int j = 0; j < V; ++j) {
       const float g = Elem<T>::load(ge[j]);
-      const float sg = Elem<T>::round(silu<T>(g));
+      const float sg = Elem<T>::round(gate_act<ACT, T>(g));
       oe[j] = Elem<T>::store(sg * Elem<T>::load(ue[j]));
     }
     *reinterpret_cast<uint4*>(out + t * inter + c) = oraw;
   }
 }
 
-extern "C" int holon_silu_mul(const void* gate_up, void* out, int64_t tokens, int inter, int dtype, void* stream) {
-  HOLON_CHECK(tokens >= 0 && inter > 0, "silu_mul: bad sizes");
+template <int ACT>
+static int gated_mul(const void* gate_up, void* out, int64_t tokens, int inter, int dtype, void* stream) {
+  HOLON_CHECK(tokens >= 0 && inter > 0, "gated activation: bad sizes");
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   const int vec = dtype == HOLON_F32 ? 4 : 8;
@@ -371,20 +372,28 @@ extern "C" int holon_silu_mul(const void* gate_up, void* out, int64_t tokens, in
     const int64_t nv = tokens * (inter / vec);
     const unsigned vgrid = (unsigned)((nv + 255) / 256 < 16384 ? (nv + 255) / 256 : 16384);
     if (dtype == HOLON_F32)
-      silu_mul_vec_kernel<float><<<vgrid, 256, 0, s>>>((const float*)gate_up, (float*)out, tokens, inter);
+      gated_mul_vec_kernel<float, ACT><<<vgrid, 256, 0, s>>>((const float*)gate_up, (float*)out, tokens, inter);
     else
-      silu_mul_vec_kernel<bf16_t><<<vgrid, 256, 0, s>>>((const bf16_t*)gate_up, (bf16_t*)out, tokens, inter);
+      gated_mul_vec_kernel<bf16_t, ACT><<<vgrid, 256, 0, s>>>((const bf16_t*)gate_up, (bf16_t*)out, tokens, inter);
     HOLON_LAUNCH_OK();
     return 0;
   }
   const int64_t n = tokens * inter;
   const unsigned grid = (unsigned)((n + 255) / 256 < 65536 ? (n + 255) / 256 : 65536);
   if (dtype == HOLON_F32)
-    silu_mul_kernel<float><<<grid, 256, 0, s>>>((const float*)gate_up, (float*)out, tokens, inter);
+    gated_mul_kernel<float, ACT><<<grid, 256, 0, s>>>((const float*)gate_up, (float*)out, tokens, inter);
   else
-    silu_mul_kernel<bf16_t><<<grid, 256, 0, s>>>((const bf16_t*)gate_up, (bf16_t*)out, tokens, inter);
+    gated_mul_kernel<bf16_t, ACT><<<grid, 256, 0, s>>>((const bf16_t*)gate_up, (bf16_t*)out, tokens, inter);
   HOLON_LAUNCH_OK();
   return 0;
+}
+
+extern "C" int holon_silu_mul(const void* gate_up, void* out, int64_t tokens, int inter, int dtype, void* stream) {
+  return gated_mul<0>(gate_up, out, tokens, inter, dtype, stream);
+}
+
+extern "C" int holon_gelu_mul(const void* gate_up, void* out, int64_t tokens, int inter, int dtype, void* stream) {
+  return gated_mul<1>(gate_up, out, tokens, inter, dtype, stream);
 }
 
 // ---------------------------------------------------------------------------------------------------------------

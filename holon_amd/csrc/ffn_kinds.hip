@@ -219,8 +219,8 @@ __global__ void __launch_bounds__(256) moe_gate_kernel(const T* __restrict__ gat
   }
 }
 // The other router, one block of 256 threads a token: float32 logits z_e = x . router[e] + bias[e]; the `top` largest
-// are chosen (equal ones: the lower index first) and weighted by the softmax over the chosen logits alone, every other
-// expert 0. `groups` > 1: only experts of the `keep` groups of neighbours whose largest logits are best can be chosen
+// are chosen (equal ones: the lower index first) and weighted by the softmax over the chosen logits alone, or (`score` 1)
+// by each one's own sigmoid, or (`score` 2) by that sigmoid squared; every other expert 0. `groups` > 1: only experts of the `keep` groups of neighbours whose largest logits are best can be chosen
 // (equal groups: the lower one). Rows of `router` beyond the experts are gates: their columns hold sigmoid(x . router[r]).
 // Every thread takes a slice of the token's row against all router rows, sixteen rows at a time (their loads do not
 // wait for each other); a wave's lanes are summed by shuffles and the four waves' partial sums in wave order. Up to 64
@@ -229,7 +229,7 @@ template <typename T>
 __global__ void __launch_bounds__(256) moe_router_top_kernel(const T* __restrict__ x, const float* __restrict__ router,
                                                              const float* __restrict__ bias, float* __restrict__ weights,
                                                              int width, int experts, int rows_r, int top, int groups,
-                                                             int keep) {
+                                                             int keep, int score) {
   __shared__ float part_s[4][ROUTE_MAX_E + 1];
   __shared__ float z_s[ROUTE_MAX_E + 1];
   __shared__ float e_s[ROUTE_MAX_E];
@@ -297,6 +297,12 @@ __global__ void __launch_bounds__(256) moe_router_top_kernel(const T* __restrict
       const float other = __shfl(mine, o, WAVE);
       ahead += (other > mine) || (other == mine && o < lane);
     }
+    if (score) {
+      const float s = lane < experts && ahead < top && mine > -INFINITY ? 1.0f / (1.0f + expf(-mine)) : 0.f;
+      if (lane < experts) weights[t * rows_r + lane] = score == 2 ? s * s : s;
+      if (rows_r > experts && lane == 0) weights[t * rows_r + experts] = 1.0f / (1.0f + expf(-logit(experts)));
+      return;
+    }
     const float top_z = wave_max(mine);                   // the largest logit is always chosen
     const float v = lane < experts && ahead < top && mine > -INFINITY ? expf(mine - top_z) : 0.f;
     const float sum = wave_sum(v);
@@ -334,16 +340,49 @@ __global__ void __launch_bounds__(256) moe_router_top_kernel(const T* __restrict
     const float mine = z_s[e];
     int ahead = 0;
     for (int o = 0; o < experts; ++o) ahead += (z_s[o] > mine) || (z_s[o] == mine && o < e);
-    const float v = ahead < top && mine > -INFINITY ? expf(mine - top_z) : 0.f;
-    e_s[e] = v;
+    float v = 0.f;
+    if (ahead < top && mine > -INFINITY) v = score ? 1.0f / (1.0f + expf(-mine)) : expf(mine - top_z);
+    e_s[e] = score == 2 ? v * v : v;
     part += v;
   }
   part = wave_sum(part);
   if (lane == 0) red_s[wave] = part;
   __syncthreads();
-  const float sum = ((red_s[0] + red_s[1]) + red_s[2]) + red_s[3];
+  const float sum = score ? 1.0f : ((red_s[0] + red_s[1]) + red_s[2]) + red_s[3];
   for (int e = threadIdx.x; e < rows_r; e += 256)
     weights[t * rows_r + e] = e < experts ? e_s[e] / sum : 1.0f / (1.0f + expf(-z_s[e]));
+}
+
+// y[t, c] = max(up[t, c], 0)^2 times the weight of the column's expert, float32 inside and one rounding, 0 where that
+// weight is 0 (columns and weights as for moe_gate_kernel, without gates).
+template <typename T, bool VEC>
+__global__ void __launch_bounds__(256) moe_relu2_kernel(const T* __restrict__ up, const float* __restrict__ weights,
+                                                        T* __restrict__ y, int experts, int ff, int shared, int wstride,
+                                                        int shared_col) {
+  const int cols = experts * ff + shared;
+  const int64_t t = blockIdx.y;
+  constexpr int N = VEC ? Elem<T>::kVec : 1;
+  for (int c = (blockIdx.x * 256 + threadIdx.x) * N; c < cols; c += gridDim.x * 256 * N) {
+    const float w = c < experts * ff ? weights[t * wstride + c / ff]
+                                     : (shared_col >= 0 ? weights[t * wstride + shared_col] : 1.0f);
+    if constexpr (VEC) {
+      uint4 out = make_uint4(0u, 0u, 0u, 0u);
+      if (w != 0.f) {
+        const uint4 raw = *reinterpret_cast<const uint4*>(up + t * cols + c);
+        const T* in = reinterpret_cast<const T*>(&raw);
+        T* o = reinterpret_cast<T*>(&out);
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+          const float v = fmaxf(Elem<T>::load(in[i]), 0.f);
+          o[i] = Elem<T>::store(v * v * w);
+        }
+      }
+      *reinterpret_cast<uint4*>(y + t * cols + c) = out;
+    } else {
+      const float v = fmaxf(Elem<T>::load(up[t * cols + c]), 0.f);
+      y[t * cols + c] = Elem<T>::store(w != 0.f ? v * v * w : 0.f);
+    }
+  }
 }
 
 template <typename T, bool VEC>
@@ -458,22 +497,49 @@ extern "C" int holon_moe_gate(const void* gate_up, const float* weights, void* y
 
 extern "C" int holon_moe_router_top(const void* x, const float* router, const float* bias, float* weights, int64_t rows,
                                     int width, int experts, int router_rows, int top, int dtype, int groups, int keep,
-                                    void* stream) {
+                                    int score, void* stream) {
   HOLON_CHECK(rows >= 0 && rows <= 0x7fffffffLL && width >= 1 && width <= 12288 && experts >= 1 &&
                   experts <= ROUTE_MAX_E && top >= 1 && top <= experts &&
                   (router_rows == experts || router_rows == experts + 1),
               "moe_router_top: rows=%lld of %d (at most 12,288), top %d of %d experts (at most %d), %d router rows",
               (long long)rows, width, top, experts, ROUTE_MAX_E, router_rows);
+  HOLON_CHECK(score >= 0 && score <= 2, "moe_router_top: no score %d", score);
   HOLON_CHECK(groups <= 1 || (experts % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (experts / groups)),
               "moe_router_top: top %d of %d experts in %d groups of which %d stay open", top, experts, groups, keep);
   if (rows == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   if (dtype == HOLON_F32)
     moe_router_top_kernel<float><<<(unsigned)rows, 256, 0, s>>>((const float*)x, router, bias, weights, width, experts,
-                                                               router_rows, top, groups, keep);
+                                                               router_rows, top, groups, keep, score);
   else
     moe_router_top_kernel<bf16_t><<<(unsigned)rows, 256, 0, s>>>((const bf16_t*)x, router, bias, weights, width,
-                                                                experts, router_rows, top, groups, keep);
+                                                                experts, router_rows, top, groups, keep, score);
+  HOLON_LAUNCH_OK();
+  return 0;
+}
+
+extern "C" int holon_moe_relu2(const void* up, const float* weights, void* y, int64_t rows, int experts, int ff, int shared,
+                               int dtype, int wstride, int shared_col, void* stream) {
+  HOLON_CHECK(rows >= 0 && rows <= 65535 * 1024LL && experts >= 1 && ff >= 1 && shared >= 0,
+              "moe_relu2: rows=%lld, %d experts of %d, %d shared columns", (long long)rows, experts, ff, shared);
+  HOLON_CHECK(wstride >= experts && shared_col < wstride, "moe_relu2: weight rows of %d for %d experts, column %d", wstride,
+              experts, shared_col);
+  if (rows == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  const int cols = experts * ff + shared;
+  const int vec = dtype == HOLON_F32 ? 4 : 8;
+  const bool wide = ff % vec == 0 && shared % vec == 0 && (uintptr_t)up % 16 == 0 && (uintptr_t)y % 16 == 0;
+  const int groups = wide ? cols / vec : cols;
+  for (int64_t r0 = 0; r0 < rows; r0 += 65535) {
+    const int n = (int)(rows - r0 < 65535 ? rows - r0 : 65535);
+    const dim3 grid((groups + 255) / 256 < 64 ? (groups + 255) / 256 : 64, n);
+#define MOE_RELU2(T, V)                                                                                                \
+  moe_relu2_kernel<T, V><<<grid, 256, 0, s>>>((const T*)up + r0 * cols, weights + r0 * wstride, (T*)y + r0 * cols, experts, \
+                                              ff, shared, wstride, shared_col)
+    if (dtype == HOLON_F32) { if (wide) MOE_RELU2(float, true); else MOE_RELU2(float, false); }
+    else { if (wide) MOE_RELU2(bf16_t, true); else MOE_RELU2(bf16_t, false); }
+#undef MOE_RELU2
+  }
   HOLON_LAUNCH_OK();
   return 0;
 }

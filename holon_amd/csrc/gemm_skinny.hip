@@ -312,9 +312,9 @@ extern "C" int holon_gemm_skinny_add_bf16(const void* x, const void* w_tiled, vo
   return 0;
 }
 
-// The gated form: w = [gate rows; up rows] (2I rows), y[M, I] = round(silu(round(x gate^T))) * round(x up^T), the
-// roundings of the two-kernel composition. A block owns gate tile t and up tile t + I/16 and streams both.
-template <int WPB, int UNROLL, bool TILED>
+// The gated form: w = [gate rows; up rows] (2I rows), y[M, I] = round(act(round(x gate^T))) * round(x up^T), act silu or
+// (ACT 1) the tanh form of gelu, the roundings of the two-kernel composition. A block owns gate tile t and up tile t + I/16 and streams both.
+template <int WPB, int UNROLL, bool TILED, int ACT>
 __global__ void __launch_bounds__(WPB * 64) gemm_skinny_glu_kernel(const bf16_t* __restrict__ x,
                                                                     const bf16_t* __restrict__ w,
                                                                     bf16_t* __restrict__ y, int M, int I, int K,
@@ -399,7 +399,7 @@ __global__ void __launch_bounds__(WPB * 64) gemm_skinny_glu_kernel(const bf16_t*
   for (int r = 0; r < 4; ++r) {
     const float gate = bf16_to_float(float_to_bf16(acc[0][r]));
     const float up = bf16_to_float(float_to_bf16(acc[1][r]));
-    const float sg = bf16_to_float(float_to_bf16(silu<bf16_t>(gate)));
+    const float sg = bf16_to_float(float_to_bf16(gate_act<ACT, bf16_t>(gate)));
     oe[r] = float_to_bf16(sg * up);
   }
   *reinterpret_cast<ushort4*>(y + (int64_t)c * I + n0 + 4 * g) = o;
@@ -407,8 +407,9 @@ __global__ void __launch_bounds__(WPB * 64) gemm_skinny_glu_kernel(const bf16_t*
 
 // `stats` (nullable, with `parts` and `eps`): x holds un-normed rows and `w` the tiled weights with the norm's weight
 // folded in; rows are scaled as in holon_gemm_skinny_scaled_bf16 (tiled).
-extern "C" int holon_gemm_skinny_glu_bf16(const void* x, const void* w, void* y, int M, int I, int K, int tiled,
-                                          const float* stats, int parts, float eps, void* stream) {
+template <int ACT>
+static int skinny_glu(const void* x, const void* w, void* y, int M, int I, int K, int tiled, const float* stats, int parts,
+                      float eps, void* stream) {
   HOLON_CHECK(M >= 1 && M <= 16 && I % 16 == 0 && K % 128 == 0, "gated gemm (few rows): M=%d I=%d K=%d not served", M, I, K);
   HOLON_CHECK(stats == nullptr || (tiled && parts >= 1), "gated gemm (few rows, folded norm): tiled=%d parts=%d", tiled, parts);
   const RowScale rs{stats, parts, eps, 1.0f / (float)K};
@@ -416,14 +417,25 @@ extern "C" int holon_gemm_skinny_glu_bf16(const void* x, const void* w, void* y,
   const bool few = I / 16 < 512;   // few tile pairs: four waves share each; otherwise two (measured at 768 pairs, K 4096:
                                    // 33 us against 36 for one wave a pair at 1 and 8 rows, the same at 16)
 #define GLU(WPB, U)                                                                                              \
-  if (tiled) gemm_skinny_glu_kernel<WPB, U, true><<<I / 16, WPB * 64, 0, s>>>((const bf16_t*)x, (const bf16_t*)w, \
+  if (tiled) gemm_skinny_glu_kernel<WPB, U, true, ACT><<<I / 16, WPB * 64, 0, s>>>((const bf16_t*)x, (const bf16_t*)w, \
                                                                              (bf16_t*)y, M, I, K, rs);           \
-  else gemm_skinny_glu_kernel<WPB, U, false><<<I / 16, WPB * 64, 0, s>>>((const bf16_t*)x, (const bf16_t*)w,      \
+  else gemm_skinny_glu_kernel<WPB, U, false, ACT><<<I / 16, WPB * 64, 0, s>>>((const bf16_t*)x, (const bf16_t*)w,      \
                                                                         (bf16_t*)y, M, I, K, rs)
   if (few) { GLU(4, 8); } else { GLU(2, 8); }
 #undef GLU
   HOLON_LAUNCH_OK();
   return 0;
+}
+
+extern "C" int holon_gemm_skinny_glu_bf16(const void* x, const void* w, void* y, int M, int I, int K, int tiled,
+                                          const float* stats, int parts, float eps, void* stream) {
+  return skinny_glu<0>(x, w, y, M, I, K, tiled, stats, parts, eps, stream);
+}
+
+// The same with the tanh form of gelu in place of silu.
+extern "C" int holon_gemm_skinny_geglu_bf16(const void* x, const void* w, void* y, int M, int I, int K, int tiled,
+                                            void* stream) {
+  return skinny_glu<1>(x, w, y, M, I, K, tiled, nullptr, 0, 0.f, stream);
 }
 
 // tiled[t][s][l][e] = w[16 t + l % 16][32 s + 8 (l / 16) + e]: the layout the few-row product streams.

@@ -25,6 +25,8 @@ int holon_rmsnorm(const void* x, void* residual, const void* weight, void* y, in
 int holon_rmsnorm_parts(const float* parts, int splits, void* residual, const void* weight, void* y, int64_t rows,
                         int dim, float eps, void* stream);
 int holon_silu_mul(const void* gate_up, void* out, int64_t tokens, int inter, int dtype, void* stream);
+// The same with the tanh form of gelu.
+int holon_gelu_mul(const void* gate_up, void* out, int64_t tokens, int inter, int dtype, void* stream);
 // Per (token, head): optional rmsnorm over head_dim, optional half-split rotation with table[pos] = cos|sin, then
 // q -> q_out [T, heads, D]; k, v -> the paged cache (pages == NULL: only q heads are processed).
 int holon_qk_norm_rope_write(const void* qkv, int64_t qkv_stride, void* q_out, int tokens, int heads, int kv_heads,
@@ -149,6 +151,7 @@ int holon_gemm_skinny_scaled_bf16(const void* x, const void* w_tiled, void* y, i
 // stats (nullable): as in holon_gemm_skinny_scaled_bf16 (tiled weights with the norm's weight folded in).
 int holon_gemm_skinny_glu_bf16(const void* x, const void* w, void* y, int M, int I, int K, int tiled, const float* stats,
                                int parts, float eps, void* stream);
+int holon_gemm_skinny_geglu_bf16(const void* x, const void* w, void* y, int M, int I, int K, int tiled, void* stream);
 // The same products for 17 <= M <= 64 rows over tiled weights with many tiles (N / 16 a multiple of 8 and at least
 // 1,024; K a multiple of 256): the rows of activations go through LDS, shared by a block's waves, and every wave sums
 // its tile over all of K in order. `gated`: N is I and the weight has 2 I rows.
@@ -202,6 +205,8 @@ int holon_logprobs(const float* logits, const int32_t* tokens, int rows, int voc
 // -- a float32 residual stream (stream32.hip) ---------------------------------------------------------------------------
 // y[i] = x[i] as float32 (x float32 or bfloat16): a new copy.
 int holon_widen_rows(const void* x, float* y, int64_t n, int dtype, void* stream);
+// y[i] = x[i] rounded to `dtype`.
+int holon_narrow_rows(const float* x, void* y, int64_t n, int dtype, void* stream);
 // x32 [rows, dim] += s1 d1 + s2 d2 in place (d1, d2 nullable, each float32 or bfloat16 by dt1, dt2); then, with
 // weight and y (both or neither): y = (x - mean) / sqrt(var + eps) * weight, weight and y of dtype dt_out.
 int holon_stream_norm(float* x32, const void* d1, float s1, int dt1, const void* d2, float s2, int dt2,
@@ -369,9 +374,11 @@ int holon_stream_rms_filter(float* x32, const void* d1, int dt1, const void* d2,
                             const void* w1, const void* w2, int dtw, void* y1, void* y2, int64_t rows, int dim,
                             float eps, int dt_out, const void* cw1, const void* cw2, void* held1, void* held2,
                             const int32_t* slots, const int32_t* starts, int taps, void* stream);
-// x32 [rows, dim] += gain term / sqrt(mean(term^2) + term_eps) in place; y = x / sqrt(mean(x^2) + eps) * w.
+// x32 [rows, dim] += gain term / sqrt(mean(term^2) + term_eps) in place; y = x / sqrt(mean(x^2) + eps) * w (w null: y =
+// x). With `second` (nullable) the term is s1 term + s2 second + mix_row (nullable, [dim] float32), formed in float32.
 int holon_stream_rms_post(float* x32, const void* term, int dtt, const float* gain, float term_eps, const void* w, int dtw,
-                          void* y, int64_t rows, int dim, float eps, int dt_out, void* stream);
+                          void* y, int64_t rows, int dim, float eps, int dt_out, const void* second, float s1, float s2,
+                          const float* mix_row, void* stream);
 // y[i] = scale * x[i] as float32 (x float32 or bfloat16): a new copy.
 int holon_scale_rows(const void* x, float* y, int64_t n, int dtype, float scale, void* stream);
 
@@ -394,9 +401,13 @@ int holon_moe_gate(const void* gate_up, const float* weights, void* y, int64_t r
                    int dtype, int wstride, int shared_col, void* stream);
 // The other router: logits x . router[e] + bias[e] (nullable), the `top` largest chosen, weights the softmax over the
 // chosen logits alone; router rows beyond the experts (none or one) are gates: their columns hold a sigmoid. groups > 1:
-// chosen among the `keep` groups of neighbours with the best largest logits. weights [rows, router_rows].
+// chosen among the `keep` groups of neighbours with the best largest logits. weights [rows, router_rows]. score 1: the
+// weights are the chosen logits' own sigmoids, 2: their squares.
 int holon_moe_router_top(const void* x, const float* router, const float* bias, float* weights, int64_t rows, int width,
-                         int experts, int router_rows, int top, int dtype, int groups, int keep, void* stream);
+                         int experts, int router_rows, int top, int dtype, int groups, int keep, int score, void* stream);
+// up [rows, C], C = experts ff + shared: y = max(up, 0)^2 times the weight of the column's expert (as for holon_moe_gate).
+int holon_moe_relu2(const void* up, const float* weights, void* y, int64_t rows, int experts, int ff, int shared, int dtype,
+                    int wstride, int shared_col, void* stream);
 // y = max(z, 0)^2 over n values.
 int holon_relu2(const void* z, void* y, int64_t n, int dtype, void* stream);
 
@@ -433,6 +444,35 @@ int holon_ssd_scan(const void* xbc, const void* dt, int64_t dt_stride, const flo
 // of rows gate_stride apart.
 int holon_gated_parts_norm(const float* y, const void* gate, int64_t gate_stride, const void* weight, void* out, int tokens,
                            int dim, int parts, float eps, int dtype, void* stream);
+
+// -- gated linear attention (linear_attention.hip) -----------------------------------------------------------------------
+// y [T, C] = sigmoid(a w2 + bias)^inv_tau, float32: a [T, rank] columns of rows a_stride apart, w2t [rank, C].
+int holon_gla_decay(const void* a, int64_t a_stride, const void* w2t, const float* bias, float inv_tau, float* y, int tokens,
+                    int channels, int rank, int dtype, void* stream);
+// Per row and head along its tokens: S <- diag(alpha) S + k v^T, out = S^T (q_scale q); q, k [T, H D] and v [T, H V]
+// columns of rows `stride` apart, alpha [T, H D], state [slots, H, D, V] and out [T, H V] float32. piece_tokens > 0 (a
+// multiple of 16): rows are cut into pieces that run side by side (at most max_pieces a row; piece_base [rows]: the number
+// of each row's first piece among all; workspaces sloc [pieces, H, D, V], pw [pieces, H, D]).
+int holon_gla_scan(const void* q, const void* k, const void* v, int64_t stride, float q_scale, const float* alpha,
+                   float* state, float* out, const int32_t* slots, const int32_t* starts, const int32_t* query_start,
+                   int rows, int heads, int dim, int vdim, int state_slots, int dtype, int piece_tokens, int max_pieces,
+                   const int32_t* piece_base, float* sloc, float* pw, void* stream);
+// A step of single tokens (row b is token b) in one kernel: decays, recurrence and read-out as above, then per head
+// y = o / sqrt(mean(o^2) + eps) weight silu(gate); all inputs columns of rows `stride` apart, y [rows, H V].
+int holon_gla_step_supported(int dim, int vdim);
+int holon_gla_step(const void* q, const void* k, const void* v, const void* gate, const void* a, int64_t stride,
+                   float q_scale, const void* w2t, const float* bias, float inv_tau, int rank, const void* weight,
+                   float eps, float* state, void* y, const int32_t* slots, const int32_t* starts, int rows, int heads,
+                   int dim, int vdim, int state_slots, int dtype, void* stream);
+
+// -- an embedding with a second table by token pair (bigram_embedding.hip) ------------------------------------------------
+// y [T, width] float32 = table[t] + bigram[(before mul_prev + t mul_cur) mod buckets] (a sequence's first token: row
+// `buckets`); prev [slots]: the token before a row's first, replaced by the row's last.
+int holon_bigram_embedding(const int32_t* ids, const int32_t* take_slot, const int32_t* last_token, const void* table,
+                           const void* bigram, int32_t* prev, const int32_t* slots, const int32_t* starts,
+                           const int32_t* query_start, const int32_t* token_row, float* y, int tokens, int rows, int width,
+                           int vocab, int buckets, int64_t mul_prev, int64_t mul_cur, int state_slots, int dtype,
+                           int rows_in_order, void* stream);
 
 #ifdef __cplusplus
 }

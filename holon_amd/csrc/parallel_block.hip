@@ -242,14 +242,23 @@ __global__ void __launch_bounds__(256) stream_rms_vec_kernel(float* __restrict__
   }
 }
 
+// A sublayer's result that is still the sum of two, s1 term + s2 second + row (`second` and `row` nullable; row [dim]
+// float32): formed in float32 as the row is read.
+struct Mixed {
+  const void* second;
+  const float* row;
+  float s1, s2;
+};
+
 // A sublayer's result on its way into the stream: x += gain * term / sqrt(mean(term^2) + term_eps), then the row normed for
-// the next sublayer, y = x / sqrt(mean(x^2) + eps) * w. One block a row; a thread holds REGS groups of N neighbouring
-// values of both rows in registers (0: it reads back what it wrote). T: the term's and the result's type, W: the weight's.
-template <typename T, typename W, int N, int REGS>
+// the next sublayer, y = x / sqrt(mean(x^2) + eps) * w (no weight: the next sublayer reads the stream itself, y = x). One
+// block a row; a thread holds REGS groups of N neighbouring values of both rows in registers (0: it reads back what it
+// wrote). T: the term's and the result's type, W: the weight's. MIX: the term is a sum (see Mixed).
+template <typename T, typename W, int N, int REGS, bool MIX, bool NORM>
 __global__ void __launch_bounds__(256) stream_rms_post_kernel(float* __restrict__ x32, const T* __restrict__ term,
                                                               const float* __restrict__ gain, float term_eps,
                                                               const W* __restrict__ w, T* __restrict__ y, int dim,
-                                                              float eps) {
+                                                              float eps, Mixed mix) {
   __shared__ float part[4];
   const int64_t base = (int64_t)blockIdx.x * dim;
   float* x = x32 + base;
@@ -262,6 +271,21 @@ __global__ void __launch_bounds__(256) stream_rms_post_kernel(float* __restrict_
   using TermT = std::integral_constant<int, DT>;
   using WeightT = std::integral_constant<int, DW>;
   using F32T = std::integral_constant<int, HOLON_F32>;
+  const T* sp = MIX ? (const T*)mix.second + base : nullptr;
+  auto take_term = [&](int i, float (&v)[N]) {
+    take(tp, i, v, TermT{});
+    if constexpr (MIX) {
+      float other[N];
+      take(sp, i, other, TermT{});
+#pragma unroll
+      for (int u = 0; u < N; ++u) v[u] = mix.s1 * v[u] + mix.s2 * other[u];
+      if (mix.row) {
+        take(mix.row, i, other, F32T{});
+#pragma unroll
+        for (int u = 0; u < N; ++u) v[u] += other[u];
+      }
+    }
+  };
   constexpr int R = REGS > 0 ? REGS : 1;
   float tv[R][N], xv[R][N];
   float sq = 0.f;
@@ -271,7 +295,7 @@ __global__ void __launch_bounds__(256) stream_rms_post_kernel(float* __restrict_
       const int i = (threadIdx.x + e * 256) * N;
 #pragma unroll
       for (int u = 0; u < N; ++u) tv[e][u] = xv[e][u] = 0.f;
-      if (i < dim) { take(tp, i, tv[e], TermT{}); take(x, i, xv[e], F32T{}); }
+      if (i < dim) { take_term(i, tv[e]); take(x, i, xv[e], F32T{}); }
     }
 #pragma unroll
     for (int e = 0; e < REGS; ++e)
@@ -279,7 +303,7 @@ __global__ void __launch_bounds__(256) stream_rms_post_kernel(float* __restrict_
       for (int u = 0; u < N; ++u) sq += tv[e][u] * tv[e][u];
   } else {
     for (int i = threadIdx.x * N; i < dim; i += 256 * N) {
-      take(tp, i, tv[0], TermT{});
+      take_term(i, tv[0]);
 #pragma unroll
       for (int u = 0; u < N; ++u) sq += tv[0][u] * tv[0][u];
     }
@@ -297,9 +321,9 @@ __global__ void __launch_bounds__(256) stream_rms_post_kernel(float* __restrict_
   };
   auto emit = [&](int i, const float (&v)[N], float r) {
     float g[N], o[N];
-    take(w, i, g, WeightT{});
+    if constexpr (NORM) take(w, i, g, WeightT{});
 #pragma unroll
-    for (int u = 0; u < N; ++u) o[u] = v[u] * r * g[u];
+    for (int u = 0; u < N; ++u) o[u] = NORM ? v[u] * r * g[u] : v[u];
     if constexpr (N == 4) store4t<DT>(y + base, i, o);
     else store_as(y + base, i, DT, o[0]);
   };
@@ -311,13 +335,16 @@ __global__ void __launch_bounds__(256) stream_rms_post_kernel(float* __restrict_
     }
   } else {
     for (int i = threadIdx.x * N; i < dim; i += 256 * N) {
-      take(tp, i, tv[0], TermT{});
+      take_term(i, tv[0]);
       take(x, i, xv[0], F32T{});
       join(i, tv[0], xv[0]);
     }
   }
-  sx = block_sum_256(sx, part);
-  const float r = 1.0f / sqrtf(sx / (float)dim + eps);
+  float r = 1.f;
+  if constexpr (NORM) {
+    sx = block_sum_256(sx, part);
+    r = 1.0f / sqrtf(sx / (float)dim + eps);
+  }
   if constexpr (REGS > 0) {
 #pragma unroll
     for (int e = 0; e < REGS; ++e) {
@@ -412,15 +439,24 @@ extern "C" int holon_stream_rms_filter(float* x32, const void* d1, int dt1, cons
 
 extern "C" int holon_stream_rms_post(float* x32, const void* term, int dtt, const float* gain, float term_eps,
                                      const void* w, int dtw, void* y, int64_t rows, int dim, float eps, int dt_out,
-                                     void* stream) {
+                                     const void* second, float s1, float s2, const float* mix_row, void* stream) {
   HOLON_CHECK(rows >= 0 && dim > 0 && rows <= 0x7fffffffLL, "stream_rms_post: rows=%lld dim=%d", (long long)rows, dim);
   HOLON_CHECK(dtt == dt_out && (dtw == dtt || dtw == HOLON_F32),
               "stream_rms_post: a term of the result's type, a weight of that type or float32");
+  HOLON_CHECK(second != nullptr || mix_row == nullptr, "stream_rms_post: a vector without the second term");
   if (rows == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
-#define SRP(T, W, N, R)                                                                                             \
-  stream_rms_post_kernel<T, W, N, R><<<(unsigned)rows, 256, 0, s>>>(x32, (const T*)term, gain, term_eps, (const W*)w, \
-                                                                    (T*)y, dim, eps)
+  const Mixed mix{second, mix_row, s1, s2};
+#define SRP_AS(T, W, N, R, M, NORM)                                                                              \
+  stream_rms_post_kernel<T, W, N, R, M, NORM><<<(unsigned)rows, 256, 0, s>>>(x32, (const T*)term, gain, term_eps, \
+                                                                             (const W*)w, (T*)y, dim, eps, mix)
+#define SRP(T, W, N, R)                                       \
+  do {                                                        \
+    if (second && w) SRP_AS(T, W, N, R, true, true);          \
+    else if (second) SRP_AS(T, W, N, R, true, false);         \
+    else if (w) SRP_AS(T, W, N, R, false, true);              \
+    else SRP_AS(T, W, N, R, false, false);                    \
+  } while (0)
 #define SRP_BY_SIZE(T, W)                                                     \
   do {                                                                        \
     if (dim % 4 == 0 && dim <= 1024) SRP(T, W, 4, 1);                         \
@@ -434,6 +470,7 @@ extern "C" int holon_stream_rms_post(float* x32, const void* term, int dtt, cons
   else SRP_BY_SIZE(bf16_t, bf16_t);
 #undef SRP_BY_SIZE
 #undef SRP
+#undef SRP_AS
   HOLON_LAUNCH_OK();
   return 0;
 }

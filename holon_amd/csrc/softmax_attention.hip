@@ -2,7 +2,8 @@
 // optional sink (one scalar per head whose exponential joins the normaliser; nothing is read from the cache for it). The general kernel: any
 // element type, any sizes. Options on the scores: a tanh cap (s <- cap tanh(s / cap)), a distance bias per head
 // (s <- s - r1 ln(1 + r2 (i - j)) for query i and key j), and under a window the first tokens of the sequence kept
-// visible (key j is seen if j <= i and (i - j < window or j < keep_first)).
+// visible (key j is seen if j <= i and (i - j < window or j < keep_first)). A negative window is a chunk: query i sees the
+// keys of its own chunk of -window positions, counted from position 0.
 //
 // A page of one site holds P tokens: keys [Hkv, P, D] (a token's key is a row), then values [Hkv, V, P] (transposed
 // inside the page); with `v_share` s > 1 only Hkv / s value heads, key head h reading value head h / s. One block of four waves per (token, head). Keys are walked in tiles of 64 that start at multiples
@@ -43,7 +44,7 @@ __global__ void __launch_bounds__(256) softmax_attention_kernel(
   const T* qp = q + ((int64_t)t * heads + h) * dim;
   for (int d = threadIdx.x; d < dim; d += 256) q_s[d] = Elem<T>::load(qp[d]);
   __syncthreads();
-  const int first = window > 0 ? max(0, pos - window + 1) : 0;
+  const int first = max(0, first_seen(pos, window));
   const int kept = window > 0 && keep_first > 0 ? min(keep_first, first) : 0;      // keys 0 .. kept - 1 are seen too
   const int tile_first = first / WAVE;
   const int extra = min((kept + WAVE - 1) / WAVE, tile_first);     // tiles of kept keys wholly before the window's first
@@ -171,7 +172,7 @@ extern "C" int holon_softmax_attention(const void* q, void* out, const void* pag
               kv_heads, v_share);
   HOLON_CHECK(dim > 0 && dim <= SMX_MAX_D && vdim > 0 && vdim <= SMX_MAX_D,
               "softmax_attention: head sizes %d/%d (at most %d)", dim, vdim, SMX_MAX_D);
-  HOLON_CHECK(page_size > 0 && num_pages > 0 && window >= 0 && table_stride > 0 && table_rows > 0,
+  HOLON_CHECK(page_size > 0 && num_pages > 0 && window > -0x7fffffff && table_stride > 0 && table_rows > 0,
               "softmax_attention: bad page geometry");
   HOLON_CHECK(softcap >= 0.f && keep_first >= 0 && (r1 == nullptr) == (r2 == nullptr),
               "softmax_attention: a cap of %g, %d kept tokens, a distance bias of two numbers a head", softcap, keep_first);

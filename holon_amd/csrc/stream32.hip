@@ -28,6 +28,11 @@ __global__ void widen_kernel(const void* __restrict__ x, float* __restrict__ y, 
     y[i] = load_as(x, i, dt);
 }
 
+__global__ void narrow_kernel(const float* __restrict__ x, void* __restrict__ y, int64_t n, int dt) {
+  for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x)
+    store_as(y, i, dt, x[i]);
+}
+
 // One block a row: x += s1 d1 + s2 d2 (either may be absent); then, with a weight, y = (x - mean) / sqrt(var + eps) * w
 // with the variance taken about the mean in a second pass over the row. REGS: the row (up to 256 * REGS values) stays in
 // registers between the passes; 0: it is read back from memory (a thread reads what it wrote itself).
@@ -109,6 +114,14 @@ extern "C" int holon_widen_rows(const void* x, float* y, int64_t n, int dtype, v
   HOLON_CHECK(n >= 0 && (dtype == HOLON_F32 || dtype == HOLON_BF16), "widen_rows: n=%lld dtype=%d", (long long)n, dtype);
   if (n == 0) return 0;
   widen_kernel<<<blocks_for(n), 256, 0, (hipStream_t)stream>>>(x, y, n, dtype);
+  HOLON_LAUNCH_OK();
+  return 0;
+}
+
+extern "C" int holon_narrow_rows(const float* x, void* y, int64_t n, int dtype, void* stream) {
+  HOLON_CHECK(n >= 0 && (dtype == HOLON_F32 || dtype == HOLON_BF16), "narrow_rows: n=%lld dtype=%d", (long long)n, dtype);
+  if (n == 0) return 0;
+  narrow_kernel<<<blocks_for(n), 256, 0, (hipStream_t)stream>>>(x, y, n, dtype);
   HOLON_LAUNCH_OK();
   return 0;
 }

@@ -148,7 +148,7 @@ class Engine:
         torch.cuda.synchronize(device)
         peak = torch.cuda.max_memory_allocated(device) - base
         del logits, drawn, runner, cache, sampler
-        for site in self.model.sites:
+        for site in self.model.all_sites:
             site.detach()
         torch.cuda.empty_cache()
         return int(peak * 1.1) + (64 << 20)           # the allocator's rounding and fragmentation

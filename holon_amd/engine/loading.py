@@ -63,7 +63,7 @@ def build_from_spec(spec: ModelSpec, *, device: torch.device, dtype: torch.dtype
 def attach_cache(model: Model, *, device: torch.device, dtype: torch.dtype, kernels, page_size: int, max_seqs: int,
                  max_model_len: int, max_step_tokens: int, cache_tokens: int, graphs: bool = False
                  ) -> tuple[CacheManager, StepRunner]:
-    cache = CacheManager(model.sites, model.state_decls(), page_size=page_size, max_seqs=max_seqs,
+    cache = CacheManager(model.all_sites, model.state_decls(), page_size=page_size, max_seqs=max_seqs,
                          max_model_len=max_model_len, tokens=cache_tokens, device=device, dtype=dtype)
     runner = StepRunner(model, cache, kernels, device, max_step_tokens=max_step_tokens, max_seqs=max_seqs,
                         graphs=graphs)
@@ -145,7 +145,7 @@ def time_products(a: Assembled, cfg: EngineConfig) -> None:
             del cache, runner
     finally:
         plan.resolving = False
-        for site in a.model.sites:
+        for site in a.model.all_sites:
             site.detach()
         torch.cuda.empty_cache()
     print(f"holon_amd: product choices timed in {time.perf_counter() - t0:.1f} s: "

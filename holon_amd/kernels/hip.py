@@ -700,7 +700,7 @@ class HipKernels:
                            rows.max_chunk_query, rows.max_chunk_len, hq, hkv, d, page_size, float(scale), int(window),
                            _ptr(sink), *mod, self._stream())
             if rows.n_decode:
-                span = rows.max_decode_len if not window else min(rows.max_decode_len, window + 31)
+                span = rows.max_decode_len if not window else min(rows.max_decode_len, abs(window) + 31)
                 splits, per, waves = self.decode_splits(rows.n_decode * hkv * ((hq // hkv + 15) // 16), span, d)
                 part_o, part_ml = self._decode_parts(rows.n_decode * hq * (splits // waves), d, q.device)
                 self._call(self.lib.holon_attention_decode_mod_bf16, *common, rows.decode_rows.data_ptr(),
@@ -716,7 +716,7 @@ class HipKernels:
                            rows.max_chunk_query, rows.max_chunk_len, hq, hkv, d, page_size, float(scale), int(window),
                            _ptr(sink), self._stream())
             if rows.n_decode:
-                span = rows.max_decode_len if not window else min(rows.max_decode_len, window + 31)
+                span = rows.max_decode_len if not window else min(rows.max_decode_len, abs(window) + 31)
                 splits, per, waves = self.decode_splits(rows.n_decode * hkv * ((hq // hkv + 15) // 16), span, d)
                 part_o, part_ml = self._decode_parts(rows.n_decode * hq * (splits // waves), d, q.device)
                 self._call(self.lib.holon_attention_decode_sink_bf16, *common, rows.decode_rows.data_ptr(),
@@ -767,7 +767,7 @@ class HipKernels:
                        rows.max_chunk_query, rows.max_chunk_len, hq, hkv, d, page_size, float(scale), int(window),
                        _ptr(sink), *mod, self._stream())
         if rows.n_decode:
-            span = rows.max_decode_len if not window else min(rows.max_decode_len, window + 31)
+            span = rows.max_decode_len if not window else min(rows.max_decode_len, abs(window) + 31)
             splits, per, waves = self.decode_splits(rows.n_decode * hkv * ((hq // hkv + 15) // 16), span, d)
             part_o, part_ml = self._decode_parts(rows.n_decode * hq * (splits // waves), d, q.device)
             self._call(self.lib.holon_attention_decode_shared_bf16, *common, rows.decode_rows.data_ptr(),
@@ -809,7 +809,7 @@ class HipKernels:
             if ix.shape[0] < t:
                 raise KernelError(f"{what}: {ix.shape[0]} entries for {t} tokens")
         out = torch.empty((t, heads, head_dim), dtype=qkv.dtype, device=qkv.device)
-        span = rows.max_decode_len if not window else min(rows.max_decode_len, window + 31)
+        span = rows.max_decode_len if not window else min(rows.max_decode_len, abs(window) + 31)
         splits, per, waves = self.decode_splits(rows.n_decode * kv_heads * ((heads // kv_heads + 15) // 16), span,
                                                 head_dim)
         part_o, part_ml = self._decode_parts(rows.n_decode * heads * (splits // waves), head_dim, qkv.device)

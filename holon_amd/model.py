@@ -58,15 +58,25 @@ class Model(Part):
         self.sites = [Site(run=at, layer=r.layer, writes=r.reads is None, owner=r.reads,
                            turn=sum(1 for before in spec.order[:at] if before.layer == r.layer))
                       for at, r in enumerate(spec.order)]
+        # an embedding that keeps state has a site of its own, behind the runs'
+        self.embed_site = Site(run=len(self.sites), layer=-1) if self.embed.state() else None
+
+    @property
+    def all_sites(self) -> list[Site]:
+        """Every place that may keep state: the runs in order, then the embedding if it keeps any."""
+        return self.sites + ([self.embed_site] if self.embed_site is not None else [])
 
     def state_decls(self) -> list[list[PagedState | SlotState]]:
-        """Per run, what its layer keeps between steps (empty for a run that reads another's cache): what the block
-        declares itself (a block with state beside its mixer's), else what its mixer declares."""
+        """Per place of `all_sites`, what it keeps between steps. A run (empty for one that reads another's cache): what
+        the block declares itself (a block with state beside its mixer's), else what its mixer declares; the embedding:
+        what it declares."""
         out = []
         for site in self.sites:
             block = self.blocks[site.layer]
             keeper = block if block.state() else getattr(block, "mixer", None)
             out.append(list(keeper.state()) if keeper is not None and site.writes else [])
+        if self.embed_site is not None:
+            out.append(list(self.embed.state()))
         return out
 
     def cut(self, start: int, count: int) -> int:
@@ -78,7 +88,8 @@ class Model(Part):
 
     def trunk(self, step) -> tuple[torch.Tensor, torch.Tensor | None]:
         """The residual stream after every run, as (h, delta) with h + delta the stream [T, hidden]."""
-        h, stats = self.embed(step.token_ids, step.token_take, want_stats=True)
+        kept = {} if self.embed_site is None else {"step": step, "site": self.embed_site}
+        h, stats = self.embed(step.token_ids, step.token_take, want_stats=True, **kept)
         stream = Stream(h, stats=stats, origin=h if self._keeps_origin else None)
         for site in self.sites:
             stream = self.blocks[site.layer](stream, step, site)

@@ -1,4 +1,4 @@
 """Architectures. Importing this package registers them by their config.json name."""
-from . import dopirax, falisun, nevodra, qwen3, relanex, tolurax
+from . import dopirax, falisun, nevodra, qwen3, relanex, sopepel, tolurax
 
-__all__ = ["dopirax", "falisun", "nevodra", "qwen3", "relanex", "tolurax"]
+__all__ = ["dopirax", "falisun", "nevodra", "qwen3", "relanex", "sopepel", "tolurax"]

@@ -33,13 +33,15 @@ class ParamDecl:
 class PagedState:
     """State that grows by `elems` values per token. Sites whose declarations are equal share a page pool and a block
     table; a window W > 0 says that tokens more than W-1 behind the newest are never read again, except the first
-    `keep_first` tokens of the sequence, which are read for as long as it lives."""
+    `keep_first` tokens of the sequence, which are read for as long as it lives. A chunk C > 0 says that a token is read
+    by tokens of its own chunk of C positions alone (chunks counted from position 0); a state has a window or chunks."""
 
     name: str
     elems: int
     window: int = 0
     dtype: torch.dtype | None = None              # None: the engine's dtype
     keep_first: int = 0
+    chunk: int = 0
 
 
 @dataclasses.dataclass(frozen=True)
@@ -206,7 +208,8 @@ class NormPart(Part):
 
 class EmbedPart(Part):
     """What the model asks of the part that turns token ids into rows of the residual stream. A part implements
-    `rows(ids)`; `forward` adds what the step function may ask for beside it."""
+    `rows(ids)`; `forward` adds what the step function may ask for beside it. An embedding that keeps state between steps
+    declares it (`state`) and is then called with `step` and `site` as well, its state in `site.slot_state`."""
 
     def rows(self, ids: torch.Tensor) -> torch.Tensor:
         raise NotImplementedError

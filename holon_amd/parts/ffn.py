@@ -16,13 +16,17 @@ from .norms import Normed
 
 @register_part("ffn", "swiglu")
 class SwiGLU(Part):
-    """down(silu(gate(x)) * up(x)); gate and up are merged into one product after loading (gate rows first)."""
+    """down(act(gate(x)) * up(x)) with act silu, or gelu in its tanh form (`act` "gelu_tanh"); gate and up are merged into
+    one product after loading (gate rows first)."""
 
     graph_safe = True
+    ACTS = ("silu", "gelu_tanh")
 
-    def __init__(self, build: Build, *, inter: int, hidden: int, layer: int) -> None:
+    def __init__(self, build: Build, *, inter: int, hidden: int, layer: int, act: str = "silu") -> None:
         super().__init__(build)
-        self.inter, self.hidden = inter, hidden
+        if act not in self.ACTS:
+            raise ValueError(f"ffn swiglu: no activation {act!r} ({', '.join(self.ACTS)})")
+        self.inter, self.hidden, self.act = inter, hidden, act
         self.attach("gate_proj", Linear(build, inp=hidden, out=inter))
         self.attach("up_proj", Linear(build, inp=hidden, out=inter))
         self.attach("down_proj", Linear(build, inp=inter, out=hidden))
@@ -37,11 +41,16 @@ class SwiGLU(Part):
     adds_residual = True
 
     def absorb_norm(self, norm: Part) -> bool:
-        """Fold the norm in front of this part into its first product; it then takes `Normed` input."""
-        return self.gate_up.absorb(norm)
+        """Fold the norm in front of this part into its first product; it then takes `Normed` input (the kernels that do
+        are silu's)."""
+        return self.act == "silu" and self.gate_up.absorb(norm)
 
     def forward(self, x: torch.Tensor | Normed, step=None, residual: Stream | None = None) -> torch.Tensor | None:
         gate_up, y = self.gate_up, None
+        if self.act == "gelu_tanh":
+            x = x.value() if isinstance(x, Normed) else x
+            y = self.kernels.linear_gelu_mul(x, gate_up.weight, gate_up.tiled)
+            return self.down_proj(self.kernels.gelu_mul(gate_up(x)) if y is None else y, residual=residual)
         if gate_up.folds(x):
             y = self.kernels.linear_silu_mul(x.h, gate_up.weight, gate_up.tiled, row_scale=gate_up.row_scale(x))
         elif gate_up.reads_folded(x, gated=True):  # 17 to 64 rows: the folded copy over rows normed without the weight
@@ -64,6 +73,42 @@ _DT = {torch.float32: 0, torch.bfloat16: 1}
 def _need(cond: bool, what: str) -> None:
     if not cond:
         raise ValueError(what)
+
+
+def gelu_mul_plain(gate_up):
+    """gate_up [T, 2 F] (gates, then ups) -> gelu(gate) * up [T, F], gelu in its tanh form; the gelu is rounded to the
+    rows' dtype before the product, as silu_mul rounds."""
+    gate, up = gate_up.chunk(2, dim=-1)
+    wide = gate if gate.dtype == torch.float64 else gate.float()
+    return torch.nn.functional.gelu(wide, approximate="tanh").to(gate.dtype) * up
+
+
+def _gelu_mul_hip(launch, gate_up):
+    _need(gate_up.is_cuda and gate_up.is_contiguous() and gate_up.dim() == 2 and gate_up.dtype in _DT
+          and gate_up.shape[1] % 2 == 0, "gelu_mul: contiguous rows of gates and ups on the GPU")
+    y = torch.empty((gate_up.shape[0], gate_up.shape[1] // 2), dtype=gate_up.dtype, device=gate_up.device)
+    launch(gate_up.data_ptr(), y.data_ptr(), y.shape[0], y.shape[1], _DT[gate_up.dtype])
+    return y
+
+
+def linear_gelu_mul_plain(x, weight, tiled=None):
+    """gelu_mul(x W^T) where one kernel does both, with the roundings of the two one after the other; None where it does
+    not (the caller then composes them). The plain form never does."""
+    return None
+
+
+def _linear_gelu_mul_hip(launch, x, weight, tiled=None):
+    """Steps of up to 16 bfloat16 rows: the few-row product with the activation in its epilogue."""
+    (m, k), n = x.shape, weight.shape[0]
+    if not (x.is_cuda and x.dtype == torch.bfloat16 and weight.dtype == torch.bfloat16 and x.is_contiguous()
+            and weight.is_contiguous() and weight.shape[1] == k and 1 <= m <= 16 and n % 32 == 0 and k % 128 == 0
+            and k >= 256 and (tiled is None or (tiled.shape == weight.shape and tiled.dtype == weight.dtype
+                                                 and tiled.is_contiguous()))):
+        return None
+    y = torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
+    launch(x.data_ptr(), (tiled if tiled is not None else weight).data_ptr(), y.data_ptr(), m, n // 2, k,
+           int(tiled is not None))
+    return y
 
 
 def polynorm_plain(z, coef, eps):
@@ -168,12 +213,16 @@ def _moe_gate_hip(launch, gate_up, weights, ff, shared, shared_weight=False):
     return y
 
 
-def moe_router_top_plain(x, router, bias, experts, top, groups=1, keep=1):
+ROUTER_SCORES = {"softmax": 0, "sigmoid": 1, "sigmoid_squared": 2}
+
+
+def moe_router_top_plain(x, router, bias, experts, top, groups=1, keep=1, score="softmax"):
     """x [T, W] (any dtype), router [R, W] float32 with R = experts or experts + 1, bias [experts] float32 or None:
     the float32 logits z = x . router[e] + bias[e]; the `top` largest are chosen (equal ones: the lower index first)
     and weighted by the softmax over the chosen logits alone, every other expert 0. `groups` > 1: only experts of the
     `keep` best of as many equal groups of neighbours can be chosen, a group's score being its largest logit. A last
-    row beyond the experts is a gate: its column holds sigmoid(x . router[experts]). -> [T, R] float32."""
+    row beyond the experts is a gate: its column holds sigmoid(x . router[experts]). `score` "sigmoid": a chosen expert's
+    weight is sigmoid(z_e) alone, "sigmoid_squared": that squared. -> [T, R] float32."""
     z = x.float() @ router.float().T
     logits = z[:, :experts] + (bias.float() if bias is not None else 0.0)
     choice = logits
@@ -184,11 +233,13 @@ def moe_router_top_plain(x, router, bias, experts, top, groups=1, keep=1):
         choice = logits.masked_fill(~open_.repeat_interleave(experts // groups, dim=1), float("-inf"))
     order = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
     chosen = logits.gather(1, order)
-    w = torch.zeros_like(logits).scatter_(1, order, torch.softmax(chosen, dim=-1))
+    weigh = {"softmax": lambda z: torch.softmax(z, dim=-1), "sigmoid": torch.sigmoid,
+             "sigmoid_squared": lambda z: torch.sigmoid(z).square()}[score]
+    w = torch.zeros_like(logits).scatter_(1, order, weigh(chosen))
     return torch.cat((w, torch.sigmoid(z[:, experts:])), dim=1).contiguous()
 
 
-def _moe_router_top_hip(launch, x, router, bias, experts, top, groups=1, keep=1):
+def _moe_router_top_hip(launch, x, router, bias, experts, top, groups=1, keep=1, score="softmax"):
     (t, w), r = x.shape, router.shape[0]
     _need(x.is_cuda and x.is_contiguous() and x.dtype in _DT and router.is_contiguous() and router.dtype == torch.float32
           and router.shape == (r, w) and r in (experts, experts + 1) and 1 <= top <= experts <= 1024 and w <= 12288
@@ -199,8 +250,32 @@ def _moe_router_top_hip(launch, x, router, bias, experts, top, groups=1, keep=1)
     weights = torch.empty((t, r), dtype=torch.float32, device=x.device)
     if t:
         launch(x.data_ptr(), router.data_ptr(), None if bias is None else bias.data_ptr(), weights.data_ptr(), t, w,
-               experts, r, int(top), _DT[x.dtype], int(groups), int(keep))
+               experts, r, int(top), _DT[x.dtype], int(groups), int(keep), ROUTER_SCORES[score])
     return weights
+
+
+def moe_relu2_plain(up, weights, ff, shared, shared_weight=False):
+    """up [T, C] with C = E ff + shared columns -> max(up, 0)^2 times the weight of the column's expert, float32 inside and
+    one rounding, exactly 0 where the weight is 0; columns and weights as for `moe_gate`."""
+    t, e = weights.shape[0], weights.shape[1] - int(bool(shared_weight))
+    w = weights[:, :e].repeat_interleave(ff, dim=1)
+    if shared:
+        last = weights[:, e:].expand(t, shared) if shared_weight else torch.ones((t, shared), dtype=w.dtype, device=w.device)
+        w = torch.cat((w, last), dim=1)
+    return torch.where(w == 0, torch.zeros_like(w), torch.relu(up.float()).square() * w).to(up.dtype)
+
+
+def _moe_relu2_hip(launch, up, weights, ff, shared, shared_weight=False):
+    t, e = weights.shape[0], weights.shape[1] - int(bool(shared_weight))
+    c = e * ff + shared
+    _need(up.is_cuda and up.is_contiguous() and up.dtype in _DT and up.shape == (t, c) and weights.is_contiguous()
+          and weights.dtype == torch.float32 and e >= 1, f"moe_relu2: rows {tuple(up.shape)} for {e} experts of {ff} and "
+          f"{shared} shared columns")
+    y = torch.empty_like(up)
+    if t:
+        launch(up.data_ptr(), weights.data_ptr(), y.data_ptr(), t, e, ff, shared, _DT[up.dtype], weights.shape[1],
+               e if shared_weight else -1)
+    return y
 
 
 def relu2_plain(z):
@@ -224,7 +299,12 @@ register_kernel(KernelOp("moe_router", moe_router_plain, "holon_moe_router",
 register_kernel(KernelOp("moe_gate", moe_gate_plain, "holon_moe_gate", [_P, _P, _P, _L, _I, _I, _I, _I, _I, _I],
                          _moe_gate_hip))
 register_kernel(KernelOp("moe_router_top", moe_router_top_plain, "holon_moe_router_top",
-                         [_P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _I], _moe_router_top_hip))
+                         [_P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _I, _I], _moe_router_top_hip))
+register_kernel(KernelOp("moe_relu2", moe_relu2_plain, "holon_moe_relu2", [_P, _P, _P, _L, _I, _I, _I, _I, _I, _I],
+                         _moe_relu2_hip))
+register_kernel(KernelOp("gelu_mul", gelu_mul_plain, "holon_gelu_mul", [_P, _P, _L, _I, _I], _gelu_mul_hip))
+register_kernel(KernelOp("linear_gelu_mul", linear_gelu_mul_plain, "holon_gemm_skinny_geglu_bf16",
+                         [_P, _P, _P, _I, _I, _I, _I], _linear_gelu_mul_hip))
 register_kernel(KernelOp("relu2", relu2_plain, "holon_relu2", [_P, _P, _L, _I], _relu2_hip))
 
 
@@ -299,14 +379,18 @@ class DenseFFN(Part):
 
 @register_part("ffn", "moe")
 class MoE(Part):
-    """A mixture of SiLU-gated experts with a router, and an optional shared expert that every token uses.
+    """A mixture of experts with a router, and an optional shared expert that every token uses. The experts are SiLU-gated,
+    or (`act` "relu2") W_down max(W_up x, 0)^2.
 
     `score` "softmax_top" is the other router: float32 logits z = W_r x + b (`router_bias`), the `top` largest z are
     chosen and weighted by the softmax over the chosen z alone (no scale); with `groups` only among the `keep` groups
     whose largest z are best. (A softmax over all experts whose chosen scores are then divided by their sum gives the
     same weights: the largest score is always among the chosen, so their sum is never near zero.) `shared_gated`: the shared
     expert's output is multiplied by sigmoid(w_sg . x), one number a token; w_sg rides as one more row of the router's
-    weights, so the router's kernel leaves that weight too. What follows describes `score` "sigmoid".
+    weights, so the router's kernel leaves that weight too. `score` "sigmoid_top" is the same choice with each chosen
+    expert's own sigmoid(z) as its weight. `weigh_input`: the weight multiplies an expert's input, not its output; for the
+    squared ReLU that is its square on the output, W_down max(W_up w x, 0)^2 = w^2 W_down max(W_up x, 0)^2 for w > 0, and
+    the router's kernel squares it. What follows describes `score` "sigmoid".
 
     Router: float32 logits (products of the input as it is with float32 weights, summed in float32), scores s =
     sigmoid(logits); experts are chosen by s + `correction` (`bias`), optionally
@@ -320,16 +404,21 @@ class MoE(Part):
 
     def __init__(self, build: Build, *, experts: int, top: int, inter: int, hidden: int, layer: int,
                  scale: float = 1.0, groups: int = 1, keep: int = 1, bias: bool = True, shared: int = 0,
-                 score: str = "sigmoid", shared_gated: bool = False) -> None:
+                 score: str = "sigmoid", shared_gated: bool = False, act: str = "silu", weigh_input: bool = False) -> None:
         super().__init__(build)
         if not 1 <= top <= experts:
             raise ValueError(f"moe: top {top} of {experts} experts")
-        if score not in ("sigmoid", "softmax_top"):
-            raise ValueError(f"moe: no router score {score!r} (sigmoid, softmax_top)")
-        if score == "softmax_top" and float(scale) != 1.0:
-            raise ValueError("moe: the softmax over the chosen logits comes without a scale")
-        if shared_gated and (not shared or score != "softmax_top"):
-            raise ValueError("moe: a gate on the shared expert needs a shared expert and the softmax_top router")
+        if score not in ("sigmoid", "softmax_top", "sigmoid_top"):
+            raise ValueError(f"moe: no router score {score!r} (sigmoid, softmax_top, sigmoid_top)")
+        if score != "sigmoid" and float(scale) != 1.0:
+            raise ValueError("moe: the router that chooses by its logits comes without a scale")
+        if shared_gated and (not shared or score == "sigmoid"):
+            raise ValueError("moe: a gate on the shared expert needs a shared expert and a router that chooses by its logits")
+        if act not in ("silu", "relu2"):
+            raise ValueError(f"moe: no expert activation {act!r} (silu, relu2)")
+        if weigh_input and (act != "relu2" or score != "sigmoid_top"):
+            raise ValueError("moe: weights on the experts' inputs come with the squared ReLU and the sigmoid_top router")
+        self.act, self.weigh_input = act, bool(weigh_input)
         self.score, self.shared_gated = score, bool(shared_gated)
         if groups > 1 and (experts % groups or not 1 <= keep <= groups or top > keep * (experts // groups)):
             raise ValueError(f"moe: {experts} experts in {groups} groups, {keep} kept, top {top}")
@@ -342,18 +431,20 @@ class MoE(Part):
             self.declare("correction" if score == "sigmoid" else "router_bias", (experts,), kind=FLOAT32, init="zero")
         if self.shared_gated:
             self.declare("shared_sg", (1, hidden), kind=FLOAT32)
-        self.declare("gate", (experts, inter, hidden))
+        if act == "silu":
+            self.declare("gate", (experts, inter, hidden))
         self.declare("up", (experts, inter, hidden))
         self.declare("down", (experts, hidden, inter))
         if self.shared:
-            self.declare("shared_gate", (self.shared, hidden))
+            if act == "silu":
+                self.declare("shared_gate", (self.shared, hidden))
             self.declare("shared_up", (self.shared, hidden))
             self.declare("shared_down", (hidden, self.shared))
         self.gate_up: Linear | None = None
         self.all_down: Linear | None = None
 
     def finalize(self) -> None:
-        if self.gate is None:
+        if self.up is None:
             return
         if self.shared_gated and self.router.shape[0] == self.experts:
             self.router = torch.cat((self.router, self.shared_sg)).contiguous()
@@ -361,11 +452,13 @@ class MoE(Part):
             self.shared_sg = None
         e, f, w = self.experts, self.inter, self.hidden
         cols = e * f + self.shared
-        gate_up, down = Linear(self.build, inp=w, out=2 * cols), Linear(self.build, inp=cols, out=w)
-        gates, ups = [self.gate.reshape(e * f, w)], [self.up.reshape(e * f, w)]
+        gated = self.act == "silu"
+        gate_up, down = Linear(self.build, inp=w, out=(2 if gated else 1) * cols), Linear(self.build, inp=cols, out=w)
+        gates, ups = [self.gate.reshape(e * f, w)] if gated else [], [self.up.reshape(e * f, w)]
         downs = [self.down.permute(1, 0, 2).reshape(w, e * f)]
         if self.shared:
-            gates.append(self.shared_gate)
+            if gated:
+                gates.append(self.shared_gate)
             ups.append(self.shared_up)
             downs.append(self.shared_down)
         gate_up.weight = torch.cat(gates + ups, dim=0).contiguous()
@@ -381,13 +474,19 @@ class MoE(Part):
 
     def forward(self, x: torch.Tensor, step=None) -> torch.Tensor:
         k = self.kernels
-        if self.score == "softmax_top":
+        if self.score != "sigmoid":
+            how = {} if self.score == "softmax_top" else {"score": "sigmoid_squared" if self.weigh_input else "sigmoid"}
             weights = k.moe_router_top(x, self.router, self.router_bias if self.has_bias else None, self.experts,
-                                       self.top, self.groups, self.keep)
+                                       self.top, self.groups, self.keep, **how)
+            if self.act == "relu2":
+                return self.all_down(k.moe_relu2(self.gate_up(x), weights, self.inter, self.shared,
+                                                 shared_weight=self.shared_gated))
             act = k.moe_gate(self.gate_up(x), weights, self.inter, self.shared, shared_weight=self.shared_gated)
             return self.all_down(act)
         weights = k.moe_router(x, self.router, self.correction if self.has_bias else None, self.top, self.groups,
                                self.keep, self.scale)
+        if self.act == "relu2":
+            return self.all_down(k.moe_relu2(self.gate_up(x), weights, self.inter, self.shared))
         act = k.moe_gate(self.gate_up(x), weights, self.inter, self.shared)
         return self.all_down(act)
 

@@ -101,7 +101,11 @@ class GQA(Part):
 class ParallelMixers(Part):
     """Two mixers side by side that read the same input; the result is left_scale * left + right_scale * right. The
     two results are handed on as terms with their scales (`Pending`) to a block whose residual add takes them in one
-    kernel; `left` and `right` are any registered mixers, each keeping its state under its own name."""
+    kernel; `left` and `right` are any registered mixers, each keeping its state under its own name.
+
+    Where both mixers say that one product reads their input (`give_projection`) and take its rows (`forward(rows=, at=)`),
+    the two products become one. A left mixer that names a bias on its last projection (`out_row`) is asked to leave it
+    out (`add_row=False`): times left_scale it joins the terms as a float32 vector."""
 
     graph_safe = True
 
@@ -111,12 +115,41 @@ class ParallelMixers(Part):
         self.left_scale, self.right_scale = float(left_scale), float(right_scale)
         self.attach("left", build.make(left, hidden=hidden, layer=layer, name="left"))
         self.attach("right", build.make(right, hidden=hidden, layer=layer, name="right"))
+        self.hidden = hidden
+        self.inp: Linear | None = None            # the product over both mixers' input, where they share one
+        self.right_at = 0
+        self.row: torch.Tensor | None = None      # left_scale times the left mixer's output bias
 
     def state(self):
         return list(self.left.state()) + list(self.right.state())
 
+    def finalize(self) -> None:
+        bias = getattr(self.left, "out_row", None)
+        if bias is not None:
+            self.row = (bias.float() * self.left_scale).contiguous()
+        if not all(hasattr(m, "give_projection") for m in (self.left, self.right)):
+            return
+        left, right = self.left.give_projection(), self.right.give_projection()
+        if left is None or right is None:
+            return
+        self.right_at = left.out
+        pad = -(left.out + right.out) % 16        # (every product of the framework serves a multiple of 16)
+        if pad:
+            right.weight = torch.cat((right.weight, right.weight.new_zeros((pad, self.hidden)))).contiguous()
+            right.out += pad
+        self.inp = self.attach("inp", Linear.merge(self.build, left, right))
+
+    def extra_tensors(self):
+        return [self.row] if self.row is not None else []
+
     def forward(self, x, step, site):
         from .stream32 import Pending
-        return Pending([(self.left(x, step, site), self.left_scale), (self.right(x, step, site), self.right_scale)])
+        left, right = {} if self.row is None else {"add_row": False}, {}
+        if self.inp is not None:
+            rows = self.inp(x)
+            left.update(rows=rows)
+            right.update(rows=rows, at=self.right_at)
+        return Pending([(self.left(x, step, site, **left), self.left_scale),
+                        (self.right(x, step, site, **right), self.right_scale)], self.row)
 
     __call__ = forward

@@ -138,27 +138,56 @@ def _stream_rms_filter_hip(launch, x32, terms, row, w1, w2, eps, out_dtype, taps
     return y1, y2
 
 
-def stream_rms_post_plain(x32, term, gain, term_eps, w, eps, out_dtype):
+def stream_rms_post_plain(x32, term, gain, term_eps, w, eps, out_dtype, mix=None):
     """x32 [T, W] float32, updated in place: x += gain * term / sqrt(mean(term^2) + term_eps) with `term` [T, W] in any
-    dtype and `gain` [W] float32. Then the answer x / sqrt(mean(x^2) + eps) * w in `out_dtype`. float32 arithmetic, one
-    rounding of the answer."""
+    dtype and `gain` [W] float32. Then the answer x / sqrt(mean(x^2) + eps) * w in `out_dtype`, or with `w` None x itself.
+    `mix` = (s1, second, s2, row): the term is s1 term + s2 second + row (`row` [W] float32 or None). float32 arithmetic,
+    one rounding of the answer."""
     t = term.float()
+    if mix is not None:
+        s1, second, s2, row = mix
+        t = s1 * t + s2 * second.float()
+        if row is not None:
+            t = t + row
     x32.add_(t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + term_eps) * gain)
+    if w is None:
+        return x32.to(out_dtype, copy=True)
     return (x32 * torch.rsqrt(x32.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
 
 
-def _stream_rms_post_hip(launch, x32, term, gain, term_eps, w, eps, out_dtype):
+def mixed_terms(term):
+    """(term, mix) for `stream_rms_post` from a sublayer's result: a tensor as it is; `Pending` terms with their scales
+    and vector, one or two."""
+    if not isinstance(term, Pending):
+        return term, None
+    terms = term.terms
+    if len(terms) == 1 and terms[0][1] == 1.0 and term.row is None:
+        return terms[0][0], None
+    if len(terms) > 2:
+        raise ValueError(f"a sublayer's result as {len(terms)} terms (at most two)")
+    second = terms[1] if len(terms) == 2 else (terms[0][0], 0.0)
+    return terms[0][0], (terms[0][1], second[0], second[1], term.row)
+
+
+def _stream_rms_post_hip(launch, x32, term, gain, term_eps, w, eps, out_dtype, mix=None):
     _need(x32.is_cuda and x32.is_contiguous() and x32.dtype == torch.float32 and x32.dim() == 2,
           "stream_rms_post: the stream is contiguous float32 rows on the GPU")
     rows, dim = x32.shape
     _need(term.is_cuda and term.is_contiguous() and term.shape == x32.shape and term.dtype in _DT,
           "stream_rms_post: the term must be contiguous rows of the stream's shape")
-    _need(gain.is_contiguous() and gain.dtype == torch.float32 and gain.shape == (dim,) and w.is_contiguous()
-          and w.shape == (dim,) and w.dtype in _DT and out_dtype in _DT, "stream_rms_post: vectors of the rows' width")
+    _need(gain.is_contiguous() and gain.dtype == torch.float32 and gain.shape == (dim,) and out_dtype in _DT
+          and (w is None or (w.is_contiguous() and w.shape == (dim,) and w.dtype in _DT)),
+          "stream_rms_post: vectors of the rows' width")
+    s1, second, s2, row = mix if mix is not None else (1.0, None, 0.0, None)
+    _need(second is None or (second.is_cuda and second.is_contiguous() and second.shape == term.shape
+                             and second.dtype == term.dtype), "stream_rms_post: two terms of one shape and type")
+    _need(row is None or (row.is_cuda and row.is_contiguous() and row.dtype == torch.float32 and row.shape == (dim,)),
+          "stream_rms_post: the added vector is float32 of the stream's width")
     y = torch.empty((rows, dim), dtype=out_dtype, device=x32.device)
     if rows:
-        launch(x32.data_ptr(), term.data_ptr(), _DT[term.dtype], gain.data_ptr(), float(term_eps), w.data_ptr(),
-               _DT[w.dtype], y.data_ptr(), rows, dim, float(eps), _DT[out_dtype])
+        launch(x32.data_ptr(), term.data_ptr(), _DT[term.dtype], gain.data_ptr(), float(term_eps), _ptr(w),
+               _DT[w.dtype if w is not None else out_dtype], y.data_ptr(), rows, dim, float(eps), _DT[out_dtype],
+               _ptr(second), float(s1), float(s2), _ptr(row))
     return y
 
 
@@ -180,7 +209,7 @@ register_kernel(KernelOp("stream_rms_filter", stream_rms_filter_plain, "holon_st
                          [_P, _P, _I, _P, _I, _P, _P, _P, _I, _P, _P, _L, _I, _F, _I, _P, _P, _P, _P, _P, _P, _I],
                          _stream_rms_filter_hip))
 register_kernel(KernelOp("stream_rms_post", stream_rms_post_plain, "holon_stream_rms_post",
-                         [_P, _P, _I, _P, _F, _P, _I, _P, _L, _I, _F, _I], _stream_rms_post_hip))
+                         [_P, _P, _I, _P, _F, _P, _I, _P, _L, _I, _F, _I, _P, _F, _F, _P], _stream_rms_post_hip))
 register_kernel(KernelOp("scale_rows", scale_rows_plain, "holon_scale_rows", [_P, _P, _L, _I, _F], _scale_rows_hip))
 
 
@@ -188,13 +217,15 @@ register_kernel(KernelOp("scale_rows", scale_rows_plain, "holon_scale_rows", [_P
 class RMSNorm32(NormPart):
     """y = x * rsqrt(mean(x^2) + eps) * weight over rows of a float32 stream (rows in the engine's dtype are widened
     first); float32 inside, the result in the engine's dtype. `one_plus`: the stored weight w lies around zero and the
-    norm multiplies by 1 + w (kept in float32: in bfloat16 the sum would lose what w holds)."""
+    norm multiplies by 1 + w (kept in float32: in bfloat16 the sum would lose what w holds). `gain`: a constant that
+    multiplies the result, formed with the weight once after loading and kept in float32 (a last norm's gain is its
+    logits')."""
 
     graph_safe = True
 
-    def __init__(self, build: Build, *, eps: float, dim: int, one_plus: bool = False) -> None:
+    def __init__(self, build: Build, *, eps: float, dim: int, one_plus: bool = False, gain: float = 1.0) -> None:
         super().__init__(build)
-        self.eps, self.dim, self.one_plus = float(eps), dim, bool(one_plus)
+        self.eps, self.dim, self.one_plus, self.gain = float(eps), dim, bool(one_plus), float(gain)
         if self.one_plus:
             self.declare("weight", (dim,), kind=FLOAT32, init="tap")
         else:
@@ -202,8 +233,8 @@ class RMSNorm32(NormPart):
         self._summed = False
 
     def finalize(self) -> None:
-        if self.one_plus and self.weight is not None and not self._summed:
-            self.weight = (self.weight.float() + 1.0).contiguous()
+        if (self.one_plus or self.gain != 1.0) and self.weight is not None and not self._summed:
+            self.weight = ((self.weight.float() + (1.0 if self.one_plus else 0.0)) * self.gain).contiguous()
             self._summed = True
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
@@ -226,8 +257,10 @@ class RMSNorm32(NormPart):
             if extra is not None:
                 residual.add_(extra)
             gain = x.gain if x.gain is not None else x.norm.output_gain(x.scale)
-            return self.kernels.stream_rms_post(residual, x.term, gain, x.norm.eps, self.weight, self.eps,
-                                                self.build.dtype), residual
+            term, mix = mixed_terms(x.term)
+            more = () if mix is None else (mix,)
+            return self.kernels.stream_rms_post(residual, term, gain, x.norm.eps, self.weight, self.eps,
+                                                self.build.dtype, *more), residual
         if extra is not None:
             residual.add_(extra)
         return self.kernels.stream_rms(residual, _terms(x), getattr(x, "row", None), self.weight, None, self.eps,

@@ -1,8 +1,9 @@
 """Softmax attention over the paged cache for heads whose keys and values may differ in width, with the options a
 design may name: biases on the q/k/v projections, rotary positions in either pairing, a scale of its own, a sliding
-window (which may keep the first tokens of the sequence visible), a sink (one trained scalar for each head whose
-exponential is added to the softmax's normaliser; nothing is read from the cache for it), one RMS norm over a token's
-whole query or key projection, a tanh cap on the scores and a logarithmic distance bias per head.
+window (which may keep the first tokens of the sequence visible) or chunks of positions that see nothing of one another, a
+sink (one trained scalar for each head whose exponential is added to the softmax's normaliser; nothing is read from the
+cache for it), an RMS norm of every query and key head or one over a token's whole query or key projection, a tanh cap on
+the scores and a logarithmic distance bias per head.
 Two mixers use it: `attention` (grouped queries) and `latent_attention` (keys and values rebuilt from a cached
 low-rank latent, computed in the latent's space so that nothing but the latent is kept).
 
@@ -33,7 +34,8 @@ def softmax_attention_plain(q, pages, table, rows, token_row, positions, kv_head
                             window, softcap=0.0, dist=None, keep_first=0, value_share=1):
     """q [T, H, D]; `pages` [pages, G P (D + V)] (keys [G, P, D], then values [G, V, P]); `table` [S, max_pages]
     int32; token t belongs to row token_row[t] (slot rows.slots[row]) and stands at positions[t]. Query at position p
-    sees keys max(0, p - window + 1) .. p (window 0: 0 .. p). weights = exp(s_j - top) / (sum_j exp(s_j - top) +
+    sees keys max(0, p - window + 1) .. p (window 0: 0 .. p; window -C: those of its own chunk of C positions, chunks
+    counted from position 0). weights = exp(s_j - top) / (sum_j exp(s_j - top) +
     exp(sink[h] - top)) with s = q . k * scale, `sink` [H] float32 or None (then no such term). With a window and
     `keep_first` > 0 the query also sees keys 0 .. keep_first - 1, at their true positions. `softcap` > 0: s <-
     softcap tanh(s / softcap); `dist` = (r1 [H], r2 [H]) float32: then s <- s - r1 ln(1 + r2 (p - j)) for the key at
@@ -49,7 +51,7 @@ def softmax_attention_plain(q, pages, table, rows, token_row, positions, kv_head
     slot_of, row_of = rows.slots.tolist(), token_row.tolist()
     group = heads // kv_heads
     for i in range(t):
-        first = max(0, pos[i] - window + 1) if window > 0 else 0
+        first = max(0, pos[i] - window + 1) if window > 0 else (pos[i] - pos[i] % -window if window < 0 else 0)
         js = torch.arange(first, pos[i] + 1, device=q.device)
         if keep_first > 0 and first > 0:
             js = torch.cat((torch.arange(0, min(keep_first, first), device=q.device), js))
@@ -461,7 +463,12 @@ class SoftmaxAttention(Part):
     the rotation), so vdim = dim, and the cache holds the turned key and the unturned one side by side. `sink_value`
     (a number): a sink that every head shares and no tensor holds (0: one is added to the softmax's denominator).
     `head_gate`: a projection `g` of one number a head, computed with q and k in the merged product; head h's result
-    is multiplied by sigmoid(g_h) before the output projection. `o_bias`: a bias on the output projection."""
+    is multiplied by sigmoid(g_h) before the output projection. `o_bias`: a bias on the output projection.
+
+    `head_norm` (an eps): every query head and every key head is divided by its root mean square and multiplied by a
+    weight of `dim` values that the heads share (`q_norm`, `k_norm`), after the biases and before the rotation. `chunk`:
+    a query sees the keys of its own chunk of that many positions alone (position i sees j <= i where i div chunk =
+    j div chunk)."""
 
     graph_safe = True
 
@@ -470,8 +477,12 @@ class SoftmaxAttention(Part):
                  position: PartRef | None = None, name: str = "", whole_norm: float | None = None,
                  softcap: float = 0.0, distance_bias: bool = False, keep_first: int = 0,
                  values_from_keys: bool = False, sink_value: float | None = None, head_gate: bool = False,
-                 o_bias: bool = False) -> None:
+                 o_bias: bool = False, head_norm: float | None = None, chunk: int = 0) -> None:
         super().__init__(build)
+        if chunk and window:
+            raise ValueError("attention: either a window or chunks")
+        if head_norm is not None and whole_norm is not None:
+            raise ValueError("attention: either a norm of every head or one over the whole projection")
         if heads % kv_heads:
             raise ValueError(f"attention: {heads} heads are not a multiple of {kv_heads} kv heads")
         self.values_from_keys = bool(values_from_keys)
@@ -484,9 +495,14 @@ class SoftmaxAttention(Part):
         if head_gate and whole_norm is not None:
             raise ValueError("attention: the gate per head comes without the norm over the whole projection")
         self.heads, self.kv_heads, self.dim, self.vdim, self.hidden = heads, kv_heads, dim, vdim, hidden
-        self.window = int(window)
+        self.window, self.chunk = int(window), int(chunk)
+        self.sees = self.window or -self.chunk    # as the operations take it: a window, or chunks as a negative number
         self.keep_first = int(keep_first) if self.window > 0 else 0
         self.softcap = float(softcap or 0.0)
+        self.head_norm = None if head_norm is None else float(head_norm)
+        if self.head_norm is not None:
+            self.declare("q_norm", (dim,), init="norm")
+            self.declare("k_norm", (dim,), init="norm")
         self.whole_norm = None if whole_norm is None else float(whole_norm)
         if self.whole_norm is not None:
             if qkv_bias or position is not None:
@@ -530,7 +546,7 @@ class SoftmaxAttention(Part):
 
     def state(self):
         return [PagedState(self.state_name, elems=self.kv_heads * (self.dim + self.vdim), window=self.window,
-                           keep_first=self.keep_first)]
+                           keep_first=self.keep_first, chunk=self.chunk)]
 
     def finalize(self) -> None:
         if self.q.weight is not None and getattr(self.position, "interleaved", False):
@@ -540,6 +556,9 @@ class SoftmaxAttention(Part):
                 proj.weight = proj.weight.index_select(0, order).contiguous()
                 if self.qkv_bias:
                     setattr(self, bias, getattr(self, bias).index_select(0, order).contiguous())
+            if self.head_norm is not None:
+                order = to_half_split(self.dim, 1, rot).to(self.q_norm.device)
+                self.q_norm, self.k_norm = (w.index_select(0, order).contiguous() for w in (self.q_norm, self.k_norm))
         if self.qkv_bias and self.q_bias is not None:
             self.bias = torch.cat([self.q_bias, self.k_bias] + ([] if self.values_from_keys else [self.v_bias])
                                   ).contiguous()
@@ -565,24 +584,35 @@ class SoftmaxAttention(Part):
         """The output projection's bias, for a caller that adds it to the stream itself (`forward(add_row=False)`)."""
         return self.o_bias if self.has_o_bias else None
 
-    def forward(self, x: torch.Tensor, step, site, add_row: bool = True) -> torch.Tensor:
+    def give_projection(self) -> Linear | None:
+        """The product that reads the input, for an owner that merges it with others behind it; `forward` then takes its
+        rows. (The norm over the whole projection reads rows that hold nothing else.)"""
+        if self.whole_norm is not None or self.qkv is None:
+            return None
+        qkv = self.qkv
+        self.drop("qkv")
+        return qkv
+
+    def forward(self, x: torch.Tensor, step, site, add_row: bool = True, rows: torch.Tensor | None = None) -> torch.Tensor:
+        """`rows`: the input's projections, this mixer's in the first columns (None: made here from `x`)."""
         k = self.kernels
         held = site.paged[self.state_name]
         view = step.paged[held.group]
         table = getattr(self.position, "table", None)
-        qkv = self.qkv(x)
+        qkv = self.qkv(x) if rows is None else rows
         if self.whole_norm is not None:
             q = k.whole_norm_prepare(qkv, self.heads, self.kv_heads, self.dim, self.vdim, self.q_norm,
                                      self.k_norm, self.whole_norm, held.pages, view.write_page, view.write_off,
                                      view.page_size)
         else:
-            q = k.head_prepare(qkv, self.heads, self.kv_heads, self.dim, self.vdim, None, None, 0.0, table,
+            norms = (self.q_norm, self.k_norm, self.head_norm) if self.head_norm is not None else (None, None, 0.0)
+            q = k.head_prepare(qkv, self.heads, self.kv_heads, self.dim, self.vdim, *norms, table,
                                step.positions, held.pages, view.write_page, view.write_off, view.page_size,
                                bias=self.bias, values="keys" if self.values_from_keys else "own")
         sink = self.sink if self.has_sink else self.fixed_sink
         gates = qkv[:, self.qkv_width: self.qkv_width + self.heads] if self.has_gate else None
         out = attend(k, q, held, view, step, self.kv_heads, self.vdim, sink, self.scale,
-                     self.window, self.softcap, (self.r1, self.r2) if self.distance_bias else None, self.keep_first,
+                     self.sees, self.softcap, (self.r1, self.r2) if self.distance_bias else None, self.keep_first,
                      head_gate=gates)
         out = self.o(out)
         return k.add_bias(out, self.o_bias) if self.has_o_bias and add_row else out

@@ -47,6 +47,19 @@ def _widen_rows_hip(launch, x):
     return y
 
 
+def narrow_rows_plain(x32, dtype):
+    """x32 [T, W] float32 -> a new tensor of the values rounded to `dtype`."""
+    return x32.to(dtype, copy=True)
+
+
+def _narrow_rows_hip(launch, x32, dtype):
+    _need(x32.is_cuda and x32.is_contiguous() and x32.dtype == torch.float32 and dtype in _DT,
+          "narrow_rows: contiguous float32 rows on the GPU")
+    y = torch.empty(x32.shape, dtype=dtype, device=x32.device)
+    launch(x32.data_ptr(), y.data_ptr(), x32.numel(), _DT[dtype])
+    return y
+
+
 def stream_norm_plain(x32, terms, weight, eps, out_dtype):
     """x32 [T, W] float32 += sum of scale * term over `terms` [(tensor [T, W], scale)], in place, float32 arithmetic in
     the order given. Then, with `weight` [W]: returns (x - mean) / sqrt(var + eps) * weight of the rows, in
@@ -108,6 +121,7 @@ def _softcap_hip(launch, logits, cap):
 
 
 register_kernel(KernelOp("widen_rows", widen_rows_plain, "holon_widen_rows", [_P, _P, _L, _I], _widen_rows_hip))
+register_kernel(KernelOp("narrow_rows", narrow_rows_plain, "holon_narrow_rows", [_P, _P, _L, _I], _narrow_rows_hip))
 register_kernel(KernelOp("stream_norm", stream_norm_plain, "holon_stream_norm",
                          [_P, _P, _F, _I, _P, _F, _I, _P, _P, _L, _I, _F, _I], _stream_norm_hip))
 register_kernel(KernelOp("pair_rows", pair_rows_plain, "holon_pair_rows", [_P, _P, _P, _L, _I, _I, _I, _I],

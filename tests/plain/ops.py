@@ -199,8 +199,11 @@ class TorchKernels:
                 far = (pos - key).clamp(min=0).to(scores.dtype)
                 scores = scores - _up(dist[0])[:, None, None] * torch.log1p(_up(dist[1])[:, None, None] * far)
             hidden = key > pos
-            if window:
+            if window > 0:
                 hidden = hidden | ((pos - key >= window) & (key >= keep_first))
+            elif window < 0:                 # chunks of -window positions, counted from position 0
+                hidden = hidden | (torch.div(pos, -window, rounding_mode="floor")
+                                   != torch.div(key, -window, rounding_mode="floor"))
             scores = scores.masked_fill(hidden, float("-inf"))
             if sink is not None:             # a column of its own in the softmax, dropped again: it has no value
                 scores = torch.cat((scores, _up(sink)[:, None, None].expand(hq, e - s, 1)), dim=-1)
