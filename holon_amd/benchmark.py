@@ -26,7 +26,8 @@ feed-forward, vocabulary; random weights): a 2,048-token prompt and decode at ba
 sizes (`--sizes`), one line with both models' figures and the bytes a decode step must read. `--only` runs one model
 (for a profiler). --workload dopirax measures Dopirax the same way, beside Nevodra (the nearest design: both sublayers
 on one float32 stream, a capped attention, experts) and Qwen3 (`--beside`); --workload falisun measures Falisun beside
-Nevodra (latent attention, experts) and Qwen3.
+Nevodra (latent attention, experts) and Qwen3; --workload sopepel measures Sopepel beside Tolurax (windowed attention
+beside a decayed memory in one layer) and Qwen3.
 """
 from __future__ import annotations
 
@@ -217,9 +218,26 @@ def falisun_config(z: dict) -> dict:
             "layers": [layer(i) for i in range(z["layers"])]}
 
 
+def sopepel_config(z: dict, chunk: int = 1024) -> dict:
+    """A Sopepel model of a size's layers: attention with the size's heads inside chunks (half of a head turned) beside
+    gated linear attention with heads of 64 keys by 128 values over the same width, in pairs: over a dense feed-forward of
+    the size's width, and over eight experts of a quarter of it of which a token uses two, beside a gated shared one."""
+    quarter = z["ff"] // 4
+    mlps = ({"kind": "dense", "ff": z["ff"]},
+            {"kind": "moe", "expert": {"ff": quarter}, "shared": {"ff": quarter}, "router": {"experts": 8, "top": 2}})
+    mixer = {"left": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"],
+                      "mask": {"size": chunk}, "scale": z["dim"] ** -0.5, "rot": {"dims": z["dim"] // 2, "base": 1e6}},
+             "right": {"heads": z["width"] // 128, "dim": 64, "vdim": 128, "tau": 16.0, "rank": 16},
+             "left_scale": 1.0, "right_scale": 1.0}
+    return {"architecture": "Sopepel", "width": z["width"], "vocab": z["vocab"], "norm": {"eps": 1e-6}, "logit_scale": 1.0,
+            "embedding": {"bigram": {"buckets": 65521, "mul_prev": 31337, "mul_cur": 17}},
+            "layers": [{"type": "parallel", "mixer": mixer, "mlp": mlps[i % 2]} for i in range(z["layers"])]}
+
+
 DESIGN_CONFIGS = {"tolurax": tolurax_config, "relanex": relanex_config, "nevodra": nevodra_config,
-                  "dopirax": dopirax_config, "falisun": falisun_config}
-BESIDE = {"dopirax": "nevodra,qwen3", "falisun": "nevodra,qwen3"}      # what a design is measured beside (others: qwen3)
+                  "dopirax": dopirax_config, "falisun": falisun_config, "sopepel": sopepel_config}
+# what a design is measured beside (others: qwen3)
+BESIDE = {"dopirax": "nevodra,qwen3", "falisun": "nevodra,qwen3", "sopepel": "tolurax,qwen3"}
 
 
 def design_cache_bytes(name: str, cfg_json: dict, z: dict, item: int, batch: int, context: int) -> int:
@@ -235,7 +253,7 @@ def design_cache_bytes(name: str, cfg_json: dict, z: dict, item: int, batch: int
         elif name == "dopirax":                       # every layer reads all of a cache, its own or another layer's
             maps = 2 if layer["type"] == "attention_2" else 1     # differential layers keep the keys of both maps
             total += m["kv_heads"] * (maps * m["dim"] + m["vdim"]) * item * batch * context
-        elif layer["type"] == "parallel":             # the window's keys and values
+        elif layer["type"] == "parallel":             # the window's (or, near its end, the chunk's) keys and values
             total += 2 * z["kv_heads"] * z["dim"] * item * batch * min(context, m["left"]["mask"]["size"])
         elif layer["type"] == "attention":
             seen = min(context, m["mask"]["size"] + m["mask"].get("keep_first", 0)) if m.get("mask") else context
@@ -280,7 +298,8 @@ def design(a) -> int:
             item = 2 if a.dtype == "bfloat16" else 4
             weights = sum(getattr(o, n).numel() * getattr(o, n).element_size()
                           for path, o, n, _ in engine.model.named_params()
-                          if not path.startswith("embed.") or engine.model.lm_head.tied)     # (a tied head reads it all)
+                          if not path.startswith("embed.") or (path == "embed.weight" and engine.model.lm_head.tied))
+            # (a tied head reads the embedding's table; of other tables a step reads a row a token)
             # what a request keeps in its slot (the recurrences' matrices, the filters' inputs): read and written a step
             state = sum(t[0].numel() * t.element_size() for _, _, t in engine.cache.slot_states)
             times = []
@@ -350,7 +369,7 @@ def main(argv: list[str] | None = None) -> int:
                     help="--workload of a design: one model only")
     ap.add_argument("--beside", default=None,
                     help="--workload of a design: the models it is measured beside, with commas (default: qwen3; for "
-                         "dopirax and falisun: nevodra,qwen3)")
+                         "dopirax and falisun: nevodra,qwen3; sopepel: tolurax,qwen3)")
     ap.add_argument("--products", choices=("own", "vendor", "timed"), default="timed",
                     help="EngineConfig.products: which kernel products of 17 to 1,024 rows take (reported in the line)")
     a = ap.parse_args(argv)

@@ -83,8 +83,8 @@ class SopepelConfig:
         if (c.get("embedding") or {}).get("bigram"):
             buckets = _get(c, "embedding.bigram.buckets", int)
             muls = [c["embedding"]["bigram"].get(key) for key in ("mul_prev", "mul_cur")]
-            if any(not isinstance(v, int) or isinstance(v, bool) or not abs(v) < 1 << 31 for v in muls):
-                raise ConfigError("embedding.bigram.mul_prev and mul_cur must be whole numbers of 31 bits")
+            if any(not isinstance(v, int) or isinstance(v, bool) for v in muls):
+                raise ConfigError("embedding.bigram.mul_prev and mul_cur must be whole numbers")
             bigram = (buckets, *muls)
         layers = _get(c, "layers")
         if not isinstance(layers, list) or not layers:

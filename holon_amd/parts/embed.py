@@ -110,8 +110,8 @@ class BigramEmbedding(EmbedPart):
         super().__init__(build)
         if buckets < 1:
             raise ValueError(f"embed bigram: {buckets} buckets")
-        self.mul_prev, self.mul_cur = int(mul_prev), int(mul_cur)
-        self.declare("weight", (vocab, hidden))
+        self.mul_prev, self.mul_cur = int(mul_prev) % buckets, int(mul_cur) % buckets      # (the same rows, and no
+        self.declare("weight", (vocab, hidden))                                             # product beyond 64 bits)
         self.declare("bigram", (buckets + 1, hidden))
 
     def state(self):

@@ -25,7 +25,7 @@ SHORT = (("_Z18gemm_skinny_kernelILi", "gemm_skinny<"), ("_Z22gemm_skinny_glu_ke
          ("_Z23argmax_of_pieces_kernel", "argmax_of_pieces"), ("_Z16embedding_kernel", "embedding"),
          ("_Z15gemm_f32_kernel", "gemm_f32"), ("_Z13sample_kernel", "sample"),
          ("_ZN12_GLOBAL__N_116gemm_rows_kernelILi", "gemm_rows<"),
-         ("_Z19silu_mul_vec_kernel", "silu_mul_vec"), ("_ZN12_GLOBAL__N_118memory_scan_kernelILi", "memory_scan<"),
+         ("_Z20gated_mul_vec_kernelI", "gated_mul_vec<"), ("_Z16gated_mul_kernelI", "gated_mul<"), ("_ZN12_GLOBAL__N_118memory_scan_kernelILi", "memory_scan<"),
          ("_ZN12_GLOBAL__N_117delta_scan_kernelILi", "delta_scan<"), ("_ZN12_GLOBAL__N_118stream_norm_kernelILi", "stream_norm<"),
          ("_ZN12_GLOBAL__N_124sigmoid_attention_kernelI", "sigmoid_attention<"),
          ("_ZN12_GLOBAL__N_118causal_conv_kernelI", "causal_conv<"), ("_ZN12_GLOBAL__N_123causal_conv_keep_kernelI", "causal_conv_keep<"),
@@ -62,11 +62,11 @@ def dispatches(path: str) -> list[tuple]:
 CLASSES = (("attention", ("attn_", "sigmoid_attention", "softmax_attention", "latent_attention", "latent_prefill", "latent_decode",
                           "latent_merge")),
            ("matrix products", ("gemm_", "Cijk_", "Custom_Cijk_", "hipBLASLt", "head_linear")),
-           ("recurrent scans", ("memory_scan", "delta_scan", "memory_pieces", "delta_pieces", "mlstm_scan", "ssd_")),
-           ("elementwise", ("rmsnorm", "silu_mul", "qk_norm_rope", "v_write", "kv_write", "embedding", "sum_parts",
-                            "row_sumsq", "scatter_rows", "stream_norm", "dyt_stream", "widen_", "pair_rows", "softcap", "causal_conv",
+           ("recurrent scans", ("memory_scan", "delta_scan", "memory_pieces", "delta_pieces", "mlstm_scan", "ssd_", "gla_")),
+           ("elementwise", ("rmsnorm", "gated_mul", "qk_norm_rope", "v_write", "kv_write", "embedding", "sum_parts",
+                            "row_sumsq", "scatter_rows", "stream_norm", "dyt_stream", "widen_", "narrow_", "pair_rows", "softcap", "causal_conv",
                             "head_prepare", "delta_prepare", "gated_out", "shift_mix", "shift_keep", "decay_lora", "stream_rms", "latent_rope_prepare", "gated_parts_norm",
-                            "moe_gate", "moe_router")),
+                            "moe_gate", "moe_router", "moe_relu2", "relu2", "keep_last_token")),
            ("sampling", ("argmax", "sample_kernel", "store_tokens", "logprobs")))
 
 

@@ -58,12 +58,12 @@ CONFIG_A = model(64, 150, [
     layer(left(4, 1, 16, 8, 0.3, 7, 2, 10.0), right(1, 40, 33, 8.0, 16), moe(5, 1, 24)),
     layer(left(4, 2, 16, 12, 0.3, 10, 8, 100.0), right(3, 12, 20, 4.0, 6), dense(72))])
 # B: another order, eps and logit scale, wide multipliers, more experts of which more are chosen, all of a head turned,
-# rows of the table whose product passes 32 bits.
+# rows of the table whose product passes 64 bits.
 CONFIG_B = model(96, 200, [
     layer(left(3, 1, 32, 32, 0.2, 64, 32, 500000.0), right(6, 16, 32, 16.0, 16), dense(128), (0.5, 0.5)),
     layer(left(6, 6, 16, 16, 0.25, 20, 6, 1000.0), right(2, 64, 48, 16.0, 12), moe(7, 3, 24, shared=40), (2.0, 1.0)),
     layer(left(2, 2, 24, 40, 0.2, 33, 8, 20.0), right(5, 8, 24, 2.5, 4), moe(4, 4, 16, shared=8))],
-    eps=1e-5, logit_scale=1.6, bigram=(101, 1 << 29, 1000003))
+    eps=1e-5, logit_scale=1.6, bigram=(101, 1 << 61, 1000003))
 # C: sizes that are 1 or equal: one head, a chunk of one position (a query sees its own key alone) and of two, one turned
 # pair, values of one number, a rank of one, a tau, scales and a logit scale of 1, one expert, one bucket.
 CONFIG_C = model(32, 50, [
