@@ -457,10 +457,6 @@ __global__ void __launch_bounds__(256) attn_prefill_kernel(AttnArgs a) {
   }
 }
 
-// A barrier that waits for this wave's LDS traffic only. __syncthreads() also waits for every global load in flight
-// (vmcnt(0)), which would make each stage wait for the loads it has just requested for a later stage.
-__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
-
 // Prompt portions, staged through LDS: a block of four waves owns 4*NT consecutive tiles (for four heads a group: 32
 // positions with NT = 2) and walks the keys in stages of 32; each stage's keys and transposed values are copied from
 // the pages into LDS once per block (double buffered: the next stage's loads are in flight while this one is

@@ -95,6 +95,10 @@ __device__ __forceinline__ void wait_loads_but() {          // until at most N o
   __builtin_amdgcn_s_waitcnt((N & 15) | ((N >> 4) << 14) | (7 << 4) | (15 << 8));
 }
 
+// A barrier that waits for this wave's LDS traffic only. __syncthreads() also waits for every global load in flight
+// (vmcnt(0)), which would make each stage wait for the loads it has just requested for a later stage.
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
 // The first key that the query at position `pos` sees: window 0: key 0; w > 0: the last w keys (what is returned may lie
 // before key 0); w < 0: the query's own chunk of -w positions, chunks counted from position 0. It never falls as `pos`
 // grows, so the first query of a tile says where its keys begin and the last one from where all of its queries see them.

@@ -147,8 +147,6 @@ struct LatArgs {
   float scale_log2;
 };
 
-__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
-
 __device__ __forceinline__ bf16x4_t read_transposed(const unsigned char* p) {
   typedef __attribute__((address_space(3))) s16x4_t* lds_ptr;
   return __builtin_bit_cast(bf16x4_t, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)p));

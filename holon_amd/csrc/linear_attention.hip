@@ -81,17 +81,17 @@ template <int CTRL> __device__ __forceinline__ float dpp_add(float v) {
 // A block: one (row or piece, head) and 16 NW value columns, wave w columns 16 w .. 16 w + 15 of them, S's KD x 16 part of
 // a wave in its matrix-core accumulators. KD: the key size padded with zeros (a zero key writes nothing).
 template <int KD, int NW, int PASS, typename T>
-__global__ void __launch_bounds__(NW * WAVE) gla_scan_kernel(const T* __restrict__ q, const T* __restrict__ k,
+__global__ void __launch_bounds__(NW * WAVE, KD <= 64 ? 4 : 1) gla_scan_kernel(const T* __restrict__ q, const T* __restrict__ k,
                                                              const T* __restrict__ v, int64_t stride, float q_scale,
                                                              const float* __restrict__ alpha, float* __restrict__ state,
                                                              float* __restrict__ out, GlaRows r) {
   constexpr bool OUT = PASS == 2;
   constexpr int TB = 16, THREADS = NW * WAVE, N = TB * KD, PER = N / THREADS, DT = KD / 16, QP = KD + 4, TP = TB + 4;
-  constexpr int U = (KD + 16 * NW - 1) / (16 * NW);        // groups of four channels a lane scores
-  static_assert(N % THREADS == 0 && KD % 16 == 0, "whole tiles");
+  constexpr int VW = KD >= 16 * NW ? 4 : KD / (4 * NW), U = KD / (4 * VW * NW);      // scores: channels a lane takes at a time, times
+  static_assert(N % THREADS == 0 && KD == 4 * VW * NW * U, "whole tiles");
   __shared__ __attribute__((aligned(16))) float as_[N], ks_[N], qs_[OUT ? N : 4];
   __shared__ __attribute__((aligned(16))) float qp_[OUT ? TB * QP : 4], kt_[KD * TP], P_[KD];
-  __shared__ __attribute__((aligned(16))) float red_[OUT ? NW * TB * TB : 4], sc_[OUT ? TB * TP : 4];
+  __shared__ __attribute__((aligned(16))) float red_[OUT ? NW * TB * TB : 4];
   const int b = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE;
   const int g4 = lane / 16, c = lane % 16;
   const int col_blocks = (r.vdim + 16 * NW - 1) / (16 * NW);
@@ -126,115 +126,119 @@ __global__ void __launch_bounds__(NW * WAVE) gla_scan_kernel(const T* __restrict
     }
   float run = 1.f;                                         // PASS 1, thread d: the product of the piece's decays so far
   const int64_t width = (int64_t)r.heads * dim;
-  float nq[OUT ? PER : 1], nk[PER], na[PER], nv[4];
-  auto ask = [&](int t0) {                                 // the operands of a block of tokens, on their way to registers
+  // The operands of a block of tokens, on their way to registers as they lie in memory: places that do not exist are read
+  // from ones that do and made harmless when the values are used, so that nothing here waits for a load.
+  T nq[OUT ? PER : 1], nk[PER], nv[4];
+  float na[PER];
+  auto ask = [&](int t0) {
 #pragma unroll
     for (int e = 0; e < PER; ++e) {
-      const int idx = tid + e * THREADS, tt = idx / KD, d = idx % KD;
-      const bool ok = t0 + tt < hi && d < dim;
-      const int64_t at = (int64_t)(t0 + tt) * stride + (int64_t)h * dim + d;
-      nk[e] = ok ? Elem<T>::load(k[at]) : 0.f;
-      na[e] = ok ? alpha[(int64_t)(t0 + tt) * width + (int64_t)h * dim + d] : 1.f;
-      if constexpr (OUT) nq[e] = ok ? Elem<T>::load(q[at]) * q_scale : 0.f;
+      const int idx = tid + e * THREADS, t = min(t0 + idx / KD, hi - 1), d = min(idx % KD, dim - 1);
+      const int64_t at = (int64_t)t * stride + (int64_t)h * dim + d;
+      nk[e] = k[at];
+      na[e] = alpha[(int64_t)t * width + (int64_t)h * dim + d];
+      if constexpr (OUT) nq[e] = q[at];
     }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = t0 + 4 * g4 + i;
-      nv[i] = t < hi && col ? Elem<T>::load(v[(int64_t)t * stride + (int64_t)h * vdim + j]) : 0.f;
-    }
+    for (int i = 0; i < 4; ++i)
+      nv[i] = v[(int64_t)min(t0 + 4 * g4 + i, hi - 1) * stride + (int64_t)h * vdim + min(j, vdim - 1)];
   };
   if (lo < hi) ask(lo);
   for (int t0 = lo; t0 < hi; t0 += TB) {
 #pragma unroll
     for (int e = 0; e < PER; ++e) {
       const int idx = tid + e * THREADS;
-      as_[idx] = na[e];
-      ks_[idx] = nk[e];
-      if constexpr (OUT) qs_[idx] = nq[e];
+      const bool ok = t0 + idx / KD < hi && idx % KD < dim;
+      as_[idx] = ok ? na[e] : 1.f;
+      ks_[idx] = ok ? Elem<T>::load(nk[e]) : 0.f;
+      if constexpr (OUT) qs_[idx] = ok ? Elem<T>::load(nq[e]) * q_scale : 0.f;
     }
     float vv[4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) vv[i] = nv[i];
-    __syncthreads();
+    for (int i = 0; i < 4; ++i) vv[i] = t0 + 4 * g4 + i < hi && col ? Elem<T>::load(nv[i]) : 0.f;
+    lds_barrier();
     if (t0 + TB < hi) ask(t0 + TB);
-    for (int d = tid; d < KD; d += THREADS) {              // a channel a thread: its products over the block
-      float a[TB], s = 1.f;
+    // a channel a thread: k times the decays behind each token (and all of the block's); q times those up to it
+    for (int e = tid; e < (OUT ? 2 * KD : KD); e += THREADS) {
+      const int d = e % KD;
+      const float* src = e < KD ? ks_ : qs_;
+      float a[TB], x[TB];
 #pragma unroll
-      for (int t = 0; t < TB; ++t) a[t] = as_[t * KD + d];
-      float p = 1.f;
+      for (int t = 0; t < TB; ++t) { a[t] = as_[t * KD + d]; x[t] = src[t * KD + d]; }
+      if (e < KD) {
+        float s = 1.f;
+        f32x4 rows[TB / 4];
 #pragma unroll
-      for (int t = 0; t < TB; ++t) {
-        p *= a[t];
-        if constexpr (OUT) qp_[t * QP + d] = qs_[t * KD + d] * p;
-      }
-      P_[d] = p;
-      if constexpr (!OUT) run *= p;                        // (KD <= THREADS there: one channel a thread)
-#pragma unroll
-      for (int q4 = TB / 4 - 1; q4 >= 0; --q4) {
-        f32x4 row;
-#pragma unroll
-        for (int i = 3; i >= 0; --i) {
-          const int t = 4 * q4 + i;
-          row[i] = ks_[t * KD + d] * s;
+        for (int t = TB - 1; t >= 0; --t) {
+          rows[t / 4][t % 4] = x[t] * s;
           s *= a[t];
         }
-        *reinterpret_cast<f32x4*>(&kt_[d * TP + 4 * q4]) = row;
+#pragma unroll
+        for (int q4 = 0; q4 < TB / 4; ++q4) *reinterpret_cast<f32x4*>(&kt_[d * TP + 4 * q4]) = rows[q4];
+        P_[d] = s;
+        if constexpr (!OUT) run *= s;                      // (KD <= THREADS there: one channel a thread)
+      } else {
+        float p = 1.f;
+#pragma unroll
+        for (int t = 0; t < TB; ++t) {
+          p *= a[t];
+          qp_[t * QP + d] = x[t] * p;
+        }
       }
     }
     if constexpr (OUT) {                                   // the block's scores, every wave over its channels
-      const int jj = lane / 4, part = lane % 4;            // lane (jj, part): key jj, channels 4 (u NW + wave) 4 + 4 part ..
-      f32x4 kj[U], car[U];
+      typedef float fv __attribute__((ext_vector_type(VW)));
+      const int jj = lane / 4, part = lane % 4;            // lane (jj, part): key jj, channels ((u NW + wave) 4 + part) VW ..
+      fv kj[U], car[U];
 #pragma unroll
       for (int u = 0; u < U; ++u) {
-        const int d = ((u * NW + wave) * 4 + part) * 4;
-        car[u] = f32x4{0.f, 0.f, 0.f, 0.f};
-        kj[u] = car[u];
-        if (d < KD) kj[u] = *reinterpret_cast<const f32x4*>(&ks_[jj * KD + d]);
+        kj[u] = *reinterpret_cast<const fv*>(&ks_[jj * KD + ((u * NW + wave) * 4 + part) * VW]);
+        car[u] = (fv)0.f;
+      }
+      float dot[TB];
+#pragma unroll
+      for (int t = 0; t < TB; ++t) {
+        dot[t] = 0.f;
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+          const int d = ((u * NW + wave) * 4 + part) * VW;
+          const fv at = *reinterpret_cast<const fv*>(&as_[t * KD + d]);
+          const fv qt = *reinterpret_cast<const fv*>(&qs_[t * KD + d]);
+#pragma unroll
+          for (int i = 0; i < VW; ++i) {
+            car[u][i] = jj == t ? kj[u][i] : car[u][i] * at[i];        // (0 until the key's own token)
+            dot[t] += qt[i] * car[u][i];
+          }
+        }
       }
 #pragma unroll
       for (int t = 0; t < TB; ++t) {
-        float dot = 0.f;
-#pragma unroll
-        for (int u = 0; u < U; ++u) {
-          const int d = ((u * NW + wave) * 4 + part) * 4;
-          if (d < KD) {
-            const f32x4 at = *reinterpret_cast<const f32x4*>(&as_[t * KD + d]);
-            const f32x4 qt = *reinterpret_cast<const f32x4*>(&qs_[t * KD + d]);
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              car[u][i] = jj == t ? kj[u][i] : car[u][i] * at[i];      // (0 until the key's own token)
-              dot += qt[i] * car[u][i];
-            }
-          }
-        }
-        dot = dpp_add<0xB1>(dot);                          // quad_perm [1, 0, 3, 2]
-        dot = dpp_add<0x4E>(dot);                          // quad_perm [2, 3, 0, 1]
-        if (part == 0) red_[(wave * TB + t) * TB + jj] = dot;
+        dot[t] = dpp_add<0xB1>(dot[t]);                    // quad_perm [1, 0, 3, 2]
+        dot[t] = dpp_add<0x4E>(dot[t]);                    // quad_perm [2, 3, 0, 1]
       }
-      __syncthreads();
-      for (int e = tid; e < TB * TB; e += THREADS) {
-        float sum = red_[e];
+      if (part == 0) {
 #pragma unroll
-        for (int w = 1; w < NW; ++w) sum += red_[w * TB * TB + e];
-        sc_[(e / TB) * TP + e % TB] = sum;
+        for (int t = 0; t < TB; ++t) red_[(wave * TB + t) * TB + jj] = dot[t];
       }
     }
-    __syncthreads();
+    lds_barrier();
     if constexpr (OUT) {
-      f32x4 o = {0.f, 0.f, 0.f, 0.f};
+      f32x4 o[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
         const f32x4 qa = *reinterpret_cast<const f32x4*>(&qp_[c * QP + 16 * dt + 4 * g4]);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[i], S[dt][i], o, 0, 0, 0);
+        for (int i = 0; i < 4; ++i) o[i % 2] = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[i], S[dt][i], o[i % 2], 0, 0, 0);
       }
-      const f32x4 sa = *reinterpret_cast<const f32x4*>(&sc_[c * TP + 4 * g4]);
+      f32x4 sa = *reinterpret_cast<const f32x4*>(&red_[c * TB + 4 * g4]);      // the waves' scores, added up in order
 #pragma unroll
-      for (int i = 0; i < 4; ++i) o = __builtin_amdgcn_mfma_f32_16x16x4f32(sa[i], vv[i], o, 0, 0, 0);
+      for (int w = 1; w < NW; ++w) sa += *reinterpret_cast<const f32x4*>(&red_[(w * TB + c) * TB + 4 * g4]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) o[i % 2] = __builtin_amdgcn_mfma_f32_16x16x4f32(sa[i], vv[i], o[i % 2], 0, 0, 0);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int t = t0 + 4 * g4 + i;
-        if (t < hi && col) out[((int64_t)t * r.heads + h) * vdim + j] = o[i];
+        if (t < hi && col) out[((int64_t)t * r.heads + h) * vdim + j] = o[0][i] + o[1][i];
       }
     }
     if (!OUT || t0 + TB < hi || to_slot) {
@@ -247,7 +251,8 @@ __global__ void __launch_bounds__(NW * WAVE) gla_scan_kernel(const T* __restrict
         for (int i = 0; i < 4; ++i) S[dt] = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[i], vv[i], S[dt], 0, 0, 0);
       }
     }
-    __syncthreads();                                       // the next block's operands take these places
+    // (no barrier: the next block's operands go where only the part before the last barrier read, and what this part reads
+    // is written again behind the next one)
   }
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
