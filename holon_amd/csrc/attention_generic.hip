@@ -47,7 +47,7 @@ __global__ void attention_generic_kernel(const T* __restrict__ q, T* __restrict_
   for (int d = lane; d < head_dim; d += WAVE) q_s[w][d] = Elem<T>::load(qp[d]);
   __syncthreads();
 
-  const int first = window > 0 ? max(0, pos - window + 1) : 0;
+  const int first = max(0, first_seen(pos, window));
   float m = -INFINITY, l = 0.f;
   Acc acc[GEN_MAX_D / WAVE];
 #pragma unroll
@@ -111,7 +111,7 @@ extern "C" int holon_attention_generic(const void* q, void* out, const void* pag
               "attention: bad head counts %d/%d", heads, kv_heads);
   HOLON_CHECK(head_dim > 0 && head_dim % 8 == 0 && head_dim <= GEN_MAX_D,
               "attention: head_dim %d must be a multiple of 8, at most %d", head_dim, GEN_MAX_D);
-  HOLON_CHECK(page_size > 0 && num_pages > 0 && window >= 0, "attention: bad page size or window");
+  HOLON_CHECK(page_size > 0 && num_pages > 0 && window > -0x7fffffff, "attention: bad page size or window");
   if (tokens == 0 || rows == 0) return 0;
   dim3 grid(tokens, (heads + 3) / 4);
   hipStream_t s = (hipStream_t)stream;

@@ -144,7 +144,8 @@ class Kernels(Protocol):
                         keep_first: int = 0, value_share: int = 1, head_gate: torch.Tensor | None = None
                         ) -> torch.Tensor:
         """softmax(q k^T * scale) v per row over its cached tokens, causal; with window W > 0 a query at position p
-        sees keys p-W+1 .. p. q [T, Hq, D] -> [T, Hq, D]. This step's keys are already in the cache. `sink` [Hq]
+        sees keys p-W+1 .. p, with -W < 0 the keys of its own chunk of W positions (from p - p mod W). q [T, Hq, D] ->
+        [T, Hq, D]. This step's keys are already in the cache. `sink` [Hq]
         float32: exp(sink[h] - max) is added to the softmax's denominator (it has no key and no value). Where
         `attention_on_cores` says so it also takes changed scores: `softcap` > 0: s <- softcap tanh(s / softcap);
         `dist` = (r1 [Hq], r2 [Hq]) float32: s <- s - r1 ln(1 + r2 (p - j)) for the key at position j; `keep_first`:

@@ -718,6 +718,8 @@ def test_chunks_in_the_attention_kernels(dim):
                     general = k.softmax_attention(q.to(dtype), flat.to(dtype), table, rows, token_row, positions, groups, dim,
                                                   page, None, scale, -chunk)
                     assert H.rel_rms(general.view(-1, heads, dim), want) < tol, (dim, heads, groups, chunk, dtype)
+                plain_form = k.paged_attention(q.float(), pages.float(), table, rows, page, scale, -chunk)   # off the cores
+                assert H.rel_rms(plain_form, want) < 2e-6, (dim, heads, groups, chunk)
     # decode rows alone, in order, of every length around a chunk's edges
     lens = [179, 180, 181, 359, 360, 361, 1, 33, 640]
     table, n_pages = _scattered(lens, page, 48, g)
